@@ -93,7 +93,8 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
     int64_t q_stride, bf16_t* __restrict__ k_cache, bf16_t* __restrict__ v_cache,
     const int32_t* __restrict__ block_table, int max_blocks, const int32_t* __restrict__ req_of_token,
     const int32_t* __restrict__ positions, const int32_t* __restrict__ rows, int heads, int kv_heads,
-    int bs_shift, int window, float scale, RopeArgs rope, int* __restrict__ counters, int v_head, float* __restrict__ out32, int value_heads, int64_t plane) {
+    int bs_shift, int window, float scale, RopeArgs rope, int* __restrict__ counters, int v_head, float* __restrict__ out32, int value_heads, int64_t plane,
+    const float* __restrict__ sink) {
   static_assert(!kRope || DT % 4 == 0, "the rotation needs a channel and its partner in the same lane: d a multiple of 64");
   constexpr int d = DT * 16;
   constexpr int DS = (d + 31) / 32;            // steps of 32 along d in the first product
@@ -391,7 +392,10 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
     float big = state[0][i][0];
 #pragma unroll
     for (int w = 1; w < NW; ++w) big = fmaxf(big, state[w][i][0]);
-    float total = 0.f, acc = 0.f;
+    const bool sinks = sink && n_parts == 1;      // (the sink joins the sum once, where the head's parts meet)
+    const float s2 = sinks ? sink[h] * 1.44269504088896340736f : -FLT_MAX;
+    big = fmaxf(big, s2);
+    float total = sinks ? __builtin_amdgcn_exp2f(s2 - big) : 0.f, acc = 0.f;
 #pragma unroll
     for (int w = 0; w < NW; ++w) {
       const float e = __builtin_amdgcn_exp2f(state[w][i][0] - big);
@@ -436,7 +440,8 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
     if (h0 + i >= group) break;
     const int h = hk * group + h0 + i;
     const float* src = partial + (static_cast<int64_t>(blockIdx.x) * heads + h) * n_parts * (d + 2);
-    float big = -FLT_MAX, total = 0.f, acc = 0.f;
+    const float s2 = sink ? sink[h] * 1.44269504088896340736f : -FLT_MAX;
+    float big = s2, total = 0.f, acc = 0.f;
     if (n_parts <= 16) {
       // up to sixteen parts: everything that is read is asked for at once (the states come from memory; one after
       // the other, every load is waited for by itself), in arrays of four, eight or sixteen; same sums in the same
@@ -475,6 +480,7 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
         acc += __hip_atomic_load(part + 2 + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) * e;
       }
     }
+    if (sink) total += __builtin_amdgcn_exp2f(s2 - big);
     put_out(out, out32, static_cast<int64_t>(t) * out_stride + static_cast<int64_t>(h) * d + c, acc / total);
   }
 }
@@ -487,7 +493,8 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
 __global__ void __launch_bounds__(256) attention_merge_kernel(bf16_t* __restrict__ out, int64_t out_stride,
                                                               const float* __restrict__ partial,
                                                               const int32_t* __restrict__ rows, int heads, int d,
-                                                              int n_splits, float* __restrict__ out32, int value_heads, int64_t plane) {
+                                                              int n_splits, float* __restrict__ out32, int value_heads, int64_t plane,
+                                                              const float* __restrict__ sink) {
   __shared__ float sums[4][256];
   const int served = value_heads > 0 ? blockIdx.x / value_heads : blockIdx.x;
   if (value_heads > 0) out32 += static_cast<int64_t>(blockIdx.x % value_heads) * plane;
@@ -497,9 +504,10 @@ __global__ void __launch_bounds__(256) attention_merge_kernel(bf16_t* __restrict
   // lane s holds part s's maximum and sum (n_splits <= 64)
   const float m = lane < n_splits ? src[lane * (d + 2)] : -FLT_MAX;
   const float l = lane < n_splits ? src[lane * (d + 2) + 1] : 0.f;
-  const float big = wave_max(m);
+  const float s2 = sink ? sink[h] * 1.44269504088896340736f : -FLT_MAX;
+  const float big = fmaxf(wave_max(m), s2);
   const float e = __builtin_amdgcn_exp2f(m - big);
-  const float total = wave_sum(l * e);
+  const float total = wave_sum(l * e) + (sink ? __builtin_amdgcn_exp2f(s2 - big) : 0.f);
   // every lane takes part in every round, so that the weights can be read from all 64 lanes
   for (int c0 = 0; c0 < d; c0 += 64) {
     const int c = c0 + lane;
@@ -557,12 +565,13 @@ extern "C" int alofa_attention_decode_can_hand_over(int tokens, int heads, int k
 // workspace (alofa_attention_decode_can_hand_over must hold; `partial` is not used), not in `partial` and a second kernel.
 // v_head >= 0: every query head's weights meet the values of that one value head (its keys stay its own key head's);
 // out32: the results go there unrounded, as float rows of `out`'s shape and stride, and `out` is not written.
+// sink: a number per query head whose exponential joins the sum of its rows' weights (null: none).
 extern "C" int alofa_attention_decode_v(void* out, int64_t out_stride, float* partial, const void* q, int64_t q_stride,
                                         void* k_cache, void* v_cache, const int32_t* block_table,
                                         int max_blocks, const int32_t* req_of_token, const int32_t* positions,
                                         const int32_t* rows, int tokens, int heads, int kv_heads, int d, int block_size, int window,
                                         float scale, int n_splits, const float* cos_t, const float* sin_t, const int64_t* slots,
-                                        int hand_over, int v_head, float* out32, int split, int value_heads, int64_t plane, hipStream_t stream) {
+                                        int hand_over, int v_head, float* out32, int split, int value_heads, int64_t plane, const float* sink, hipStream_t stream) {
   ALOFA_REQUIRE(!split || !cos_t, "attention_decode: split weights and the rotary variant do not go together");
   // value_heads > 0: all of them in one launch, value head c's results in out32 + c * plane; `tokens` then counts (token, value head) pairs
   // wherever it sizes scratch, workspace and grid
@@ -597,11 +606,11 @@ extern "C" int alofa_attention_decode_v(void* out, int64_t out_stride, float* pa
   if (split && !ROPE) attention_decode_kernel<DT, NW, false, true><<<grid, 64 * NW, 0, stream>>>(                         \
       static_cast<bf16_t*>(out), out_stride, partial, static_cast<const bf16_t*>(q), q_stride,                            \
       static_cast<bf16_t*>(k_cache), static_cast<bf16_t*>(v_cache), block_table, max_blocks, req_of_token,                \
-      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane);       \
+      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane, sink);       \
   else attention_decode_kernel<DT, NW, ROPE><<<grid, 64 * NW, 0, stream>>>(                                                    \
       static_cast<bf16_t*>(out), out_stride, partial, static_cast<const bf16_t*>(q), q_stride,                            \
       static_cast<bf16_t*>(k_cache), static_cast<bf16_t*>(v_cache), block_table, max_blocks, req_of_token,                \
-      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane)
+      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane, sink)
   if (fused) {
     switch (d / 64) {
       case 1: ALOFA_DECODE(4, 8, true); break;
@@ -633,7 +642,7 @@ extern "C" int alofa_attention_decode_v(void* out, int64_t out_stride, float* pa
   if (check_launch("attention_decode")) return 1;
   if (n_splits > 1 && !counters) {
     // (one wave up to sixteen parts, whose loads are all on their way at once; four beyond)
-    attention_merge_kernel<<<dim3(tokens, heads), n_splits <= 16 ? 64 : 256, 0, stream>>>(static_cast<bf16_t*>(out), out_stride, partial, rows, heads, d, n_splits, out32, value_heads, plane);
+    attention_merge_kernel<<<dim3(tokens, heads), n_splits <= 16 ? 64 : 256, 0, stream>>>(static_cast<bf16_t*>(out), out_stride, partial, rows, heads, d, n_splits, out32, value_heads, plane, sink);
     return check_launch("attention_merge");
   }
   return 0;
@@ -646,5 +655,5 @@ extern "C" int alofa_attention_decode(void* out, int64_t out_stride, float* part
                                       float scale, int n_splits, const float* cos_t, const float* sin_t, const int64_t* slots,
                                       int hand_over, hipStream_t stream) {
   return alofa_attention_decode_v(out, out_stride, partial, q, q_stride, k_cache, v_cache, block_table, max_blocks, req_of_token, positions, rows, tokens,
-                                  heads, kv_heads, d, block_size, window, scale, n_splits, cos_t, sin_t, slots, hand_over, -1, nullptr, 0, 0, 0, stream);
+                                  heads, kv_heads, d, block_size, window, scale, n_splits, cos_t, sin_t, slots, hand_over, -1, nullptr, 0, 0, 0, nullptr, stream);
 }

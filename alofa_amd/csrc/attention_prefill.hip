@@ -67,7 +67,7 @@ __global__ void __launch_bounds__(64 * WPT * TEAMS, (RW == 32 && 64 * WPT * TEAM
     bf16_t* __restrict__ out, int64_t out_stride, const bf16_t* __restrict__ q, int64_t q_stride,
     const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache, const int32_t* __restrict__ block_table,
     int max_blocks, const int32_t* __restrict__ tiles, int heads, int kv_heads, int bs_shift, int window,
-    float scale, int v_head, float* __restrict__ out32, int value_heads, int64_t plane) {
+    float scale, int v_head, float* __restrict__ out32, int value_heads, int64_t plane, const float* __restrict__ sink) {
   constexpr int d = DT * 16;
   constexpr int BKV = KT;
   static_assert(KT == 64 || (KT == 32 && RW == 32), "tiles of 64 keys, or of 32 with 32 rows a wave");
@@ -403,6 +403,7 @@ __global__ void __launch_bounds__(64 * WPT * TEAMS, (RW == 32 && 64 * WPT * TEAM
   }
 
   l = RW == 32 ? halves_sum(l) : rows_sum(l);
+  float top = m;      // what l and o are relative to
   if (TEAMS > 1) {
     // the other teams leave their states where their tiles were; team 0 adds them in team order
     __syncthreads();      // every tile has been read
@@ -421,6 +422,7 @@ __global__ void __launch_bounds__(64 * WPT * TEAMS, (RW == 32 && 64 * WPT * TEAM
 #pragma unroll
       for (int k = 1; k < TEAMS; ++k) big = fmaxf(big, state[k * (kTeamBytes / 4)]);
       const float e0 = __builtin_amdgcn_exp2f(m - big);
+      top = big;
       l *= e0;
 #pragma unroll
       for (int nt = 0; nt < OT; ++nt) o[nt] *= e0;
@@ -441,7 +443,12 @@ __global__ void __launch_bounds__(64 * WPT * TEAMS, (RW == 32 && 64 * WPT * TEAM
     }
   }
   if (row_ok && team == 0) {
-    const float inv = 1.f / l;
+    float inv = 1.f / l;
+    if (sink) {      // a number per head whose exponential joins the row's sum (no key, no value, not scaled)
+      const float s2 = sink[head] * 1.44269504088896340736f, most = fmaxf(top, s2);
+      const float shrink = __builtin_amdgcn_exp2f(top - most);
+      inv = shrink / (l * shrink + __builtin_amdgcn_exp2f(s2 - most));
+    }
     const int64_t at = static_cast<int64_t>(row0 + my_row) * out_stride + static_cast<int64_t>(head) * d;
     bf16_t* dst = out + at;
 #pragma unroll
@@ -519,16 +526,16 @@ extern "C" int alofa_attention_prefill_supports(int d) {
 
 // v_head >= 0: every query head's weights meet the values of that one value head (its keys stay its own key head's);
 // out32: the results go there unrounded, as float rows of `out`'s shape and stride (16-byte aligned), and `out` is not written.
-// split: the weights enter the second product with sixteen bits each (see kSplit).
+// split: the weights enter the second product with sixteen bits each (see kSplit). sink: a number per query head whose exponential joins the sum of its rows' weights (null: none).
 extern "C" int alofa_attention_prefill_v(void* out, int64_t out_stride, const void* q, int64_t q_stride,
                                          const void* k_cache, const void* v_cache, const int32_t* block_table,
                                          int max_blocks, const int32_t* tiles, int n_tiles, int heads, int kv_heads, int d,
                                          int block_size, int window, float scale, int share, int rows_per_wave, int v_head, float* out32, int split,
-                                         int value_heads, int64_t plane, hipStream_t stream) {
+                                         int value_heads, int64_t plane, const float* sink, hipStream_t stream) {
   // value_heads > 0: all of them in one launch, value head c's results in out32 + c * plane
   ALOFA_REQUIRE(value_heads == 0 || (value_heads == kv_heads && out32 && v_head < 0 && plane > 0 && plane % 4 == 0), "attention_prefill: all %d value heads in one launch need float rows and no value head named", kv_heads);
   if (value_heads > 0) n_tiles *= value_heads;      // (the grid's first dimension)
-  ALOFA_REQUIRE(!split || (share == 0 && rows_per_wave == 16), "attention_prefill: split weights run with 16 rows a wave and no shared tiles (share=%d rows=%d)", share, rows_per_wave);
+  ALOFA_REQUIRE(!split || rows_per_wave == 16, "attention_prefill: split weights run with 16 rows a wave (rows=%d)", rows_per_wave);
   ALOFA_REQUIRE(v_head < kv_heads && reinterpret_cast<uintptr_t>(out32) % 16 == 0, "attention_prefill: value head %d of %d; float rows 16-byte aligned", v_head, kv_heads);
   ALOFA_REQUIRE(n_tiles > 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0,
                 "attention_prefill: tiles=%d heads=%d kv_heads=%d (kv_heads must divide heads)", n_tiles, heads, kv_heads);
@@ -550,11 +557,30 @@ extern "C" int alofa_attention_prefill_v(void* out, int64_t out_stride, const vo
 #define ALOFA_PREFILL_AS(DT, TEAMS, WPT, SHARE, GRID)                                                                         \
   attention_prefill_kernel<DT, TEAMS, WPT, SHARE><<<GRID, 64 * WPT * TEAMS, 0, stream>>>(                                    \
       static_cast<bf16_t*>(out), out_stride, static_cast<const bf16_t*>(q), q_stride, static_cast<const bf16_t*>(k_cache), \
-      static_cast<const bf16_t*>(v_cache), block_table, max_blocks, tiles, heads, kv_heads, bs_shift, window, scale, v_head, out32, value_heads, plane)
+      static_cast<const bf16_t*>(v_cache), block_table, max_blocks, tiles, heads, kv_heads, bs_shift, window, scale, v_head, out32, value_heads, plane, sink)
 #define ALOFA_PREFILL_SPLIT(DT)                                                                                               \
   attention_prefill_kernel<DT, kTeams<DT>, 4, false, 16, 64, true><<<dim3(n_tiles, heads), 64 * 4 * kTeams<DT>, 0, stream>>>(  \
       static_cast<bf16_t*>(out), out_stride, static_cast<const bf16_t*>(q), q_stride, static_cast<const bf16_t*>(k_cache), \
-      static_cast<const bf16_t*>(v_cache), block_table, max_blocks, tiles, heads, kv_heads, bs_shift, window, scale, v_head, out32, value_heads, plane)
+      static_cast<const bf16_t*>(v_cache), block_table, max_blocks, tiles, heads, kv_heads, bs_shift, window, scale, v_head, out32, value_heads, plane, sink)
+#define ALOFA_PREFILL_SPLIT_AS(DT, WPT)                                                                                       \
+  attention_prefill_kernel<DT, kShareTeams<DT>, WPT, true, 16, 64, true><<<dim3(n_tiles, kv_heads * chunks, 4), 64 * WPT * kShareTeams<DT>, 0, stream>>>(  \
+      static_cast<bf16_t*>(out), out_stride, static_cast<const bf16_t*>(q), q_stride, static_cast<const bf16_t*>(k_cache), \
+      static_cast<const bf16_t*>(v_cache), block_table, max_blocks, tiles, heads, kv_heads, bs_shift, window, scale, v_head, out32, value_heads, plane, sink)
+#define ALOFA_PREFILL_SPLIT_WIDE(DT)                                                                                          \
+  if (width == 8) ALOFA_PREFILL_SPLIT_AS(DT, 8); else if (width == 7) ALOFA_PREFILL_SPLIT_AS(DT, 7); else ALOFA_PREFILL_SPLIT_AS(DT, 6)
+  if (split && width) {
+    switch (d / 16) {
+      case 1: ALOFA_PREFILL_SPLIT_WIDE(1); break;
+      case 2: ALOFA_PREFILL_SPLIT_WIDE(2); break;
+      case 3: ALOFA_PREFILL_SPLIT_WIDE(3); break;
+      case 4: ALOFA_PREFILL_SPLIT_WIDE(4); break;
+      case 6: ALOFA_PREFILL_SPLIT_WIDE(6); break;
+      case 8: ALOFA_PREFILL_SPLIT_WIDE(8); break;
+    }
+    return check_launch("attention_prefill");
+  }
+#undef ALOFA_PREFILL_SPLIT_WIDE
+#undef ALOFA_PREFILL_SPLIT_AS
   if (split) {
     switch (d / 16) {
       case 1: ALOFA_PREFILL_SPLIT(1); break;
@@ -571,7 +597,7 @@ extern "C" int alofa_attention_prefill_v(void* out, int64_t out_stride, const vo
 #define ALOFA_PREFILL_AS32(DT, TEAMS, WPT, SHARE, GRID)                                                                       \
   attention_prefill_kernel<DT, TEAMS, WPT, SHARE, 32, (DT > 6 ? 32 : 64)><<<GRID, 64 * WPT * TEAMS, 0, stream>>>(            \
       static_cast<bf16_t*>(out), out_stride, static_cast<const bf16_t*>(q), q_stride, static_cast<const bf16_t*>(k_cache), \
-      static_cast<const bf16_t*>(v_cache), block_table, max_blocks, tiles, heads, kv_heads, bs_shift, window, scale, v_head, out32, value_heads, plane)
+      static_cast<const bf16_t*>(v_cache), block_table, max_blocks, tiles, heads, kv_heads, bs_shift, window, scale, v_head, out32, value_heads, plane, sink)
 #define ALOFA_PREFILL_WIDE32(DT, WPT)                                                                            \
   if (width == WPT) ALOFA_PREFILL_AS32(DT, (kShareTeams<DT>), WPT, true, dim3(n_tiles, kv_heads * chunks, 2))
 #define ALOFA_PREFILL32(DT)                                                                         \
@@ -613,5 +639,5 @@ extern "C" int alofa_attention_prefill(void* out, int64_t out_stride, const void
                                        int max_blocks, const int32_t* tiles, int n_tiles, int heads, int kv_heads, int d,
                                        int block_size, int window, float scale, int share, int rows_per_wave, hipStream_t stream) {
   return alofa_attention_prefill_v(out, out_stride, q, q_stride, k_cache, v_cache, block_table, max_blocks, tiles, n_tiles, heads, kv_heads, d, block_size, window,
-                                   scale, share, rows_per_wave, -1, nullptr, 0, 0, 0, stream);
+                                   scale, share, rows_per_wave, -1, nullptr, 0, 0, 0, nullptr, stream);
 }

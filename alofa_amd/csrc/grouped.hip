@@ -20,7 +20,7 @@ namespace alofa {
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
-enum GroupedEpilogue : int { kGrStore = 0, kGrSigmoidGate = 1, kGrClampedGlu = 2 };
+enum GroupedEpilogue : int { kGrStore = 0, kGrSigmoidGate = 1, kGrClampedGlu = 2, kGrReluSquared = 3, kGrTurn = 4 };
 
 struct GroupedShape {
   int64_t out_stride, out_batch_step;   // out[row, batch * out_batch_step + o]
@@ -33,7 +33,20 @@ struct GroupedShape {
   int tiles, tiles_per_batch;           // tiles in all; dense: row tiles of a batch (0: listed)
   int64_t gate_stride;                  // kGrSigmoidGate: gate[row, batch * out_batch_step + o]
   float limit, limit_last, slope, offset;       // kGrClampedGlu: a sigmoid(slope a) (b + offset)
+  const int32_t* positions;             // kGrTurn: outputs 2 i and 2 i + 1 of every batch, i < turn_pairs, are turned by the angle of (the row's position, i)
+  const float* cos_t;
+  const float* sin_t;
+  int turn_pairs;
 };
+
+// Output o of a row whose pair (o & ~1, o | 1) has the values (a, b) before the turn.
+__device__ __forceinline__ float turned(const GroupedShape& s, int row, int o, float a, float b) {
+  const bool second = o & 1;
+  if (o >= 2 * s.turn_pairs) return second ? b : a;
+  const int64_t at = static_cast<int64_t>(s.positions[row]) * s.turn_pairs + (o >> 1);
+  const float cs = s.cos_t[at], sn = s.sin_t[at];
+  return second ? b * cs + a * sn : a * cs - b * sn;
+}
 
 // Every lane issues every load (from the operand's first bytes where its own are not wanted) and what is not wanted is cleared
 // afterwards: loads under a branch are waited for one by one, loads without one are in flight together.
@@ -166,10 +179,8 @@ __global__ void __launch_bounds__(256) grouped_product_kernel(TO* __restrict__ o
     const int out_row = s.tiles_per_batch > 0 ? row[t] : slot;
     TO* dst = out + static_cast<int64_t>(out_row) * s.out_stride + batch * s.out_batch_step;
     float weight = 1.f, lim = 0.f;
-    if constexpr (kGlu) {
-      weight = slot_weight ? slot_weight[slot] : 1.f;
-      lim = last ? s.limit_last : s.limit;
-    }
+    if constexpr (kGlu || kEpilogue == kGrReluSquared) weight = slot_weight ? slot_weight[slot] : 1.f;
+    if constexpr (kGlu) lim = last ? s.limit_last : s.limit;
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
 #pragma unroll
@@ -184,6 +195,11 @@ __global__ void __launch_bounds__(256) grouped_product_kernel(TO* __restrict__ o
           const float a = fminf(y, lim);
           const float b = fminf(fmaxf(acc2[t][c][i], -lim), lim);
           y = weight * (a * (1.f / (1.f + __expf(-s.slope * a))) * (b + s.offset));
+        } else if constexpr (kEpilogue == kGrReluSquared) {
+          const float a = fmaxf(y, 0.f);
+          y = weight * (a * a);
+        } else if constexpr (kEpilogue == kGrTurn) {
+          y = turned(s, out_row, o, acc[t][c][i & ~1], acc[t][c][i | 1]);
         }
         store_f32(dst + o, y);
       }
@@ -295,10 +311,8 @@ __global__ void __launch_bounds__(256) grouped_tiled_kernel(TO* __restrict__ out
     const int out_row = s.tiles_per_batch > 0 ? row : slot;
     TO* dst = out + static_cast<int64_t>(out_row) * s.out_stride + batch * s.out_batch_step;
     float weight = 1.f, lim = 0.f;
-    if constexpr (kGlu) {
-      weight = slot_weight ? slot_weight[slot] : 1.f;
-      lim = last ? s.limit_last : s.limit;
-    }
+    if constexpr (kGlu || kEpilogue == kGrReluSquared) weight = slot_weight ? slot_weight[slot] : 1.f;
+    if constexpr (kGlu) lim = last ? s.limit_last : s.limit;
 #pragma unroll
     for (int c = 0; c < (kGlu ? 2 : 4); ++c) {
 #pragma unroll
@@ -313,6 +327,11 @@ __global__ void __launch_bounds__(256) grouped_tiled_kernel(TO* __restrict__ out
           const float a = fminf(y, lim);
           const float b = fminf(fmaxf(acc[t][c + 2][i], -lim), lim);
           y = weight * (a * (1.f / (1.f + __expf(-s.slope * a))) * (b + s.offset));
+        } else if constexpr (kEpilogue == kGrReluSquared) {
+          const float a = fmaxf(y, 0.f);
+          y = weight * (a * a);
+        } else if constexpr (kEpilogue == kGrTurn) {
+          y = turned(s, out_row, o, acc[t][c][i & ~1], acc[t][c][i | 1]);
         }
         store_f32(dst + o, y);
       }
@@ -324,13 +343,13 @@ __global__ void __launch_bounds__(256) grouped_tiled_kernel(TO* __restrict__ out
 // chosen, weights [T, top]: the experts a row takes and its weights. Slots: every expert's rows together, an
 // expert's share padded to a multiple of `pad` (a tile's rows: 16 or 64), in expert order; then (with `shared`) all T rows once more for the
 // expert every row takes, as batch E. Outputs: row_in[slot] (the row, or -1), slot_weight[slot], slot_of[t * top + k]
-// (where row t's k-th choice went) and slot_of[T * top + t] (its slot of the shared expert), tile_batch[tile] (the
+// (where row t's k-th choice went) and slot_of[T * top + t] (its slot of the shared expert, whose weight is shared_weight[t], or 1 without), tile_batch[tile] (the
 // expert of a tile of `pad` slots, -1 beyond the last). Which slot of its expert's share a row gets depends on the
 // order in which threads arrive, which changes no result: a slot's values depend on its row alone.
 // One block; experts up to 512.
 __global__ void __launch_bounds__(1024) expert_rows_kernel(const int32_t* __restrict__ chosen, const float* __restrict__ weights, int32_t* __restrict__ row_in,
                                                            float* __restrict__ slot_weight, int32_t* __restrict__ slot_of, int32_t* __restrict__ tile_batch,
-                                                           int T, int top, int experts, int shared, int slots, int tiles, int pad) {
+                                                           const float* __restrict__ shared_weight, int T, int top, int experts, int shared, int slots, int tiles, int pad) {
   __shared__ int count[512], first[513], cursor[512];
   for (int e = threadIdx.x; e < experts; e += 1024) count[e] = cursor[e] = 0;
   for (int i = threadIdx.x; i < slots; i += 1024) {
@@ -369,7 +388,7 @@ __global__ void __launch_bounds__(1024) expert_rows_kernel(const int32_t* __rest
     const int base = first[experts];
     for (int t = threadIdx.x; t < T; t += 1024) {
       row_in[base + t] = t;
-      slot_weight[base + t] = 1.f;
+      slot_weight[base + t] = shared_weight ? shared_weight[t] : 1.f;
       slot_of[pairs + t] = base + t;
     }
     for (int t = threadIdx.x; t < (T + pad - 1) / pad; t += 1024) tile_batch[base / pad + t] = experts;
@@ -392,6 +411,66 @@ __global__ void __launch_bounds__(256) experts_sum_kernel(float* __restrict__ re
   if (pass_weight) sum += pass_weight[t] * bf16_to_f32(pass_x[static_cast<int64_t>(t) * pass_stride + c]);      // (the row itself, handed on with a weight)
   if (scale) sum *= scale[c];
   residual[idx] = assign ? sum : residual[idx] + sum;
+}
+
+// ---- residual[t, :] += rmsnorm(sum of row t's slots) * w, rows[t, :] = the stream's new row in the activation type: the sum above with the
+// norm behind the mixture and the sum into the stream (a block per row; the sums wait in registers, or, in rows wider than a block keeps,
+// in `wide` [T, width]) ----
+template <typename TO>
+__global__ void __launch_bounds__(256) experts_sum_norm_kernel(float* __restrict__ residual, const float* __restrict__ y, const int32_t* __restrict__ slot_of,
+                                                               const float* __restrict__ w, float eps, TO* __restrict__ rows, float* __restrict__ wide, int T, int width,
+                                                               int top, int shared) {
+  __shared__ float scratch[4];
+  constexpr int kOwn = 16;      // values a thread keeps: rows up to 4,096 wide
+  const int t = blockIdx.x;
+  const int64_t at = static_cast<int64_t>(t) * width;
+  float own[kOwn];
+#pragma unroll
+  for (int i = 0; i < kOwn; ++i) own[i] = 0.f;
+  float ss = 0.f;
+  const int parts = top + (shared ? 1 : 0);
+  if (width <= kOwn * 256) {      // (uniform over the launch)
+    for (int k = 0; k < parts; ++k) {
+      const int slot = k < top ? slot_of[t * top + k] : slot_of[T * top + t];
+      if (slot < 0) continue;      // (a choice without a slot)
+      const float* src = y + static_cast<int64_t>(slot) * width;
+#pragma unroll
+      for (int i = 0; i < kOwn; ++i) {
+        const int c = threadIdx.x + i * 256;
+        if (c < width) own[i] += src[c];
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < kOwn; ++i) ss += own[i] * own[i];
+  } else {
+    for (int c = threadIdx.x; c < width; c += 256) {
+      float sum = 0.f;
+      for (int k = 0; k < parts; ++k) {
+        const int slot = k < top ? slot_of[t * top + k] : slot_of[T * top + t];
+        if (slot >= 0) sum += y[static_cast<int64_t>(slot) * width + c];
+      }
+      wide[at + c] = sum;      // (read back by the thread that wrote it)
+      ss += sum * sum;
+    }
+  }
+  const float inv = 1.f / sqrtf(block_sum<float, 256>(ss, scratch) / static_cast<float>(width) + eps);
+  if (width <= kOwn * 256) {
+#pragma unroll
+    for (int i = 0; i < kOwn; ++i) {
+      const int c = threadIdx.x + i * 256;
+      if (c < width) {
+        const float now = residual[at + c] + own[i] * inv * w[c];
+        residual[at + c] = now;
+        if (rows) store_f32(rows + at + c, now);
+      }
+    }
+  } else {
+    for (int c = threadIdx.x; c < width; c += 256) {
+      const float now = residual[at + c] + wide[at + c] * inv * w[c];
+      residual[at + c] = now;
+      if (rows) store_f32(rows + at + c, now);
+    }
+  }
 }
 
 }  // namespace alofa
@@ -429,11 +508,13 @@ static int launch_grouped(void* out, const void* x, const void* W, const void* W
   return check_launch("grouped_product");
 }
 
-// out dtype: kBF16 or kF32; x, W, W2, gate bfloat16. epilogue: 0 store, 1 times sigmoid(gate), 2 clamped GLU of (W, W2) times slot_weight.
+// out dtype: kBF16 or kF32; x, W, W2, gate bfloat16. epilogue: 0 store, 1 times sigmoid(gate), 2 clamped GLU of (W, W2) times slot_weight, 3 the square of relu times
+// slot_weight, 4 (dense tiles) the first 2 * turn_pairs outputs of every batch turned by the row's position (pairs of neighbours; cos, sin [positions, turn_pairs]).
 extern "C" int alofa_grouped_product(void* out, int out_dtype, int64_t out_stride, int64_t out_batch_step, const void* x, int64_t x_stride, int64_t x_batch_step,
                                      const void* W, const void* W2, int64_t w_stride, int64_t w_batch_step, int n_out, int K, int last_batch, int n_out_last,
                                      int K_last, int rows, int x_by_slot, int tiles, int tiles_per_batch, int tile_rows, const int32_t* tile_batch, const int32_t* row_in, const void* gate,
-                                     int64_t gate_stride, const float* slot_weight, float limit, float limit_last, float slope, float offset, int epilogue, hipStream_t stream) {
+                                     int64_t gate_stride, const float* slot_weight, float limit, float limit_last, float slope, float offset, int epilogue,
+                                     const int32_t* positions, const float* cos_t, const float* sin_t, int turn_pairs, hipStream_t stream) {
   ALOFA_REQUIRE(n_out > 0 && K > 0 && rows >= 0 && tiles >= 0, "grouped_product: bad sizes (n_out=%d K=%d rows=%d tiles=%d)", n_out, K, rows, tiles);
   ALOFA_REQUIRE(K % 8 == 0 && K_last % 8 == 0 && x_stride % 8 == 0 && x_batch_step % 8 == 0 && w_stride % 8 == 0 && w_batch_step % 8 == 0 &&
                     reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(W) % 16 == 0 && (W2 == nullptr || reinterpret_cast<uintptr_t>(W2) % 16 == 0),
@@ -442,24 +523,29 @@ extern "C" int alofa_grouped_product(void* out, int out_dtype, int64_t out_strid
   ALOFA_REQUIRE(tile_rows == 16 || tile_rows == 64, "grouped_product: tiles of 16 or 64 rows (tile_rows=%d)", tile_rows);
   ALOFA_REQUIRE(epilogue != kGrSigmoidGate || gate, "grouped_product: the gate epilogue needs gates");
   ALOFA_REQUIRE(epilogue != kGrClampedGlu || (W2 && out_dtype == kBF16), "grouped_product: the GLU epilogue needs a second matrix and writes bfloat16");
+  ALOFA_REQUIRE(epilogue != kGrTurn || (tiles_per_batch > 0 && positions && cos_t && sin_t && turn_pairs > 0 && 2 * turn_pairs <= n_out && out_dtype == kBF16),
+                "grouped_product: turned outputs need dense tiles, positions, a table and %d pairs within %d outputs", turn_pairs, n_out);
+  ALOFA_REQUIRE(epilogue != kGrReluSquared || out_dtype == kBF16, "grouped_product: the square of relu is written as bfloat16");
   if (rows == 0 || tiles == 0) return 0;
   GroupedShape s{out_stride, out_batch_step, x_stride, x_batch_step, w_stride, w_batch_step, n_out, K, last_batch, n_out_last, K_last, rows, x_by_slot, tiles, tiles_per_batch,
-                 gate_stride, limit, limit_last, slope, offset};
+                 gate_stride, limit, limit_last, slope, offset, positions, cos_t, sin_t, turn_pairs};
   if (epilogue == kGrStore && out_dtype == kBF16) return launch_grouped<kGrStore, bf16_t>(out, x, W, W2, tile_batch, row_in, gate, slot_weight, s, tile_rows, stream);
   if (epilogue == kGrStore && out_dtype == kF32) return launch_grouped<kGrStore, float>(out, x, W, W2, tile_batch, row_in, gate, slot_weight, s, tile_rows, stream);
   if (epilogue == kGrSigmoidGate && out_dtype == kBF16) return launch_grouped<kGrSigmoidGate, bf16_t>(out, x, W, W2, tile_batch, row_in, gate, slot_weight, s, tile_rows, stream);
   if (epilogue == kGrClampedGlu) return launch_grouped<kGrClampedGlu, bf16_t>(out, x, W, W2, tile_batch, row_in, gate, slot_weight, s, tile_rows, stream);
+  if (epilogue == kGrReluSquared) return launch_grouped<kGrReluSquared, bf16_t>(out, x, W, W2, tile_batch, row_in, gate, slot_weight, s, tile_rows, stream);
+  if (epilogue == kGrTurn) return launch_grouped<kGrTurn, bf16_t>(out, x, W, W2, tile_batch, row_in, gate, slot_weight, s, tile_rows, stream);
   ALOFA_REQUIRE(false, "grouped_product: no such epilogue and output type (epilogue=%d out=%d)", epilogue, out_dtype);
   return 1;
 }
 
 extern "C" int alofa_expert_rows(const int32_t* chosen, const float* weights, int32_t* row_in, float* slot_weight, int32_t* slot_of, int32_t* tile_batch,
-                                 int T, int top, int experts, int shared, int slots, int tiles, int pad, hipStream_t stream) {
+                                 const float* shared_weight, int T, int top, int experts, int shared, int slots, int tiles, int pad, hipStream_t stream) {
   ALOFA_REQUIRE(T > 0 && top > 0 && experts > 0 && experts <= 512 && top <= experts, "expert_rows: bad sizes (T=%d top=%d experts=%d)", T, top, experts);
   ALOFA_REQUIRE(pad == 16 || pad == 64, "expert_rows: tiles of 16 or 64 rows (pad=%d)", pad);
   const int64_t need = (static_cast<int64_t>(T) * top + pad - 1) / pad * pad + pad * static_cast<int64_t>(experts) + (shared ? (T + pad - 1) / pad * pad : 0);
   ALOFA_REQUIRE(slots >= need && static_cast<int64_t>(tiles) * pad >= slots, "expert_rows: room for %lld slots is needed (slots=%d tiles=%d)", (long long)need, slots, tiles);
-  expert_rows_kernel<<<1, 1024, 0, stream>>>(chosen, weights, row_in, slot_weight, slot_of, tile_batch, T, top, experts, shared, slots, tiles, pad);
+  expert_rows_kernel<<<1, 1024, 0, stream>>>(chosen, weights, row_in, slot_weight, slot_of, tile_batch, shared_weight, T, top, experts, shared, slots, tiles, pad);
   return check_launch("expert_rows");
 }
 
@@ -469,4 +555,13 @@ extern "C" int alofa_experts_sum(float* residual, const float* y, const int32_t*
   if (T == 0) return 0;
   experts_sum_kernel<<<static_cast<unsigned>((static_cast<int64_t>(T) * width + 255) / 256), 256, 0, stream>>>(residual, y, slot_of, scale, T, width, top, shared, pass_weight, static_cast<const bf16_t*>(pass_x), pass_stride, assign);
   return check_launch("experts_sum");
+}
+
+extern "C" int alofa_experts_sum_norm(float* residual, const float* y, const int32_t* slot_of, const float* w, float eps, void* rows, float* wide, int T, int width, int top,
+                                      int shared, hipStream_t stream) {
+  ALOFA_REQUIRE(T >= 0 && width > 0 && top > 0 && w && eps > 0.f, "experts_sum_norm: bad arguments");
+  ALOFA_REQUIRE(width <= 4096 || wide, "experts_sum_norm: rows of %d values need room for their sums", width);
+  if (T == 0) return 0;
+  experts_sum_norm_kernel<bf16_t><<<static_cast<unsigned>(T), 256, 0, stream>>>(residual, y, slot_of, w, eps, static_cast<bf16_t*>(rows), wide, T, width, top, shared);
+  return check_launch("experts_sum_norm");
 }

@@ -11,19 +11,23 @@ namespace alofa {
 // sigmoid(z), without its saturation), the lower index first among equals. Outputs:
 //   dense [T, E]: sigmoid(z) * scale at the chosen experts, 0 elsewhere (weights sum to one first when `renorm`);
 //   chosen [T, top], weights [T, top]: the same as lists, in order of falling score.
+// With `softmax` the weights are the softmax over the chosen products alone instead of sigmoids. z has rows of z_stride values; with
+// `shared_weight` the value behind the E products is the gate of an expert that every token takes: shared_weight[t] = its sigmoid.
 // A wavefront per token: lane l holds the products l, l + 64, ... (E up to kMaxExperts); a pick is the best of the lanes'
 // own bests, found by exchanges between lanes (value falling, index rising).
 constexpr int kMaxExperts = 512;
 
 template <typename Acc>
-__global__ void __launch_bounds__(256) route_top_kernel(const float* __restrict__ z, float* __restrict__ dense, int32_t* __restrict__ chosen,
-                                                        float* __restrict__ weights, int tokens, int experts, int top, float scale, int renorm) {
+__global__ void __launch_bounds__(256) route_top_kernel(const float* __restrict__ z, int64_t z_stride, float* __restrict__ dense, int32_t* __restrict__ chosen,
+                                                        float* __restrict__ weights, float* __restrict__ shared_weight, int tokens, int experts, int top, float scale,
+                                                        int renorm, int softmax) {
   constexpr int kOwn = kMaxExperts / kWave;
   const int t = blockIdx.x * 4 + threadIdx.x / kWave, lane = threadIdx.x % kWave;
   if (t >= tokens) return;
-  const float* row = z + static_cast<int64_t>(t) * experts;
+  const float* row = z + static_cast<int64_t>(t) * z_stride;
   float* d = dense + static_cast<int64_t>(t) * experts;
-  float own[kOwn];
+  if (shared_weight && lane == 0) shared_weight[t] = static_cast<float>(static_cast<Acc>(1) / (static_cast<Acc>(1) + exp(-static_cast<Acc>(row[experts]))));
+  float own[kOwn], largest = 0.f;
   bool taken[kOwn];
 #pragma unroll
   for (int i = 0; i < kOwn; ++i) {
@@ -56,7 +60,8 @@ __global__ void __launch_bounds__(256) route_top_kernel(const float* __restrict_
 #pragma unroll
     for (int i = 0; i < kOwn; ++i)
       if (lane + i * kWave == best_e) taken[i] = true;
-    const Acc s = static_cast<Acc>(1) / (static_cast<Acc>(1) + exp(-static_cast<Acc>(best)));
+    if (k == 0) largest = best;
+    const Acc s = softmax ? exp(static_cast<Acc>(best) - static_cast<Acc>(largest)) : static_cast<Acc>(1) / (static_cast<Acc>(1) + exp(-static_cast<Acc>(best)));
     total += s;
     if (lane == 0) {
       chosen[static_cast<int64_t>(t) * top + k] = best_e;
@@ -69,7 +74,7 @@ __global__ void __launch_bounds__(256) route_top_kernel(const float* __restrict_
   if (lane == 0) {
     for (int k = 0; k < top; ++k) {
       Acc w = static_cast<Acc>(weights[static_cast<int64_t>(t) * top + k]);
-      if (renorm) w /= total;
+      if (renorm || softmax) w /= total;
       const float f = static_cast<float>(w * static_cast<Acc>(scale));
       weights[static_cast<int64_t>(t) * top + k] = f;
       d[chosen[static_cast<int64_t>(t) * top + k]] = f;
@@ -219,17 +224,34 @@ __global__ void __launch_bounds__(256) clamped_glu_kernel(T* __restrict__ act, c
   store_f32(act + idx, y);
 }
 
+// ---- the square of relu of all experts side by side ------------------------------------------------
+// act[t, c] = w * max(u[t, c], 0)^2, u [T, F] the up products of E experts of `ff` channels each, then `shared_ff` channels of an expert
+// every token takes; w = dense[t, expert of c], and shared_weight[t] (null: 1) for the shared channels.
+template <typename T, typename Acc>
+__global__ void __launch_bounds__(256) weighted_relu_squared_kernel(T* __restrict__ act, const T* __restrict__ u, const float* __restrict__ dense,
+                                                                    const float* __restrict__ shared_weight, int64_t rows, int experts, int ff, int shared_ff) {
+  const int F = experts * ff + shared_ff;
+  const int64_t idx = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
+  if (idx >= rows * F) return;
+  const int64_t t = idx / F;
+  const int c = static_cast<int>(idx % F);
+  const float w = c < experts * ff ? dense[t * experts + c / ff] : (shared_weight ? shared_weight[t] : 1.f);
+  const Acc z = static_cast<Acc>(fmaxf(load_f32(u + idx), 0.f));
+  store_f32(act + idx, w == 0.f ? 0.f : static_cast<float>(static_cast<Acc>(w) * (z * z)));
+}
+
 }  // namespace alofa
 
 using namespace alofa;
 
-extern "C" int alofa_route_top(const float* z, float* dense, int32_t* chosen, float* weights, int tokens, int experts, int top, float scale, int renorm,
-                               int exact, hipStream_t stream) {
+extern "C" int alofa_route_top(const float* z, int64_t z_stride, float* dense, int32_t* chosen, float* weights, float* shared_weight, int tokens, int experts, int top, float scale, int renorm,
+                               int softmax, int exact, hipStream_t stream) {
+  ALOFA_REQUIRE(z_stride >= experts + (shared_weight ? 1 : 0), "route_top: rows of %lld values do not hold the products", static_cast<long long>(z_stride));
   ALOFA_REQUIRE(tokens >= 0 && experts > 0 && experts <= kMaxExperts && top > 0 && top <= experts, "route_top: bad sizes (tokens=%d experts=%d top=%d)", tokens, experts, top);
   if (tokens == 0) return 0;
   const unsigned grid = static_cast<unsigned>((tokens + 3) / 4);
-  if (exact) route_top_kernel<double><<<grid, 256, 0, stream>>>(z, dense, chosen, weights, tokens, experts, top, scale, renorm);
-  else route_top_kernel<float><<<grid, 256, 0, stream>>>(z, dense, chosen, weights, tokens, experts, top, scale, renorm);
+  if (exact) route_top_kernel<double><<<grid, 256, 0, stream>>>(z, z_stride, dense, chosen, weights, shared_weight, tokens, experts, top, scale, renorm, softmax);
+  else route_top_kernel<float><<<grid, 256, 0, stream>>>(z, z_stride, dense, chosen, weights, shared_weight, tokens, experts, top, scale, renorm, softmax);
   return check_launch("route_top");
 }
 
@@ -243,6 +265,18 @@ extern "C" int alofa_clamped_glu(void* act, const void* g, const void* u, int dt
   else if (dtype == kF32) clamped_glu_kernel<float, float><<<grid, 256, 0, stream>>>(static_cast<float*>(act), static_cast<const float*>(g), static_cast<const float*>(u), dense, rows, experts, ff, shared_ff, limit, shared_limit, slope, offset);
   else clamped_glu_kernel<bf16_t, float><<<grid, 256, 0, stream>>>(static_cast<bf16_t*>(act), static_cast<const bf16_t*>(g), static_cast<const bf16_t*>(u), dense, rows, experts, ff, shared_ff, limit, shared_limit, slope, offset);
   return check_launch("clamped_glu");
+}
+
+extern "C" int alofa_weighted_relu_squared(void* act, const void* u, int dtype, const float* dense, const float* shared_weight, int64_t rows, int experts, int ff, int shared_ff,
+                                           int exact, hipStream_t stream) {
+  ALOFA_REQUIRE(rows >= 0 && experts >= 0 && ff >= 0 && shared_ff >= 0 && experts * ff + shared_ff > 0 && (experts == 0 || dense), "weighted_relu_squared: bad sizes");
+  ALOFA_REQUIRE(!exact || dtype == kF32, "weighted_relu_squared: the exact path is float32");
+  if (rows == 0) return 0;
+  const unsigned grid = static_cast<unsigned>((rows * (experts * ff + shared_ff) + 255) / 256);
+  if (exact) weighted_relu_squared_kernel<float, double><<<grid, 256, 0, stream>>>(static_cast<float*>(act), static_cast<const float*>(u), dense, shared_weight, rows, experts, ff, shared_ff);
+  else if (dtype == kF32) weighted_relu_squared_kernel<float, float><<<grid, 256, 0, stream>>>(static_cast<float*>(act), static_cast<const float*>(u), dense, shared_weight, rows, experts, ff, shared_ff);
+  else weighted_relu_squared_kernel<bf16_t, float><<<grid, 256, 0, stream>>>(static_cast<bf16_t*>(act), static_cast<const bf16_t*>(u), dense, shared_weight, rows, experts, ff, shared_ff);
+  return check_launch("weighted_relu_squared");
 }
 
 extern "C" int alofa_route_groups(const float* z, const float* correction, float* dense, int32_t* chosen, float* weights, float* pass_weight, int tokens,

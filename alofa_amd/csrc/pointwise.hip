@@ -539,6 +539,50 @@ __global__ void __launch_bounds__(256) add_channel_scaled_norm_kernel(float* __r
     store_f32(normed + at + c, static_cast<float>(static_cast<Acc>(residual[at + c]) * inv * static_cast<Acc>(w[c])));
 }
 
+// ---- residual[t, :] += rmsnorm(x[t, :]) * w, and rows[t, :] = the stream's new row as it stands, in the activation type (rows null:
+// not left): the norm behind a sub-layer on its way into the stream, and what the next sub-layer reads (a block per row; the row waits
+// in registers) ----
+template <typename TO, typename Acc>
+__global__ void __launch_bounds__(256) rmsnorm_add_kernel(float* __restrict__ residual, const float* __restrict__ x, const float* __restrict__ w,
+                                                          TO* __restrict__ rows, int width, float eps) {
+  __shared__ Acc scratch[4];
+  constexpr int kOwn = 8;      // values a thread keeps (rows up to 2,048 wide; wider ones are read again)
+  const int64_t at = static_cast<int64_t>(blockIdx.x) * width;
+  float own[kOwn], old[kOwn];
+  Acc ss = 0;
+#pragma unroll
+  for (int i = 0; i < kOwn; ++i) {
+    const int c = threadIdx.x + i * 256;
+    own[i] = c < width ? x[at + c] : 0.f;
+    old[i] = c < width ? residual[at + c] : 0.f;
+    ss += static_cast<Acc>(own[i]) * static_cast<Acc>(own[i]);
+  }
+  for (int c = threadIdx.x + kOwn * 256; c < width; c += 256) ss += static_cast<Acc>(x[at + c]) * static_cast<Acc>(x[at + c]);
+  const Acc inv = static_cast<Acc>(1) / sqrt(block_sum<Acc, 256>(ss, scratch) / static_cast<Acc>(width) + static_cast<Acc>(eps));
+#pragma unroll
+  for (int i = 0; i < kOwn; ++i) {
+    const int c = threadIdx.x + i * 256;
+    if (c < width) {
+      const float now = static_cast<float>(static_cast<Acc>(old[i]) + static_cast<Acc>(own[i]) * inv * static_cast<Acc>(w[c]));
+      residual[at + c] = now;
+      if (rows) store_f32(rows + at + c, now);
+    }
+  }
+  for (int c = threadIdx.x + kOwn * 256; c < width; c += 256) {
+    const float now = static_cast<float>(static_cast<Acc>(residual[at + c]) + static_cast<Acc>(x[at + c]) * inv * static_cast<Acc>(w[c]));
+    residual[at + c] = now;
+    if (rows) store_f32(rows + at + c, now);
+  }
+}
+
+// ---- out = x in the activation type (eight values a thread) ------------------------------------------------------------
+__global__ void __launch_bounds__(256) to_bf16_kernel(bf16_t* __restrict__ out, const float* __restrict__ x, int64_t elements) {
+  const int64_t e = (static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x) * 8;
+#pragma unroll
+  for (int i = 0; i < 8; ++i)
+    if (e + i < elements) out[e + i] = f32_to_bf16(x[e + i]);
+}
+
 // ---- x = cap * tanh(x / cap) ---------------------------------------------------------------------------------------
 template <typename Acc>
 __global__ void __launch_bounds__(256) softcap_kernel(float* __restrict__ x, float cap, int64_t elements) {
@@ -630,6 +674,25 @@ extern "C" int alofa_add_channel_scaled_norm(float* residual, const float* x, co
   else if (normed_dtype == kF32) add_channel_scaled_norm_kernel<float, float><<<grid, 256, 0, stream>>>(residual, x, scale, static_cast<float*>(normed), w, width, eps);
   else add_channel_scaled_norm_kernel<bf16_t, float><<<grid, 256, 0, stream>>>(residual, x, scale, static_cast<bf16_t*>(normed), w, width, eps);
   return check_launch("add_channel_scaled_norm");
+}
+
+// normed_dtype names the type of `rows` (null: the new rows are left nowhere else).
+extern "C" int alofa_rmsnorm_add(float* residual, const float* x, const float* w, void* rows, int rows_dtype, int64_t n, int width, float eps, int exact, hipStream_t stream) {
+  ALOFA_REQUIRE(n >= 0 && width > 0 && w && eps > 0.f, "rmsnorm_add: bad arguments");
+  ALOFA_REQUIRE(!exact || rows == nullptr || rows_dtype == kF32, "rmsnorm_add: the exact path writes float32");
+  if (n == 0) return 0;
+  const unsigned grid = static_cast<unsigned>(n);
+  if (exact) rmsnorm_add_kernel<float, double><<<grid, 256, 0, stream>>>(residual, x, w, static_cast<float*>(rows), width, eps);
+  else if (rows_dtype == kF32) rmsnorm_add_kernel<float, float><<<grid, 256, 0, stream>>>(residual, x, w, static_cast<float*>(rows), width, eps);
+  else rmsnorm_add_kernel<bf16_t, float><<<grid, 256, 0, stream>>>(residual, x, w, static_cast<bf16_t*>(rows), width, eps);
+  return check_launch("rmsnorm_add");
+}
+
+extern "C" int alofa_to_bf16(void* out, const float* x, int64_t elements, hipStream_t stream) {
+  ALOFA_REQUIRE(elements >= 0, "to_bf16: bad sizes");
+  if (elements == 0) return 0;
+  to_bf16_kernel<<<blocks_of((elements + 7) / 8), 256, 0, stream>>>(static_cast<bf16_t*>(out), x, elements);
+  return check_launch("to_bf16");
 }
 
 extern "C" int alofa_softcap(float* x, float cap, int64_t elements, int exact, hipStream_t stream) {

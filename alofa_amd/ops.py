@@ -662,10 +662,18 @@ def _value_planes(out, all_value_heads: bool, v_head, kv_heads: int) -> int:
     return kv_heads
 
 
+def _sink_of(sink: Optional[torch.Tensor], heads: int) -> Optional[torch.Tensor]:
+    if sink is not None:
+        _gpu("sink", sink, torch.float32, 1), _contig("sink", sink)
+        if sink.shape[0] != heads:
+            raise AlofaError("shape_mismatch", "one sink per head", f"sink={tuple(sink.shape)} heads={heads}")
+    return sink
+
+
 def attention_decode(out, q, k_cache, v_cache, block_table, req_of_token, positions, heads, kv_heads, d, window, scale,
                      max_context: int, scratch: Optional[torch.Tensor], rows: Optional[torch.Tensor] = None,
                      rope: Optional[tuple] = None, n_splits: Optional[int] = None, hand_over: Optional[bool] = None,
-                     v_head: Optional[int] = None, fine_weights: bool = False, all_value_heads: bool = False) -> None:
+                     v_head: Optional[int] = None, fine_weights: bool = False, all_value_heads: bool = False, sink: Optional[torch.Tensor] = None) -> None:
     """bfloat16 attention for tokens of requests that bring few tokens: every
     token of the batch, or the tokens ``rows`` (int32 indices into the batch).
     ``req_of_token`` None: every request brings one token and token i is request
@@ -681,7 +689,8 @@ def attention_decode(out, q, k_cache, v_cache, block_table, req_of_token, positi
     ``all_value_heads``: one launch serves every value head in turn as ``v_head``; ``out`` is then float32 [kv_heads, T, heads * d], a
     plane per value head, and a scratch buffer is sized with tokens x kv_heads for ``tokens``.
     ``out`` may be float32: the results are then stored unrounded. ``fine_weights``: every softmax weight meets the values as two bfloat16
-    numbers, its rounding and what the rounding took away, so that sixteen bits of it count (twice the second product's instructions)."""
+    numbers, its rounding and what the rounding took away, so that sixteen bits of it count (twice the second product's instructions).
+    ``sink`` [heads] float32: exp(sink) joins the denominator of the head's rows."""
     planes = _value_planes(out, all_value_heads, v_head, kv_heads)
     T, bs = _attention_operands(out[0] if planes else out, q, k_cache, v_cache, block_table, heads, kv_heads, d)
     for n, t in (("req_of_token", req_of_token), ("positions", positions)):
@@ -729,7 +738,7 @@ def attention_decode(out, q, k_cache, v_cache, block_table, req_of_token, positi
           _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _I(block_table.shape[1]), _ptr(req_of_token), _ptr(positions), _ptr(rows),
           _I(served), _I(heads), _I(kv_heads), _I(d), _I(bs), _I(int(window or 0)), _F(scale), _I(n_splits),
           _ptr(cos), _ptr(sin), _ptr(slots), _I(int(hand_over)), _I(-1 if v_head is None else v_head), _ptr(out if as32 else None), _I(int(fine_weights)),
-          _I(planes), _L(out.stride(0) if planes else 0), _stream())
+          _I(planes), _L(out.stride(0) if planes else 0), _ptr(_sink_of(sink, heads)), _stream())
 
 
 def can_fuse_rope_into_decode(d: int) -> bool:
@@ -804,15 +813,16 @@ def pair_tiles(runs: list, window: Optional[int] = None, heads: Optional[int] = 
 
 
 def attention_prefill(out, q, k_cache, v_cache, block_table, tiles, heads, kv_heads, d, window, scale, share: int = 0,
-                      rows: int = 16, v_head: Optional[int] = None, fine_weights: bool = False, all_value_heads: bool = False) -> None:
+                      rows: int = 16, v_head: Optional[int] = None, fine_weights: bool = False, all_value_heads: bool = False,
+                      sink: Optional[torch.Tensor] = None) -> None:
     """bfloat16 attention for portions of prompts. ``tiles`` is int32 [n, 2, 4]
     from ``pair_tiles``: per block up to two runs of rows, each (request index,
     first row, rows <= 64 or 0 for none, position of the first row). ``share``
     (from ``prefill_share``; the tiles were paired for its count of blocks):
     that many heads of a group are served from one staged tile. ``rows``: query rows a wave owns
     (from ``prefill_rows``; the tiles were paired for it too). ``v_head``: every query head's weights meet the values of this one
-    value head; ``all_value_heads``: one launch serves every value head in turn so, ``out`` float32 [kv_heads, T, heads * d]. ``out`` may be float32: the results are then stored unrounded. ``fine_weights`` (with ``share`` 0 and 16 ``rows``): every softmax
-    weight meets the values as two bfloat16 numbers, so that sixteen bits of it count."""
+    value head; ``all_value_heads``: one launch serves every value head in turn so, ``out`` float32 [kv_heads, T, heads * d]. ``out`` may be float32: the results are then stored unrounded. ``fine_weights`` (with 16 ``rows``): every softmax
+    weight meets the values as two bfloat16 numbers, so that sixteen bits of it count. ``sink`` [heads] float32: exp(sink) joins the denominator of the head's rows."""
     planes = _value_planes(out, all_value_heads, v_head, kv_heads)
     T, bs = _attention_operands(out[0] if planes else out, q, k_cache, v_cache, block_table, heads, kv_heads, d)
     if d not in PREFILL_HEAD_DIMS:
@@ -826,7 +836,7 @@ def attention_prefill(out, q, k_cache, v_cache, block_table, tiles, heads, kv_he
     _call("alofa_attention_prefill_v", _ptr(None if as32 else out), _L(_rows("out", out[0] if planes else out)), _ptr(q), _L(_rows("q", q)), _ptr(k_cache), _ptr(v_cache),
           _ptr(block_table), _I(block_table.shape[1]), _ptr(tiles), _I(tiles.shape[0]), _I(heads), _I(kv_heads), _I(d), _I(bs),
           _I(int(window or 0)), _F(scale), _I(share), _I(rows), _I(-1 if v_head is None else v_head), _ptr(out if as32 else None), _I(int(fine_weights)),
-          _I(planes), _L(out.stride(0) if planes else 0), _stream())
+          _I(planes), _L(out.stride(0) if planes else 0), _ptr(_sink_of(sink, heads)), _stream())
 
 
 # ------------------------------------------------------------------ sampling
@@ -1392,6 +1402,28 @@ def add_channel_scaled(residual: torch.Tensor, x: torch.Tensor, scale: torch.Ten
     _call("alofa_add_channel_scaled", _ptr(residual), _ptr(x), _ptr(scale), _L(residual.shape[0]), _I(residual.shape[1]), _I(int(exact)), _stream())
 
 
+def rmsnorm_add(residual: torch.Tensor, x: torch.Tensor, w: torch.Tensor, eps: float, rows: Optional[torch.Tensor] = None, exact: bool = False) -> None:
+    """residual[t] += rmsnorm(x[t]) * w (residual and x float32); ``rows`` (the stream's shape): the stream's new rows are left there too, in its dtype."""
+    _gpu("residual", residual, torch.float32, 2), _gpu("x", x, torch.float32, 2), _gpu("w", w, torch.float32, 1)
+    _contig("residual", residual), _contig("x", x), _contig("w", w)
+    T, h = residual.shape
+    if x.shape != residual.shape or w.shape[0] != h:
+        raise AlofaError("shape_mismatch", "rows of the stream's shape, one norm weight per channel", f"residual={tuple(residual.shape)} x={tuple(x.shape)} w={tuple(w.shape)}")
+    if rows is not None:
+        _gpu("rows", rows, None, 2), _contig("rows", rows)
+        if rows.shape != residual.shape:
+            raise AlofaError("shape_mismatch", "the new rows do not fit the stream", f"rows={tuple(rows.shape)} residual={tuple(residual.shape)}")
+    _call("alofa_rmsnorm_add", _ptr(residual), _ptr(x), _ptr(w), _ptr(rows), _I(dtype_code(rows) if rows is not None else F32), _L(T), _I(h), _F(eps), _I(int(exact)), _stream())
+
+
+def to_bfloat16(out: torch.Tensor, x: torch.Tensor) -> None:
+    """out = x rounded to bfloat16 (x float32)."""
+    _gpu("out", out, torch.bfloat16), _gpu("x", x, torch.float32), _contig("out", out), _contig("x", x)
+    if out.shape != x.shape:
+        raise AlofaError("shape_mismatch", "input and output must agree", f"out={tuple(out.shape)} x={tuple(x.shape)}")
+    _call("alofa_to_bf16", _ptr(out), _ptr(x), _L(x.numel()), _stream())
+
+
 def softcap_(x: torch.Tensor, cap: float, exact: bool = False) -> None:
     """x = cap * tanh(x / cap) (float32, contiguous)."""
     _gpu("x", x, torch.float32), _contig("x", x)
@@ -1410,17 +1442,24 @@ MAX_EXPERTS = 512
 
 
 def route_top(z: torch.Tensor, dense: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor, top: int, scale: float = 1.0,
-              renormalize: bool = False, exact: bool = False) -> None:
+              renormalize: bool = False, exact: bool = False, softmax: bool = False, shared_weight: Optional[torch.Tensor] = None) -> None:
     """Per row of the router products z [T, E] (float32) the ``top`` largest (the lower index among equals):
     ``chosen`` int32 [T, top] and ``weights`` float32 [T, top] = sigmoid(z) * scale (made to sum to one first with
-    ``renormalize``), in order of falling score; ``dense`` float32 [T, E] holds the same weights at the chosen places and 0 elsewhere."""
+    ``renormalize``), in order of falling score; ``dense`` float32 [T, E] holds the same weights at the chosen places and 0 elsewhere.
+    ``softmax``: the weights are the softmax over the chosen products alone (times ``scale``). ``shared_weight`` float32 [T]: z has one column
+    more, the gate of an expert that every row takes, and its sigmoid is left here."""
     _gpu("z", z, torch.float32, 2), _gpu("dense", dense, torch.float32, 2), _gpu("chosen", chosen, torch.int32, 2), _gpu("weights", weights, torch.float32, 2)
-    for n, t in (("z", z), ("dense", dense), ("chosen", chosen), ("weights", weights)):
+    for n, t in (("dense", dense), ("chosen", chosen), ("weights", weights)):
         _contig(n, t)
-    T, E = z.shape
-    if tuple(dense.shape) != (T, E) or tuple(chosen.shape) != (T, top) or tuple(weights.shape) != (T, top) or not 0 < top <= E <= MAX_EXPERTS:
+    T, E = dense.shape
+    if shared_weight is not None:
+        _gpu("shared_weight", shared_weight, torch.float32, 1), _contig("shared_weight", shared_weight)
+        if shared_weight.shape[0] != T:
+            raise AlofaError("shape_mismatch", "one weight of the shared expert per row", f"shared_weight={tuple(shared_weight.shape)} rows={T}")
+    if tuple(z.shape) != (T, E + (0 if shared_weight is None else 1)) or tuple(chosen.shape) != (T, top) or tuple(weights.shape) != (T, top) or not 0 < top <= E <= MAX_EXPERTS:
         raise AlofaError("shape_mismatch", "the choice's outputs do not fit", f"z={tuple(z.shape)} dense={tuple(dense.shape)} chosen={tuple(chosen.shape)} top={top}")
-    _call("alofa_route_top", _ptr(z), _ptr(dense), _ptr(chosen), _ptr(weights), _I(T), _I(E), _I(top), _F(scale), _I(int(renormalize)), _I(int(exact)), _stream())
+    _call("alofa_route_top", _ptr(z), _L(_rows("z", z)), _ptr(dense), _ptr(chosen), _ptr(weights), _ptr(shared_weight), _I(T), _I(E), _I(top), _F(scale), _I(int(renormalize)),
+          _I(int(softmax)), _I(int(exact)), _stream())
 
 
 def route_groups(z: torch.Tensor, correction: Optional[torch.Tensor], dense: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor,
@@ -1463,6 +1502,23 @@ def clamped_glu(act: torch.Tensor, g: torch.Tensor, u: torch.Tensor, dense: Opti
           _F(limit), _F(shared_limit), _F(slope), _F(offset), _I(int(exact)), _stream())
 
 
+def weighted_relu_squared(act: torch.Tensor, u: torch.Tensor, dense: Optional[torch.Tensor], shared_weight: Optional[torch.Tensor], experts: int, ff: int, shared_ff: int,
+                          exact: bool = False) -> None:
+    """act[t, c] = w max(u[t, c], 0)^2 for the channels of ``experts`` experts of ``ff`` channels side by side (w = dense[t, expert]) and then
+    ``shared_ff`` channels with w = shared_weight[t] (None: 1)."""
+    _gpu("act", act, None, 2), _gpu("u", u, act.dtype, 2), _contig("act", act), _contig("u", u)
+    T, F = act.shape[0], experts * ff + shared_ff
+    if tuple(u.shape) != (T, F) or act.shape[1] != F:
+        raise AlofaError("shape_mismatch", "input and output are [rows, all experts' channels]", f"act={tuple(act.shape)} u={tuple(u.shape)} F={F}")
+    for n, t, shape in (("dense", dense if experts else None, (T, experts)), ("shared_weight", shared_weight, (T,))):
+        if t is not None:
+            _gpu(n, t, torch.float32), _contig(n, t)
+            if tuple(t.shape) != shape:
+                raise AlofaError("shape_mismatch", "one weight per row and expert", f"operand={n} shape={tuple(t.shape)}")
+    _call("alofa_weighted_relu_squared", _ptr(act), _ptr(u), _I(dtype_code(act)), _ptr(dense if experts else None), _ptr(shared_weight), _L(T), _I(experts), _I(ff), _I(shared_ff),
+          _I(int(exact)), _stream())
+
+
 def gemm_channel_scaled(residual: torch.Tensor, a: torch.Tensor, w: torch.Tensor, scale: torch.Tensor, tmp: torch.Tensor, exact: bool = False,
                         then_norm: Optional[tuple] = None, bias: Optional[torch.Tensor] = None) -> None:
     """residual[t, c] += scale[c] * ((a @ w.T)[t, c] + bias[c]); ``tmp`` float32 of the residual's shape takes the product on its way.
@@ -1488,26 +1544,92 @@ def add_channel_scaled_norm(residual: torch.Tensor, x: torch.Tensor, scale: torc
           _I(int(exact)), _stream())
 
 
-GR_STORE, GR_SIGMOID_GATE, GR_CLAMPED_GLU = 0, 1, 2
+GR_STORE, GR_SIGMOID_GATE, GR_CLAMPED_GLU, GR_RELU_SQUARED, GR_TURN = 0, 1, 2, 3, 4
 GROUPED_BIG_TILES = 256     # rows of a step from which the many-small-products kernel takes tiles of 64 rows instead of 16
 
 
 def _grouped(out, out_step, x, x_step, w, w2, w_stride, w_step, n_out, K, last, rows, x_by_slot, tiles, tiles_per_batch, tile_batch, row_in,
-             gate, slot_weight, limit, limit_last, slope, epilogue, tile_rows=16, offset=1.0) -> None:
+             gate, slot_weight, limit, limit_last, slope, epilogue, tile_rows=16, offset=1.0, turn=None) -> None:
     last_batch, n_out_last, K_last = last if last is not None else (-1, n_out, K)
+    positions, cos, sin = turn if turn is not None else (None, None, None)
     _call("alofa_grouped_product", _ptr(out), _I(dtype_code(out)), _L(_rows("out", out)), _L(out_step), _ptr(x), _L(_rows("x", x)), _L(x_step),
           _ptr(w), _ptr(w2), _L(w_stride), _L(w_step), _I(n_out), _I(K), _I(last_batch), _I(n_out_last), _I(K_last), _I(rows), _I(int(x_by_slot)), _I(tiles),
           _I(tiles_per_batch), _I(tile_rows), _ptr(tile_batch), _ptr(row_in), _ptr(gate), _L(_rows("gate", gate) if gate is not None else 0), _ptr(slot_weight),
-          _F(limit), _F(limit_last), _F(slope), _F(offset), _I(epilogue), _stream())
+          _F(limit), _F(limit_last), _F(slope), _F(offset), _I(epilogue), _ptr(positions), _ptr(cos), _ptr(sin), _I(cos.shape[1] if cos is not None else 0), _stream())
 
 
 def _aligned_rows(t: torch.Tensor) -> bool:
     return t.dtype is torch.bfloat16 and t.stride(-1) == 1 and t.stride(0) % 8 == 0 and t.data_ptr() % 16 == 0
 
 
-def head_project(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, exact: bool = False, gate: Optional[torch.Tensor] = None) -> None:
+def _angles(positions: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor, rows: int) -> None:
+    _gpu("positions", positions, torch.int32, 1), _contig("positions", positions)
+    _gpu("cos", cos, torch.float32, 2), _gpu("sin", sin, torch.float32, 2), _contig("cos", cos), _contig("sin", sin)
+    if positions.shape[0] != rows or cos.shape != sin.shape:
+        raise AlofaError("shape_mismatch", "one position per row, cos and sin alike", f"positions={tuple(positions.shape)} rows={rows} cos={tuple(cos.shape)} sin={tuple(sin.shape)}")
+
+
+def turn_pairs(x: torch.Tensor, positions: torch.Tensor, table: tuple, heads: int, first: int, exact: bool = False) -> None:
+    """Channels first + 2 i and first + 2 i + 1 of every head of x [T, heads * size] turned in place by the row's position (cos, sin [positions, pairs])."""
+    _gpu("x", x, None, 2)
+    cos, sin = table
+    T, pairs = x.shape[0], cos.shape[1]
+    _angles(positions, cos, sin, T)
+    size = x.shape[1] // heads
+    if x.shape[1] != heads * size or first + 2 * pairs > size:
+        raise AlofaError("shape_mismatch", "the pairs do not fit the heads", f"x={tuple(x.shape)} heads={heads} first={first} pairs={pairs}")
+    _call("alofa_turn_pairs", _ptr(x), _L(_rows("x", x)), _I(dtype_code(x)), _ptr(positions), _ptr(cos), _ptr(sin), _I(T), _I(heads), _I(size), _I(first), _I(pairs),
+          _I(int(exact)), _stream())
+
+
+def latent_rows(x: torch.Tensor, queries: Optional[tuple], keys: tuple, turned: int = 0, positions: Optional[torch.Tensor] = None, table: Optional[tuple] = None,
+                pages: Optional[tuple] = None, rows: Optional[torch.Tensor] = None, exact: bool = False) -> None:
+    """What a row's latents become. ``queries`` = (first column, weight, eps, out) or None: out[t] = rmsnorm(x[t, columns]) * weight. ``keys`` = (first column,
+    weight, eps): c = rmsnorm(x[t, columns]) * weight; the ``turned`` values behind them are the key part that all heads share. With ``pages`` = (slots int64 [T],
+    keys [pages, 1, page, d], values [pages, 1, d, page]) the row's slot gets the key [turned part, turned by its position | c | zeros] and the value [zeros | c | zeros];
+    with ``rows`` its row there gets [c | turned part as it is | zeros]."""
+    _gpu("x", x, None, 2)
+    T = x.shape[0]
+    q_at = q_rank = 0
+    q_w = cq = None
+    q_eps = 0.0
+    if queries is not None:
+        q_at, q_w, q_eps, cq = queries
+        q_rank = q_w.shape[0]
+        _gpu("query weight", q_w, torch.float32, 1), _contig("query weight", q_w), _gpu("cq", cq, x.dtype, 2)
+        if tuple(cq.shape) != (T, q_rank) or q_at + q_rank > x.shape[1]:
+            raise AlofaError("shape_mismatch", "the queries' latent does not fit", f"x={tuple(x.shape)} at={q_at} cq={tuple(cq.shape)}")
+    at, w, eps = keys
+    _gpu("key weight", w, torch.float32, 1), _contig("key weight", w)
+    r = w.shape[0]
+    if at + r + turned > x.shape[1] or (pages is None) == (rows is None):
+        raise AlofaError("shape_mismatch", "the keys' latent does not fit, or it goes to pages or to rows", f"x={tuple(x.shape)} at={at} r={r} turned={turned}")
+    slots = k = v = cos = sin = None
+    block = d = 0
+    if pages is not None:
+        slots, k, v = pages
+        _gpu("slots", slots, torch.int64, 1), _contig("slots", slots), _gpu("k", k, x.dtype, 4), _gpu("v", v, x.dtype, 4), _contig("k", k), _contig("v", v)
+        block, d = k.shape[2], k.shape[3]
+        if slots.shape[0] != T or k.shape[1] != 1 or tuple(v.shape) != (k.shape[0], 1, d, block) or d < r + turned:
+            raise AlofaError("shape_mismatch", "caches or slots do not fit", f"k={tuple(k.shape)} v={tuple(v.shape)} slots={tuple(slots.shape)} r={r} turned={turned}")
+        if turned:
+            cos, sin = table
+            _angles(positions, cos, sin, T)
+            if 2 * cos.shape[1] != turned:
+                raise AlofaError("shape_mismatch", "the table of angles does not fit the turned part", f"table={tuple(cos.shape)} turned={turned}")
+    else:
+        _gpu("rows", rows, x.dtype, 2)
+        if rows.shape[0] != T or rows.shape[1] < r + turned:
+            raise AlofaError("shape_mismatch", "the rows do not hold the latent and what lies behind it", f"rows={tuple(rows.shape)} r={r} turned={turned}")
+    _call("alofa_latent_rows", _ptr(x), _L(_rows("x", x)), _I(dtype_code(x)), _I(T), _I(q_at), _I(q_rank), _ptr(q_w), _F(q_eps), _ptr(cq), _L(_rows("cq", cq) if cq is not None else 0),
+          _I(at), _I(r), _I(turned), _ptr(w), _F(eps), _ptr(positions), _ptr(cos), _ptr(sin), _ptr(slots), _ptr(k), _ptr(v), _I(block), _I(d), _ptr(rows),
+          _L(_rows("rows", rows) if rows is not None else 0), _I(rows.shape[1] if rows is not None else 0), _I(int(exact)), _stream())
+
+
+def head_project(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, exact: bool = False, gate: Optional[torch.Tensor] = None, turn: Optional[tuple] = None) -> None:
     """out[t, a, :] = w[a] @ x[t, a, :] for every head a: x [T, H * din] and out [T, H * dout] hold the heads side by side (row
-    strides allowed), w is [H, dout, din]. With ``gate`` (out's shape): out *= sigmoid(gate). bfloat16 rows whose heads start at
+    strides allowed), w is [H, dout, din]. With ``gate`` (out's shape): out *= sigmoid(gate). With ``turn`` = (positions, cos, sin): a head's first
+    2 * pairs outputs are turned, in neighbouring pairs, by the row's position (cos, sin [positions, pairs]). bfloat16 rows whose heads start at
     16-byte borders run as one launch on the matrix cores; everything else head by head through ``gemm``."""
     _gpu("out", out, None, 2), _gpu("x", x, out.dtype, 2), _gpu("w", w, None, 3), _contig("w", w)
     H, dout, din = w.shape
@@ -1518,16 +1640,22 @@ def head_project(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, exact: boo
         if gate.shape != out.shape:
             raise AlofaError("shape_mismatch", "one gate per output", f"gate={tuple(gate.shape)} out={tuple(out.shape)}")
     T = x.shape[0]
+    if turn is not None:
+        _angles(*turn, T)
+        if gate is not None or 2 * turn[1].shape[1] > dout:
+            raise AlofaError("unsupported", "outputs are turned or gated, and the pairs lie within a head", f"pairs={turn[1].shape[1]} dout={dout}")
     if not exact and out.dtype is torch.bfloat16 and w.dtype is torch.bfloat16 and din % 8 == 0 and _aligned_rows(x) and w.data_ptr() % 16 == 0 and T > 0:
         tile_rows = 64 if T >= GROUPED_BIG_TILES else 16      # (tiles of 64 rows, which use a fragment of the matrix four times, once there are rows for them)
         per = (T + tile_rows - 1) // tile_rows
         _grouped(out, dout, x, din, w, None, din, dout * din, dout, din, None, T, False, H * per, per, None, None, gate, None, 0.0, 0.0, 0.0,
-                 GR_SIGMOID_GATE if gate is not None else GR_STORE, tile_rows)
+                 GR_TURN if turn is not None else GR_SIGMOID_GATE if gate is not None else GR_STORE, tile_rows, turn=turn)
         return
     for a in range(H):
         gemm(out[:, a * dout:(a + 1) * dout], x[:, a * din:(a + 1) * din], w[a], exact=exact)
     if gate is not None:
         sigmoid_gate(out, gate, exact)
+    if turn is not None:
+        turn_pairs(out, turn[0], turn[1:], H, 0, exact)
 
 
 class ExpertRows:
@@ -1545,12 +1673,17 @@ class ExpertRows:
         self.slot_of, self.tile_batch = scratch("expert_slot_of", (T * (top + 1),), torch.int32), scratch("expert_tile_batch", (self.tiles,), torch.int32)
 
 
-def expert_rows(rows: ExpertRows, chosen: torch.Tensor, weights: torch.Tensor) -> None:
+def expert_rows(rows: ExpertRows, chosen: torch.Tensor, weights: torch.Tensor, shared_weight: Optional[torch.Tensor] = None) -> None:
+    """``shared_weight`` float32 [T]: the weight of every row's place in the shared expert (None: 1)."""
     _gpu("chosen", chosen, torch.int32, 2), _gpu("weights", weights, torch.float32, 2), _contig("chosen", chosen), _contig("weights", weights)
     if tuple(chosen.shape) != (rows.T, rows.top) or tuple(weights.shape) != (rows.T, rows.top):
         raise AlofaError("shape_mismatch", "one choice and one weight per row and place", f"chosen={tuple(chosen.shape)} weights={tuple(weights.shape)}")
+    if shared_weight is not None:
+        _gpu("shared_weight", shared_weight, torch.float32, 1), _contig("shared_weight", shared_weight)
+        if shared_weight.shape[0] != rows.T:
+            raise AlofaError("shape_mismatch", "one weight of the shared expert per row", f"shared_weight={tuple(shared_weight.shape)} rows={rows.T}")
     _call("alofa_expert_rows", _ptr(chosen), _ptr(weights), _ptr(rows.row_in), _ptr(rows.slot_weight), _ptr(rows.slot_of), _ptr(rows.tile_batch),
-          _I(rows.T), _I(rows.top), _I(rows.experts), _I(int(rows.shared)), _I(rows.slots), _I(rows.tiles), _I(rows.tile_rows), _stream())
+          _ptr(shared_weight), _I(rows.T), _I(rows.top), _I(rows.experts), _I(int(rows.shared)), _I(rows.slots), _I(rows.tiles), _I(rows.tile_rows), _stream())
 
 
 def can_group_experts(x: torch.Tensor, w_gate: torch.Tensor, ff: int, shared_ff: int) -> bool:
@@ -1570,6 +1703,34 @@ def experts_gate_up(act: torch.Tensor, x: torch.Tensor, w_gate: torch.Tensor, w_
         raise AlofaError("shape_mismatch", "the experts' matrices or the slots' rows do not fit", f"act={tuple(act.shape)} x={tuple(x.shape)} w_gate={tuple(w_gate.shape)} F={F}")
     _grouped(act, 0, x, 0, w_gate, w_up, h, ff * h, ff, h, (rows.experts, shared_ff, h) if rows.shared else None, rows.slots, False, rows.tiles, 0,
              rows.tile_batch, rows.row_in, None, rows.slot_weight, limit, shared_limit, slope, GR_CLAMPED_GLU, rows.tile_rows, offset)
+
+
+def experts_up(act: torch.Tensor, x: torch.Tensor, w_up: torch.Tensor, rows: ExpertRows, ff: int, shared_ff: int) -> None:
+    """act[slot, :] = weight[slot] * max(up_e(x[row]), 0)^2 for the expert e of the slot; w_up holds the experts' matrices one below the other."""
+    _gpu("act", act, torch.bfloat16, 2), _gpu("x", x, torch.bfloat16, 2), _gpu("w_up", w_up, torch.bfloat16, 2), _contig("w_up", w_up), _contig("act", act)
+    h = x.shape[1]
+    F = rows.experts * ff + (shared_ff if rows.shared else 0)
+    if tuple(w_up.shape) != (F, h) or act.shape[0] < rows.slots or act.shape[1] < max(ff, shared_ff) or x.shape[0] != rows.T:
+        raise AlofaError("shape_mismatch", "the experts' matrices or the slots' rows do not fit", f"act={tuple(act.shape)} x={tuple(x.shape)} w_up={tuple(w_up.shape)} F={F}")
+    _grouped(act, 0, x, 0, w_up, None, h, ff * h, ff, h, (rows.experts, shared_ff, h) if rows.shared else None, rows.slots, False, rows.tiles, 0,
+             rows.tile_batch, rows.row_in, None, rows.slot_weight, 0.0, 0.0, 0.0, GR_RELU_SQUARED, rows.tile_rows)
+
+
+def experts_sum_norm(residual: torch.Tensor, y: torch.Tensor, rows: ExpertRows, weight: torch.Tensor, eps: float, out: Optional[torch.Tensor] = None,
+                     scratch=None) -> None:
+    """residual[t] += rmsnorm(s) * weight with s the sum of row t's slots (``experts_sum``'s); ``out`` bfloat16 of the stream's shape: the stream's new rows are left
+    there too. ``scratch(name, shape, dtype)`` gives the room that rows of more than 4,096 values need."""
+    _gpu("residual", residual, torch.float32, 2), _gpu("y", y, torch.float32, 2), _gpu("weight", weight, torch.float32, 1)
+    _contig("residual", residual), _contig("y", y), _contig("weight", weight)
+    T, h = residual.shape
+    if T != rows.T or tuple(y.shape) != (rows.slots, h) or weight.shape[0] != h:
+        raise AlofaError("shape_mismatch", "the slots' results or the norm's weight do not fit the stream", f"residual={tuple(residual.shape)} y={tuple(y.shape)} weight={tuple(weight.shape)}")
+    if out is not None:
+        _gpu("out", out, torch.bfloat16, 2), _contig("out", out)
+        if out.shape != residual.shape:
+            raise AlofaError("shape_mismatch", "the new rows do not fit the stream", f"out={tuple(out.shape)} residual={tuple(residual.shape)}")
+    wide = scratch("experts_wide_sum", (T, h), torch.float32) if h > 4096 else None
+    _call("alofa_experts_sum_norm", _ptr(residual), _ptr(y), _ptr(rows.slot_of), _ptr(weight), _F(eps), _ptr(out), _ptr(wide), _I(T), _I(h), _I(rows.top), _I(int(rows.shared)), _stream())
 
 
 def experts_down(y: torch.Tensor, act: torch.Tensor, w_down: torch.Tensor, rows: ExpertRows, ff: int, shared_ff: int) -> None:

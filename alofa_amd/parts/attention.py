@@ -44,15 +44,20 @@ class RowPlan:
                 self.short_rows = torch.tensor([r for s in spans if s.n <= SHORT for r in range(s.row0, s.row0 + s.n)],
                                                dtype=torch.int32, device=self.device)
 
-    def tiles(self, heads: int, kv_heads: int, d: int, window, plain: bool = False):
+    def runs_of_sixteen(self):
+        """The runs in pieces of up to sixteen rows: int32 [n, 3] (request index, first row, rows)."""
+        return torch.tensor([(r, row0 + q0, min(16, n - q0)) for r, row0, n, _ in self.long_runs for q0 in range(0, n, 16)], dtype=torch.int32, device=self.device)
+
+    def tiles(self, heads: int, kv_heads: int, d: int, window, plain: bool = False, fine: bool = False):
         """The runs as blocks of the prefill kernel for a mixer with these head counts, how many heads
         of a group share a block's tiles and how many rows a wave owns (all three depend on how many
         blocks there are). ``plain``: every head has blocks of its own and a wave owns 16 rows (the
-        one form of the kernel that takes the weights in two parts)."""
-        key = (heads, kv_heads, d, window, plain)
+        first form of the kernel that takes the weights in two parts). ``fine``: a wave owns 16 rows and takes the
+        weights in two parts, and heads may share."""
+        key = (heads, kv_heads, d, window, plain, fine)
         if key not in self._tiles:
             share = 0 if plain else ops.prefill_share(heads, kv_heads, d, len(self.long_runs))
-            rows = 16 if plain else ops.prefill_rows(heads, kv_heads, d, share, len(self.long_runs))
+            rows = 16 if plain or fine else ops.prefill_rows(heads, kv_heads, d, share, len(self.long_runs))
             per_run = ops.prefill_blocks_per_run(heads, kv_heads, share, rows)
             self._tiles[key] = (torch.tensor(ops.pair_tiles(self.long_runs, window, per_run), dtype=torch.int32, device=self.device), share, rows)
         return self._tiles[key]
@@ -101,6 +106,31 @@ def paged_attend(ctx, entry, qkv, attn, heads, kv_heads, d, window, scale, posit
             one_each = ctx.max_q_len == 1 and plan.short_rows is None and plan.long_runs is None
             ops.attention_decode(attn, qkv, kv.k, kv.v, kv.block_table, None if one_each else ctx.req_of_token, ctx.positions, *common,
                                  ctx.max_context, partial, rows=plan.short_rows, rope=(cos, sin, kv.slots) if fused else None)
+
+
+def attend_pages(ctx, kv, q, attn, heads, kv_heads, d, window, scale, rt, sink=None) -> None:
+    """The rows of one step through attention over pages that already hold their keys and values: ``q`` [T, heads d] are the step's queries as they
+    ask, ``attn`` [T, heads d] receives the softmax's sums; ``sink`` (float32 [heads] or None) joins the denominators. Softmax weights are 32-bit
+    numbers here: on the matrix cores each meets the values as two bfloat16 numbers."""
+    common = (heads, kv_heads, d, window, scale)
+    page = kv.k.shape[2]
+    if rt.exact or not ops.span_attention_fast(d, page, rt.dtype):      # the exact path, and page or head sizes the bfloat16 kernels are not built for
+        ops.span_attention(attn, q, kv.k, kv.v, kv.block_table, ctx.req_of_token, ctx.positions, heads, kv_heads, d, d, window, scale, rt.exact, sink=sink)
+        return
+    plan = ctx.memo("gqa_attention.rows", lambda: RowPlan(ctx))
+    if plan.long_runs is not None and d not in ops.PREFILL_HEAD_DIMS:
+        runs = ctx.memo("runs of sixteen rows", lambda: plan.runs_of_sixteen())
+        ops.span_attention_mfma(attn, q, kv.k, kv.v, kv.block_table, runs, ctx.req_of_token, ctx.positions, *common, sink=sink)
+    elif plan.long_runs is not None:      # portions of prompts
+        tiles, share, rows = plan.tiles(heads, kv_heads, d, window, fine=True)
+        ops.attention_prefill(attn, q, kv.k, kv.v, kv.block_table, tiles, *common, share=share, rows=rows, fine_weights=True, sink=sink)
+    if plan.n_short:                    # single tokens and very short portions, all query heads of a key head together
+        floats = ops.decode_scratch_floats(plan.n_short, heads, kv_heads, d, ctx.max_context, window)
+        partial = ctx.scratch("attn_partial", (floats,), torch.float32) if floats else None
+        # (one token per request and nothing else in the step: token i is request i)
+        one_each = ctx.max_q_len == 1 and plan.short_rows is None and plan.long_runs is None
+        ops.attention_decode(attn, q, kv.k, kv.v, kv.block_table, None if one_each else ctx.req_of_token, ctx.positions, *common,
+                             ctx.max_context, partial, rows=plan.short_rows, fine_weights=True, sink=sink)
 
 
 NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight",

@@ -271,6 +271,7 @@ class Block(Part):
 
 class Norm(Part):
     family = "norm"
+    identity = False      # True: the rows as they are (in the reader's dtype)
 
     def as_rmsnorm(self):
         """(weight float32 [width], eps) when the norm is x / sqrt(mean(x^2) + eps) * weight, which

@@ -12,7 +12,10 @@ filtered_prenorm: the same as prenorm with a filter over time in front of every 
 optional weighted average over the outputs of all layers so far.
 
 sandwich: a += post0(mixer(pre0(a))); a += post1(feed_forward(pre1(a))): a norm in front of every sub-layer and one behind it, before
-the sum; the feed-forward optional."""
+the sum; the feed-forward optional.
+
+postnorm: a += post0(mixer(a)); a += post1(feed_forward(a)): the sub-layers read the stream itself, and a norm stands behind every one of
+them, before the sum; the feed-forward optional."""
 from __future__ import annotations
 
 import os
@@ -20,6 +23,7 @@ import os
 import torch
 
 from .. import ops
+from ..config.base import PartSpec
 from ..errors import AlofaError
 from ..weights.loader import TensorRule
 from .base import Block, build_part, register_part, tensors_of
@@ -308,9 +312,80 @@ class SandwichBlock(Block):
         return self._join_then(hidden, apart, self.norms[3], then)
 
 
+class PostNormBlock(Block):
+    """a += post0(mixer(a)), then, where the layer has a feed-forward, a += post1(feed_forward(a)): the sub-layers read the stream itself (in the
+    activation dtype). It reads the layer's parts ``mixer``, ``feed_forward`` (may be None) and ``norms`` (one per sub-layer).
+    Mixer and feed-forward leave their results apart (``out=``); an RMSNorm behind one is applied by the launch that adds to the stream and
+    leaves the stream's new rows for the next reader. A part that says ``takes_post_norm`` is handed that norm (``post=`` (weight, eps, rows
+    or None)) and sees to norm and sum itself."""
+
+    @classmethod
+    def layer_tensors(cls, layer) -> dict:
+        out = {}
+        for n in layer.part("norms"):
+            out.update(tensors_of("norm", n))
+        out.update(tensors_of("mixer", layer.part("mixer")))
+        if layer.part("feed_forward") is not None:
+            out.update(tensors_of("feed_forward", layer.part("feed_forward")))
+        return out
+
+    def __init__(self, layer, weights, rt):
+        super().__init__(layer, weights, rt)
+        ff = layer.part("feed_forward")
+        norms = layer.part("norms")
+        if len(norms) != (1 if ff is None else 2):
+            raise AlofaError("invalid_argument", "one norm behind every sub-layer", f"prefix={layer.prefix} norms={len(norms)} feed_forward={ff is not None}")
+        self.norms = [build_part("norm", n, weights, rt) for n in norms]
+        self.front = build_part("norm", PartSpec("identity"), weights, rt)
+        self.mixer = build_part("mixer", layer.part("mixer"), weights, rt)
+        self.feed_forward = build_part("feed_forward", ff, weights, rt) if ff is not None else None
+        self.parts = [p for p in (*self.norms, self.mixer, self.feed_forward) if p is not None]
+
+    def mixers(self):
+        return self.mixer.stateful_parts()
+
+    takes_normed = True
+    leaves_rows = True      # the launch that adds this block's last result can leave the stream's rows in the activation dtype
+
+    def wants_normed(self, rows):
+        return None if self.rt.dtype is torch.float32 else self.front      # (float32: the sub-layers read the stream where it lies)
+
+    def _sub_layer(self, ctx, part, norm, x, hidden, rows, where=()):
+        """hidden += norm(part(x)); ``rows`` (or None) holds the stream's new rows afterwards."""
+        rms = norm.as_rmsnorm()
+        if rms is not None and FUSE_SUMS and getattr(part, "takes_post_norm", False):
+            part.forward(ctx, *where, x, hidden, post=(*rms, rows))
+            return
+        apart = ctx.scratch("sub_out", tuple(hidden.shape), torch.float32)
+        part.forward(ctx, *where, x, hidden, out=apart)
+        if rms is not None and FUSE_SUMS:
+            ops.rmsnorm_add(hidden, apart, *rms, rows=rows, exact=self.rt.exact)
+            return
+        norm.forward(apart, apart)
+        ops.add_scaled(hidden, apart, 1.0, exact=self.rt.exact)
+        if rows is not None:
+            self.front.forward(rows, hidden)
+
+    def forward(self, ctx, entry, hidden, normed=None, then=None):
+        """``normed``: the stream's rows in the activation dtype, where the block before has left them; ``then`` = (norm, rows): what the next
+        block starts with; rows of the stream itself are left there. Returns whether that was done."""
+        buf = None if self.rt.dtype is torch.float32 else ctx.scratch("normed", tuple(hidden.shape), self.rt.dtype)
+        x = hidden if buf is None else normed
+        if x is None:
+            self.front.forward(buf, hidden)
+            x = buf
+        left = then[1] if then is not None and then[0].identity else None
+        ff = self.feed_forward
+        self._sub_layer(ctx, self.mixer, self.norms[0], x, hidden, buf if ff is not None else left, where=((entry, 0),))
+        if ff is not None:
+            self._sub_layer(ctx, ff, self.norms[1], hidden if buf is None else buf, hidden, left)
+        return left is not None
+
+
 FUSE_SUMS = os.environ.get("ALOFA_FUSE_SUMS", "1") != "0"      # 0 (for measurements): a scaled sum into the stream and the norm behind it are two launches
 
 register_part("block", "prenorm", PreNormBlock)
 register_part("block", "scaled_prenorm", ScaledPreNormBlock)
 register_part("block", "filtered_prenorm", FilteredPreNormBlock)
 register_part("block", "sandwich", SandwichBlock)
+register_part("block", "postnorm", PostNormBlock)

@@ -22,26 +22,28 @@ from .base import FeedForward, register_part
 
 
 class SwiGLU(FeedForward):
-    """params: prefix, hidden, intermediate."""
+    """params: prefix, hidden, intermediate; optional: names (tensor names after the prefix for gate, up, down, default the *_proj ones), init (the rule
+    random weights are drawn by). ``forward(..., out=)``: the result is stored there (float32, the stream's shape) and the stream left alone."""
+    NAMES = {"gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
     capturable = True   # native kernels on the current stream only: a decode step may be graph-captured
 
     @classmethod
     def tensors(cls, spec):
         p = spec.params
         pre, h, i = p["prefix"], p["hidden"], p["intermediate"]
-        return {pre + "gate_proj.weight": TensorRule((i, h)), pre + "up_proj.weight": TensorRule((i, h)),
-                pre + "down_proj.weight": TensorRule((h, i))}
+        n, init = {**cls.NAMES, **p.get("names", {})}, p.get("init", "matrix")
+        return {pre + n["gate"]: TensorRule((i, h), init), pre + n["up"]: TensorRule((i, h), init), pre + n["down"]: TensorRule((h, i), init)}
 
     def __init__(self, spec, weights, rt):
         super().__init__(spec, weights, rt)
         p = spec.params
         self.hidden, self.intermediate = int(p["hidden"]), int(p["intermediate"])
-        pre = p["prefix"]
-        gate, up = weights[pre + "gate_proj.weight"], weights[pre + "up_proj.weight"]
+        pre, n = p["prefix"], {**self.NAMES, **p.get("names", {})}
+        gate, up = weights[pre + n["gate"]], weights[pre + n["up"]]
         if gate.dtype is not up.dtype:
             gate, up = gate.float(), up.float()
         self.w_gate, self.w_up = rt.matrix(gate), rt.matrix(up)
-        self.w_down = rt.matrix(weights[pre + "down_proj.weight"])
+        self.w_down = rt.matrix(weights[pre + n["down"]])
 
     def fuses_norm(self, norm, rows):
         return (not self.rt.exact and norm.as_rmsnorm() is not None
@@ -49,12 +51,15 @@ class SwiGLU(FeedForward):
 
     gives_normed = True
 
-    def forward(self, ctx, x, residual, norm=None, then=None):
+    def forward(self, ctx, x, residual, norm=None, then=None, out=None):
         act = ctx.scratch("ff_act", (residual.shape[0], self.intermediate), self.rt.dtype)
         if norm is not None:      # the norm before the feed-forward rides on the gate/up product
             ops.gemm_swiglu(act, residual, self.w_gate, self.w_up, norm=norm.as_rmsnorm())
         else:
             ops.gemm_swiglu(act, x, self.w_gate, self.w_up, exact=self.rt.exact)
+        if out is not None:
+            ops.gemm(out, act, self.w_down, exact=self.rt.exact)
+            return
         then_norm = None
         if then is not None:      # the norm behind this part, left in the rows given with it
             weight, eps = then[0].as_rmsnorm()

@@ -12,7 +12,17 @@ The cache holds c twice, as keys [page, 1, slot, d] and as transposed values [pa
 the kernels are built for, with zeros), the layouts those kernels read.
 
 A latent wider than the largest head the kernels take cannot be a head: there the keys and values of every head are formed
-from c when it is made (k_a = Uk_a c, v_a = Uv_a c) and kept per head in the pages, as for any attention with H key heads."""
+from c when it is made (k_a = Uk_a c, v_a = Uv_a c) and kept per head in the pages, as for any attention with H key heads.
+
+Optional, each chosen by a parameter:
+  q_latent   queries through a latent of their own: q = Wuq norm(Wdq x).
+  turned     n more channels of every head's query, turned by the row's position in neighbouring pairs, and one key part of n channels for all heads,
+             the last n rows of Wd x (not normed), turned likewise: the score is scale * (q_a . k_a + q'_a . k'). The key that all heads ask is then
+             [k' | c], the query of a head [q'_a | Uk_a^T q_a]; what the pages hold beside c is k'. (Where the pages hold every head's keys, k' is
+             a part of each.)
+  sink       a number per head whose exponential joins the softmax's denominator (no key, no value, not scaled).
+  window     a row sees itself and the window - 1 rows before it.
+With any of the first three, softmax weights meet the values with sixteen bits each on the matrix cores."""
 from __future__ import annotations
 
 import torch
@@ -21,10 +31,10 @@ from .. import ops
 from ..errors import AlofaError
 from ..config.base import PartSpec
 from ..weights.loader import TensorRule
-from .attention import GQAAttention, _padded_heads, paged_attend
+from .attention import GQAAttention, _padded_heads, attend_pages, paged_attend
 from .base import CacheNeed, Mixer, build_part, register_part, tensors_of
 
-NAMES = {"q": "q", "down": "down", "up_k": "up_k", "up_v": "up_v", "gate": "gate", "o": "o"}
+NAMES = {"q_down": "q_down", "sink": "sink", "q": "q", "down": "down", "up_k": "up_k", "up_v": "up_v", "gate": "gate", "o": "o"}
 
 
 class LatentAttention(Mixer):
@@ -32,7 +42,9 @@ class LatentAttention(Mixer):
     the norm of the latent, an RMSNorm), gate ("sigmoid" or None), window (None or a count of keys), names (tensor names after the
     prefix for q, down, up_k, up_v, gate, o); optional: keep ("latent", the default: the pages hold the latent where the kernels take
     its size; "heads": they hold every head's keys and values). ``forward(..., scale=)`` with a float32 vector: what is added to the stream is
-    multiplied by it channel by channel."""
+    multiplied by it channel by channel. Further optional: q_latent {rank, norm (PartSpec, an RMSNorm)}: ``q`` then names the matrix behind
+    that latent and ``q_down`` the one in front of it; turned {size, position (PartSpec of a rotary encoding of ``size`` channels)}: ``q`` has head_dim + size
+    rows per head, the turned ones last, and ``down`` latent + size rows; sink (True: a tensor [heads])."""
     capturable = True
     takes_channel_scale = True
 
@@ -40,11 +52,22 @@ class LatentAttention(Mixer):
     def tensors(cls, spec):
         p = spec.params
         n, pre, h, H, dk, dv, r = {**NAMES, **p.get("names", {})}, p["prefix"], p["hidden"], p["heads"], p["head_dim"], p["v_head_dim"], p["latent"]
-        out = {pre + n["q"]: TensorRule((H * dk, h), "fan_in"), pre + n["down"]: TensorRule((r, h), "fan_in")}
+        turned = p["turned"]["size"] if p.get("turned") is not None else 0
+        out = {}
+        if p.get("q_latent") is not None:
+            rank = p["q_latent"]["rank"]
+            out[pre + n["q_down"]] = TensorRule((rank, h), "fan_in")
+            out.update(tensors_of("norm", p["q_latent"]["norm"]))
+            out[pre + n["q"]] = TensorRule((H * (dk + turned), rank), "fan_in")
+        else:
+            out[pre + n["q"]] = TensorRule((H * (dk + turned), h), "fan_in")
+        out[pre + n["down"]] = TensorRule((r + turned, h), "fan_in")
         out.update(tensors_of("norm", p["latent_norm"]))
         out.update({pre + n["up_k"]: TensorRule((H * dk, r), "fan_in"), pre + n["up_v"]: TensorRule((H * dv, r), "fan_in")})
         if p.get("gate") is not None:
             out[pre + n["gate"]] = TensorRule((H * dv, h), "fan_in")
+        if p.get("sink", False):
+            out[pre + n["sink"]] = TensorRule((H,), "unit")
         out[pre + n["o"]] = TensorRule((h, H * dv), "fan_in")
         return out
 
@@ -63,6 +86,10 @@ class LatentAttention(Mixer):
         self.norm = build_part("norm", norm, weights, rt).as_rmsnorm() if norm is not None else None
         if self.norm is None:
             raise AlofaError("unsupported", "the latent's norm is an RMSNorm", f"norm={norm.kind if norm is not None else None}")
+        if p.get("q_latent") is not None or p.get("turned") is not None or p.get("sink", False):
+            self._init_turned(spec, weights, rt)
+            return
+        self.turned_form = False
         self.w_down = rt.matrix(weights[pre + n["down"]])
         # the one head size of the attention kernels: the latent's, widened to a size they are built for
         d = GQAAttention.common_head_size(r, r)
@@ -99,11 +126,91 @@ class LatentAttention(Mixer):
         self.w_o = rt.matrix(w_o)
         self.position = build_part("position", PartSpec("none", {"head_dim": d}), weights, rt)
 
+    def _init_turned(self, spec, weights, rt):
+        """Queries through a latent, a turned part, a sink: see the module's first lines."""
+        p = spec.params
+        n, pre = {**NAMES, **p.get("names", {})}, p["prefix"]
+        H, dk, dv, r = self.heads, self.dk, self.dv, self.r
+        self.turned_form = True
+        if self.gated:
+            raise AlofaError("unsupported", "a gate goes with neither a latent of the queries, a turned part nor a sink")
+        turned = p.get("turned")
+        self.turned = int(turned["size"]) if turned is not None else 0
+        if self.turned < 0 or self.turned % 2:
+            raise AlofaError("invalid_argument", "the turned part is made of pairs", f"size={self.turned}")
+        self.angles = build_part("position", turned["position"], weights, rt) if self.turned else None
+        if self.turned and self.angles.table(1) is None:
+            raise AlofaError("unsupported", "the turned part takes a position encoding that gives a table of angles", f"position={turned['position'].kind}")
+        t = self.turned
+        w_q, w_d, w_o = weights[pre + n["q"]], weights[pre + n["down"]], weights[pre + n["o"]]
+        uk, uv = weights[pre + n["up_k"]].reshape(H, dk, r), weights[pre + n["up_v"]].reshape(H, dv, r)
+        q_latent = p.get("q_latent")
+        self.q_norm = build_part("norm", q_latent["norm"], weights, rt).as_rmsnorm() if q_latent is not None else None
+        if q_latent is not None and self.q_norm is None:
+            raise AlofaError("unsupported", "the latents' norms are RMSNorms", f"norm={q_latent['norm'].kind}")
+        self.q_rank = int(q_latent["rank"]) if q_latent is not None else 0
+        self.sink = rt.vector(weights[pre + n["sink"]]) if p.get("sink", False) else None
+        # the one head size of the attention kernels: turned part and latent side by side, widened to a size they are built for
+        d = GQAAttention.common_head_size(t + r, t + r)
+        if d not in ops.PREFILL_HEAD_DIMS:
+            d = next((s for s in ops.PREFILL_HEAD_DIMS if s >= d), d)
+        self.latent_heads = d <= ops.MAX_HEAD_DIM and p.get("keep", "latent") == "latent"
+        if self.latent_heads:
+            # per head a query [dk | t] as projected goes to [turned t | latent's channels r | zeros] and a result comes out of the latent's channels
+            into = torch.zeros(H, d, dk + t, dtype=uk.dtype, device=uk.device)
+            for i in range(t):
+                into[:, i, dk + i] = 1
+            into[:, t:t + r, :dk] = uk.transpose(1, 2)
+            self.w_query = rt.matrix(into)
+            out_of = torch.zeros(H, dv, d, dtype=uv.dtype, device=uv.device)
+            out_of[:, :, t:t + r] = uv
+            self.w_result = rt.matrix(out_of)
+            self.kv_heads = 1
+        else:
+            # keys [turned pairs' first channels | their second ones | Uk c] and values per head, every head widened to one size with zero rows; the
+            # turned key part reaches every head through an identity in the matrix that makes keys and values of [c | the part as projected]
+            d = GQAAttention.common_head_size(dk + t, dv)
+            if d > ops.MAX_HEAD_DIM:
+                raise AlofaError("unsupported", f"the attention kernels take heads of up to {ops.MAX_HEAD_DIM} channels", f"head_dim={dk} turned={t} v_head_dim={dv}")
+            order = [*range(dk, dk + t, 2), *range(dk + 1, dk + t, 2), *range(dk)]
+            order += range(dk + t, d)
+            w_q = _padded_heads(w_q, H, dk + t, d, order)
+            self.c_width = (r + t + 7) // 8 * 8
+            keys = torch.zeros(H, d, self.c_width, dtype=uk.dtype, device=uk.device)
+            for i in range(t // 2):
+                keys[:, i, r + 2 * i] = 1
+                keys[:, t // 2 + i, r + 2 * i + 1] = 1
+            keys[:, t:t + dk, :r] = uk
+            values = torch.zeros(H, d, self.c_width, dtype=uv.dtype, device=uv.device)
+            values[:, :dv, :r] = uv
+            if keys.dtype is not values.dtype:
+                keys, values = keys.float(), values.float()
+            self.w_kv = rt.matrix(torch.cat([keys.reshape(H * d, -1), values.reshape(H * d, -1)], dim=0))
+            if d != dv:
+                w_o = _padded_heads(w_o.t(), H, dv, d).t()
+            self.kv_heads = H
+        self.d = d
+        self.w_o = rt.matrix(w_o)
+        # what reads the mixer's input, in one product: the queries' latent (or the queries), then the keys' latent with the turned part behind it
+        first = weights[pre + n["q_down"]] if q_latent is not None else w_q
+        rows = first.shape[0] + w_d.shape[0]
+        mats = [first, w_d]
+        if rows % 8:      # (rows of the projection stay 16-byte aligned)
+            mats.append(torch.zeros((8 - rows % 8, self.hidden), dtype=w_d.dtype, device=w_d.device))
+        if len({m.dtype for m in mats}) > 1:
+            mats = [m.float() for m in mats]
+        self.first_width = first.shape[0]
+        self.w_in = rt.matrix(torch.cat(mats, dim=0))
+        self.w_uq = rt.matrix(w_q) if q_latent is not None else None
+
     def cache_need(self):
         return CacheNeed.keys_and_values(self.kv_heads, self.d, self.window)
 
     def prepare(self, n_positions):
-        self.position.table(n_positions)
+        if not self.turned_form:
+            self.position.table(n_positions)
+        elif self.angles is not None:
+            self.angles.table(n_positions)
 
     def _latent(self, ctx, x, out, pad, copies, down=None):
         """The step's latents, normed, ``copies`` times side by side in ``out`` (each widened to ``pad`` channels with zeros)."""
@@ -122,7 +229,9 @@ class LatentAttention(Mixer):
         T, exact, H, d = residual.shape[0], self.rt.exact, self.heads, self.d
         attn = ctx.scratch("attn", (T, H * d), self.rt.dtype)
         down = None
-        if self.latent_heads:
+        if self.turned_form:
+            heads_out = self._forward_turned(ctx, where, x, residual, attn, norm)
+        elif self.latent_heads:
             if self.w_in is not None:
                 qg = ctx.scratch("latent_in", (T, self.w_in.shape[0]), self.rt.dtype)
                 if norm is not None:
@@ -162,6 +271,46 @@ class LatentAttention(Mixer):
             ops.gemm(residual, heads_out, self.w_o, add_to_out=True, exact=exact)
         else:
             ops.gemm_channel_scaled(residual, heads_out, self.w_o, scale, ctx.scratch("sub_out", tuple(residual.shape), torch.float32), exact, then_norm=then)
+
+
+    def _forward_turned(self, ctx, where, x, residual, attn, norm):
+        """The heads' outputs side by side, for the form with a latent of the queries, a turned part or a sink."""
+        T, exact, H, d, t = residual.shape[0], self.rt.exact, self.heads, self.d, self.turned
+        kv = ctx.kv(where)
+        proj = ctx.scratch("latent_in", (T, self.w_in.shape[0]), self.rt.dtype)
+        if norm is not None:
+            ops.gemm(proj, residual, self.w_in, norm=norm.as_rmsnorm())
+        else:
+            ops.gemm(proj, x, self.w_in, exact=exact)
+        table = self.angles.table(ctx.n_positions) if t else None
+        queries, q = None, proj[:, :self.first_width]
+        if self.q_rank:
+            cq = ctx.scratch("latent_cq", (T, self.q_rank), self.rt.dtype)
+            queries = (0, *self.q_norm, cq)
+        keys = (self.first_width, *self.norm)
+        q_size = self.dk + t if self.latent_heads else d
+        if self.latent_heads:
+            ops.latent_rows(proj, queries, keys, t, ctx.positions, table, pages=(kv.slots, kv.k, kv.v), exact=exact)
+            if self.q_rank:
+                q = ctx.scratch("latent_q", (T, H * q_size), self.rt.dtype)
+                ops.gemm(q, cq, self.w_uq, exact=exact)
+            ql = ctx.scratch("qkv", (T, H * d), self.rt.dtype)
+            ops.head_project(ql, q, self.w_query, exact, turn=(ctx.positions, *table) if t else None)
+            attend_pages(ctx, kv, ql, attn, H, 1, d, self.window, self.scale, self.rt, sink=self.sink)
+            heads_out = ctx.scratch("latent_out", (T, H * self.dv), self.rt.dtype)
+            ops.head_project(heads_out, attn, self.w_result, exact)
+            return heads_out
+        qkv = ctx.scratch("qkv", (T, 3 * H * d), self.rt.dtype)
+        c = ctx.scratch("latent", (T, self.c_width), self.rt.dtype)
+        ops.latent_rows(proj, queries, keys, t, rows=c, exact=exact)
+        if self.q_rank:
+            ops.gemm(qkv[:, :H * d], cq, self.w_uq, exact=exact)
+        else:
+            qkv[:, :H * d].copy_(q)
+        ops.gemm(qkv[:, H * d:], c, self.w_kv, exact=exact)
+        ops.norm_turn_write(qkv, ctx.positions, table, H, H, d, d, ops.NORM_NONE, None, None, 0.0, exact, kv.slots, kv.k, kv.v)
+        attend_pages(ctx, kv, qkv[:, :H * d], attn, H, H, d, self.window, self.scale, self.rt, sink=self.sink)
+        return attn
 
 
 register_part("mixer", "latent_attention", LatentAttention)

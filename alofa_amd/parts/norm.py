@@ -5,6 +5,8 @@ scale, eps sits inside the root, no 1+w, no bias
 (src/alofa/kernels/cpu/scalar.mojo:93-129)."""
 from __future__ import annotations
 
+import torch
+
 from .. import ops
 from ..weights.loader import TensorRule
 from .base import Norm, register_part
@@ -59,3 +61,19 @@ class LayerNorm(Norm):
 
 
 register_part("norm", "layernorm", LayerNorm)
+
+
+class IdentityNorm(Norm):
+    """No norm: the rows as they are, rounded to the reader's dtype. It stands where a sub-layer reads the stream itself."""
+    identity = True
+
+    def forward(self, out, x, rows=None):
+        if rows is not None:
+            x = x.index_select(0, rows.long())
+        if out.dtype is torch.bfloat16:
+            ops.to_bfloat16(out, x)
+        else:
+            out.copy_(x)
+
+
+register_part("norm", "identity", IdentityNorm)

@@ -3,7 +3,7 @@ every token decays and adds to, S_t = diag(w_t) S_(t-1) + k_t v_t^T, and reads o
 where the decay comes from and in the order of read-out and update; the recurrence itself is one kernel
 (``ops.linear_recurrence``), and so are the norm of every head's read-out with the gate (``ops.headnorm_gate``).
 
-retention       w = a constant per head; rotary positions on q and k; k scaled by dk^(-1/2); o_t = S_t^T q_t;
+retention       w = a constant per head; rotary positions on q and k, or none; k scaled by dk^(-1/2); o_t = S_t^T q_t;
                 o / rms(o) per head, times silu(gate), output projection.
 gated_linear    w_t = sigmoid(z_t)^(1/tau) per key channel, z = W_a2 (W_a1 x) + b; q scaled by dk^(-1/2); o_t = S_t^T q_t;
                 RMS norm per head with a weight shared by the heads, times silu(gate), output projection.
@@ -76,7 +76,7 @@ class RecurrentMixer(Mixer):
 
 class Retention(RecurrentMixer):
     """params: prefix, hidden, heads, key_dim, value_dim, decay (one per head), position (PartSpec, for heads of
-    key_dim), eps. Tensors: prefix + q, k, v, g, o."""
+    key_dim, or None: queries and keys as projected), eps. Tensors: prefix + q, k, v, g, o."""
 
     @classmethod
     def tensors(cls, spec):
@@ -94,26 +94,29 @@ class Retention(RecurrentMixer):
         self.decay = torch.tensor(decay, dtype=torch.float32, device=rt.device)
         self.k_scale = float(self.dk) ** -0.5
         # the rotation pairs channels, so a head of odd size gets one more key channel whose q and k are zero (it adds nothing to any product)
-        position, true_dk = p["position"], self.dk
-        if self.dk % 2:
+        position, true_dk = p.get("position"), self.dk
+        if position is not None and self.dk % 2:
             self.dk += 1
             position = part_class("position", position.kind).for_head(position, self.dk)
-        self.position = build_part("position", position, weights, rt)
-        order = self.position.channel_order()
+        self.position = build_part("position", position, weights, rt) if position is not None else None
+        order = self.position.channel_order() if self.position is not None else None
         self.w_in = _stacked(rt, [_padded_heads(weights[pre + "q"], self.heads, true_dk, self.dk, order), _padded_heads(weights[pre + "k"], self.heads, true_dk, self.dk, order),
                                   weights[pre + "v"], weights[pre + "g"]])
         self.w_o = rt.matrix(weights[pre + "o"])
-        self.capturable = self.position.table(1) is not None
+        self.capturable = self.position is None or self.position.table(1) is not None
 
     def prepare(self, n_positions):
-        self.position.table(n_positions)
+        if self.position is not None:
+            self.position.table(n_positions)
 
     def forward(self, ctx, where, x, residual, out=None):
         T, kd, vd = x.shape[0], self.heads * self.dk, self.heads * self.dv
         proj = ctx.scratch("recurrent_proj", (T, 2 * kd + 2 * vd), self.rt.dtype)
         ops.gemm(proj, x, self.w_in, exact=self.rt.exact)
-        table = self.position.table(ctx.n_positions)
-        if table is None:
+        table = self.position.table(ctx.n_positions) if self.position is not None else None
+        if self.position is None:
+            pass
+        elif table is None:
             self.position.apply(ctx, proj[:, :kd].unflatten(1, (self.heads, self.dk)), proj[:, kd:2 * kd].unflatten(1, (self.heads, self.dk)))
         else:      # queries and keys alike: 2 * heads heads to rotate, nothing to write to pages
             ops.rope_kv_write(proj, table[0], table[1], ctx.positions, 2 * self.heads, 0, self.dk)
