@@ -28,7 +28,8 @@ context of 4,096) through the same engine and print their own line;
 ``--config 1.5b``, ``3b`` and ``14b`` run the continuous batch at those sizes.
 ``--sweep batch`` and ``--sweep context`` take any of the configurations.
 
-``--design tugalix``, ``--design rerupel``, ``--design retotar`` and ``--design ludelorn`` measure another design beside Qwen2 (Retotar and Ludelorn: beside Tugalix) at equal sizes: prefill of one prompt and
+``--design tugalix``, ``--design rerupel``, ``--design retotar``, ``--design ludelorn`` and ``--design lalepel`` measure another design beside Qwen2 (Retotar and Ludelorn: beside
+Tugalix; Lalepel: beside Rerupel) at equal sizes: prefill of one prompt and
 decode steps at batch 1, 8 and 64, at a few widths (``--sizes``), a line per point and model."""
 import argparse
 import json
@@ -567,8 +568,24 @@ def ludelorn_sizes(width, heads, dim, ff, layers, vocab=32000):
     return lud, tugalix_sizes(width, heads, dim, ff, layers, vocab)[0]
 
 
-DESIGN_MODELS = {"tugalix": tugalix_sizes, "rerupel": rerupel_sizes, "retotar": retotar_sizes, "ludelorn": ludelorn_sizes}
-DESIGN_BESIDE = {"retotar": "tugalix", "ludelorn": "tugalix"}      # the model a design is measured beside, where that is not Qwen2
+def lalepel_sizes(width, heads, dim, ff, layers, vocab=32000):
+    """A Lalepel model of ``layers`` layers in the order latent attention (a window of 1,024 keys, latents that make one head of twice a head's size
+    with the turned part of half a head's), retention, latent attention, latent attention, the first with a dense feed-forward, the others with
+    sixteen experts of which a token takes four and one that every token takes, and beside it the closest other design, Rerupel (attention over
+    latents, the same experts with a gate matrix), at equal width, heads, layers and feed-forward."""
+    expert = max(64, ff // 8 // 64 * 64)
+    latent = {"heads": heads, "dim": dim, "rot_dim": dim // 2, "vdim": dim, "q_rank": 3 * width // 8 // 64 * 64 or 64, "kv_rank": 3 * dim // 2, "scale": (1.5 * dim) ** -0.5,
+              "rot": {"dims": dim // 2, "base": 250000.0, "scaling": {"factor": 4.0, "original": 4096, "fast": 16.0, "slow": 2.0}}, "mask": {"size": 1024}}
+    retention = {"heads": heads, "dim": dim, "vdim": dim, "decay": [1.0 - 2.0 ** (-5 - h % 8) for h in range(heads)]}
+    moe = {"kind": "moe", "router": {"experts": 16, "top": 4}, "expert": {"ff": expert}, "shared": {"ff": expert}}
+    lal = {"architecture": "Lalepel", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+           "layers": [{"type": "retention" if i % 4 == 1 else "latent_attention", "mixer": retention if i % 4 == 1 else latent,
+                       "mlp": {"kind": "dense", "ff": ff} if i == 0 else moe} for i in range(layers)]}
+    return lal, rerupel_sizes(width, heads, dim, ff, layers, vocab)[0]
+
+
+DESIGN_MODELS = {"tugalix": tugalix_sizes, "rerupel": rerupel_sizes, "retotar": retotar_sizes, "ludelorn": ludelorn_sizes, "lalepel": lalepel_sizes}
+DESIGN_BESIDE = {"retotar": "tugalix", "ludelorn": "tugalix", "lalepel": "rerupel"}      # the model a design is measured beside, where that is not Qwen2
 DESIGN_SIZES = {"256": (256, 4, 64, 1024, 4), "1k": (1024, 16, 64, 4096, 8), "2k": (2048, 16, 128, 8192, 8), "4k": (4096, 32, 128, 14336, 4)}
 DESIGN_DEFAULT = ("1k", "2k", "4k")      # ("256": a small one, for a quick look)
 
@@ -620,7 +637,7 @@ def main():
     ap.add_argument("--serve", action="store_true", help="the continuous batch of 64 requests (prompts of 128..2,048 tokens, 256 new tokens, chunks of 512) at the sizes of --config")
     ap.add_argument("--batches", default=None, help="with --sweep batch: these batch sizes only (comma-separated), e.g. to profile one point")
     ap.add_argument("--sweep", choices=["batch", "context"], default=None, help="decode steps over batch sizes or over contexts, a line per point (the sizes of --config)")
-    ap.add_argument("--design", choices=sorted(DESIGN_MODELS), default=None, help="prefill and decode of this design beside Qwen2 at equal sizes (--sizes), a line per point")
+    ap.add_argument("--design", choices=sorted(DESIGN_MODELS), default=None, help="prefill and decode of this design beside the closest one at equal sizes (--sizes), a line per point")
     ap.add_argument("--sizes", default=None, help=f"with --design: which of {','.join(DESIGN_SIZES)} (comma-separated; default {','.join(DESIGN_DEFAULT)})")
     ap.add_argument("--only", choices=sorted(DESIGN_MODELS) + ["qwen2"], default=None, help="with --design: this model alone (for profiling)")
     ap.add_argument("--prompt-tokens", type=int, default=2048, help="with --design: tokens of the prefill point's prompt")

@@ -140,3 +140,17 @@ def ludelorn_dirs(tmp_path_factory):
         write_random_model(cfg, d, seed=5000 + ord(name))
         out[name] = d
     return out
+
+
+@pytest.fixture(scope="session")
+def lalepel_dirs(tmp_path_factory):
+    """Model folders of the small Lalepel configurations, written by the engine's random-weights mode."""
+    from alofa_amd.weights import write_random_model
+    from lalepel_cases import LALEPEL
+    out = {}
+    for name, cfg in LALEPEL.items():
+        d = tmp_path_factory.mktemp(f"lalepel_{name}")
+        # (of a few seeds the ones with which no router's call is changed by rounding alone: a changed call moves every later position, through states and windows)
+        write_random_model(cfg, d, seed={"A": 5, "B": 4, "C": 6067, "D": 6, "E": 5}[name])
+        out[name] = d
+    return out

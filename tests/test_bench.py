@@ -51,7 +51,7 @@ def test_the_default_run_prints_one_line_with_the_agreed_keys():
 
 
 @pytest.mark.gpu
-@pytest.mark.parametrize("design,beside", [("tugalix", "qwen2"), ("rerupel", "qwen2"), ("ludelorn", "tugalix")])
+@pytest.mark.parametrize("design,beside", [("tugalix", "qwen2"), ("rerupel", "qwen2"), ("ludelorn", "tugalix"), ("lalepel", "rerupel")])
 def test_another_design_beside_the_closest_one_prints_a_line_per_point(design, beside):
     rc, out, err = run_bench("--design", design, "--sizes", "256", "--prompt-tokens", "256", "--batches", "1,4", "--steps", "6", "--warmup", "2")
     assert rc == 0, err[-2000:]
