@@ -50,7 +50,7 @@ __device__ __forceinline__ void put_out(bf16_t* out, float* out32, int64_t at, f
   if (out32) out32[at] = v;
   else store_f32(out + at, v);
 }
-constexpr int kHeadsPerBlock = 16;   // query heads of one key head that a block serves (the columns of a tile)
+constexpr int kHeadsPerBlock = 16;   // query heads of one key head that a block serves at most (the columns of a tile)
 
 // What the kernel needs to take the new token's projections as they come out of the fused query / key / value
 // product (kRope): q then points to rows [queries | keys | values] that are not yet rotated, one token per
@@ -85,7 +85,7 @@ __device__ __forceinline__ Pair8 rotate8(uint4 lo, uint4 hi, float4 c_lo, float4
   return Pair8{make_uint4(ra[0], ra[1], ra[2], ra[3]), make_uint4(rb[0], rb[1], rb[2], rb[3])};
 }
 
-// DT = d / 16; NW: waves per block. blockIdx.y = key head * chunks + chunk of up to 16 heads of its group.
+// DT = d / 16; NW: waves per block. blockIdx.y = key head * chunks + chunk of up to `block_heads` (<= 16) heads of its group.
 // kSplit: a weight enters the second product as two bfloat16 numbers, its rounding and what the rounding took away: sixteen bits of every weight count.
 template <int DT, int NW, bool kRope, bool kSplit = false>
 __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
@@ -94,7 +94,7 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
     const int32_t* __restrict__ block_table, int max_blocks, const int32_t* __restrict__ req_of_token,
     const int32_t* __restrict__ positions, const int32_t* __restrict__ rows, int heads, int kv_heads,
     int bs_shift, int window, float scale, RopeArgs rope, int* __restrict__ counters, int v_head, float* __restrict__ out32, int value_heads, int64_t plane,
-    const float* __restrict__ sink) {
+    const float* __restrict__ sink, int block_heads) {
   static_assert(!kRope || DT % 4 == 0, "the rotation needs a channel and its partner in the same lane: d a multiple of 64");
   constexpr int d = DT * 16;
   constexpr int DS = (d + 31) / 32;            // steps of 32 along d in the first product
@@ -102,7 +102,7 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
   __shared__ __attribute__((aligned(16))) float state[NW][kHeadsPerBlock][d + 4];
   __shared__ int last_block;
   const int group = heads / kv_heads;
-  const int chunks = (group + kHeadsPerBlock - 1) / kHeadsPerBlock;
+  const int chunks = (group + block_heads - 1) / block_heads;
   // the tokens served are rows[0..gridDim.x) of the packed batch, or all of it
   // (value_heads > 0: blockIdx.x counts (token, value head) pairs: every value head in turn serves all key heads, and its results go to a plane of their own)
   const int served = value_heads > 0 ? blockIdx.x / value_heads : blockIdx.x;
@@ -111,7 +111,7 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
     out32 += static_cast<int64_t>(v_head) * plane;
   }
   const int t = rows ? rows[served] : served;
-  const int hk = blockIdx.y / chunks, h0 = (blockIdx.y % chunks) * kHeadsPerBlock;
+  const int hk = blockIdx.y / chunks, h0 = (blockIdx.y % chunks) * block_heads;
   const int hv = v_head >= 0 ? v_head : hk;      // the value head whose values the weights meet (v_head >= 0: one for all key heads)
   const int wave = threadIdx.x / 64, lane = threadIdx.x % 64;
   const int c16 = lane % 16, g = lane / 16;
@@ -131,7 +131,7 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
   const int bs_mask = (1 << bs_shift) - 1;
 
   // this lane's head and its fragments of Q (heads beyond the group: zeros)
-  const bool head_ok = h0 + c16 < group;
+  const bool head_ok = c16 < block_heads && h0 + c16 < group;
   const int head = hk * group + (head_ok ? h0 + c16 : 0);
   bf16x8 qf[DS];
 #pragma unroll
@@ -385,7 +385,7 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
   __syncthreads();
 
   // the waves' states are combined in wave order; thread x takes channel x % d of head x / d
-  for (int x = threadIdx.x; x < kHeadsPerBlock * d; x += 64 * NW) {
+  for (int x = threadIdx.x; x < block_heads * d; x += 64 * NW) {
     const int i = x / d, c = x % d;
     if (h0 + i >= group) break;
     const int h = hk * group + h0 + i;
@@ -435,7 +435,7 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
   __syncthreads();
   if (!last_block) return;
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup");
-  for (int x = threadIdx.x; x < kHeadsPerBlock * d; x += 64 * NW) {
+  for (int x = threadIdx.x; x < block_heads * d; x += 64 * NW) {
     const int i = x / d, c = x % d;
     if (h0 + i >= group) break;
     const int h = hk * group + h0 + i;
@@ -552,10 +552,10 @@ extern "C" int64_t alofa_attention_decode_scratch(int tokens, int heads, int d, 
 
 // Whether the parts of these sizes fit the library's workspace (their states and a counter per (token, key head,
 // chunk of heads)), so that the last block of a (token, key head) can combine them and no second kernel is needed.
-extern "C" int alofa_attention_decode_can_hand_over(int tokens, int heads, int kv_heads, int d, int n_splits) {
-  if (tokens <= 0 || heads <= 0 || kv_heads <= 0 || heads % kv_heads != 0 || n_splits <= 1) return 0;
+extern "C" int alofa_attention_decode_can_hand_over(int tokens, int heads, int kv_heads, int d, int n_splits, int block_heads) {
+  if (tokens <= 0 || heads <= 0 || kv_heads <= 0 || heads % kv_heads != 0 || n_splits <= 1 || block_heads < 1 || block_heads > kHeadsPerBlock) return 0;
   const Workspace& ws = workspace();
-  const int64_t counters = static_cast<int64_t>(tokens) * kv_heads * ((heads / kv_heads + kHeadsPerBlock - 1) / kHeadsPerBlock);
+  const int64_t counters = static_cast<int64_t>(tokens) * kv_heads * ((heads / kv_heads + block_heads - 1) / block_heads);
   return ws.tiles != nullptr && counters <= ws.n_counters && alofa_attention_decode_scratch(tokens, heads, d, n_splits) <= ws.tile_floats;
 }
 
@@ -565,13 +565,14 @@ extern "C" int alofa_attention_decode_can_hand_over(int tokens, int heads, int k
 // workspace (alofa_attention_decode_can_hand_over must hold; `partial` is not used), not in `partial` and a second kernel.
 // v_head >= 0: every query head's weights meet the values of that one value head (its keys stay its own key head's);
 // out32: the results go there unrounded, as float rows of `out`'s shape and stride, and `out` is not written.
-// sink: a number per query head whose exponential joins the sum of its rows' weights (null: none).
+// sink: a number per query head whose exponential joins the sum of its rows' weights (null: none). block_heads: how many heads of a key head a block serves.
 extern "C" int alofa_attention_decode_v(void* out, int64_t out_stride, float* partial, const void* q, int64_t q_stride,
                                         void* k_cache, void* v_cache, const int32_t* block_table,
                                         int max_blocks, const int32_t* req_of_token, const int32_t* positions,
                                         const int32_t* rows, int tokens, int heads, int kv_heads, int d, int block_size, int window,
                                         float scale, int n_splits, const float* cos_t, const float* sin_t, const int64_t* slots,
-                                        int hand_over, int v_head, float* out32, int split, int value_heads, int64_t plane, const float* sink, hipStream_t stream) {
+                                        int hand_over, int v_head, float* out32, int split, int value_heads, int64_t plane, const float* sink, int block_heads, hipStream_t stream) {
+  ALOFA_REQUIRE(block_heads >= 1 && block_heads <= kHeadsPerBlock, "attention_decode: a block serves 1 to %d heads (%d)", kHeadsPerBlock, block_heads);
   ALOFA_REQUIRE(!split || !cos_t, "attention_decode: split weights and the rotary variant do not go together");
   // value_heads > 0: all of them in one launch, value head c's results in out32 + c * plane; `tokens` then counts (token, value head) pairs
   // wherever it sizes scratch, workspace and grid
@@ -588,7 +589,7 @@ extern "C" int alofa_attention_decode_v(void* out, int64_t out_stride, float* pa
   ALOFA_REQUIRE(n_splits >= 1 && n_splits <= kMaxSplits && (n_splits == 1 || partial || hand_over), "attention_decode: n_splits=%d (1..%d) needs scratch when above 1", n_splits, kMaxSplits);
   int* counters = nullptr;
   if (hand_over && n_splits > 1) {
-    ALOFA_REQUIRE(alofa_attention_decode_can_hand_over(tokens, heads, kv_heads, d, n_splits),
+    ALOFA_REQUIRE(alofa_attention_decode_can_hand_over(tokens, heads, kv_heads, d, n_splits, block_heads),
                   "attention_decode: the states of %d parts of %d tokens do not fit the workspace", n_splits, tokens);
     partial = workspace().tiles;
     counters = workspace().counters;
@@ -601,16 +602,16 @@ extern "C" int alofa_attention_decode_v(void* out, int64_t out_stride, float* pa
   ALOFA_REQUIRE(!fused || (reinterpret_cast<uintptr_t>(cos_t) % 16 == 0 && reinterpret_cast<uintptr_t>(sin_t) % 16 == 0), "attention_decode: cos and sin must be 16-byte aligned");
   const int group = heads / kv_heads;
   const RopeArgs rope{cos_t, sin_t, slots};
-  dim3 grid(tokens, kv_heads * ((group + kHeadsPerBlock - 1) / kHeadsPerBlock), n_splits);
+  dim3 grid(tokens, kv_heads * ((group + block_heads - 1) / block_heads), n_splits);
 #define ALOFA_DECODE(DT, NW, ROPE)                                                                                        \
   if (split && !ROPE) attention_decode_kernel<DT, NW, false, true><<<grid, 64 * NW, 0, stream>>>(                         \
       static_cast<bf16_t*>(out), out_stride, partial, static_cast<const bf16_t*>(q), q_stride,                            \
       static_cast<bf16_t*>(k_cache), static_cast<bf16_t*>(v_cache), block_table, max_blocks, req_of_token,                \
-      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane, sink);       \
+      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane, sink, block_heads);       \
   else attention_decode_kernel<DT, NW, ROPE><<<grid, 64 * NW, 0, stream>>>(                                                    \
       static_cast<bf16_t*>(out), out_stride, partial, static_cast<const bf16_t*>(q), q_stride,                            \
       static_cast<bf16_t*>(k_cache), static_cast<bf16_t*>(v_cache), block_table, max_blocks, req_of_token,                \
-      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane, sink)
+      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane, sink, block_heads)
   if (fused) {
     switch (d / 64) {
       case 1: ALOFA_DECODE(4, 8, true); break;
@@ -655,5 +656,5 @@ extern "C" int alofa_attention_decode(void* out, int64_t out_stride, float* part
                                       float scale, int n_splits, const float* cos_t, const float* sin_t, const int64_t* slots,
                                       int hand_over, hipStream_t stream) {
   return alofa_attention_decode_v(out, out_stride, partial, q, q_stride, k_cache, v_cache, block_table, max_blocks, req_of_token, positions, rows, tokens,
-                                  heads, kv_heads, d, block_size, window, scale, n_splits, cos_t, sin_t, slots, hand_over, -1, nullptr, 0, 0, 0, nullptr, stream);
+                                  heads, kv_heads, d, block_size, window, scale, n_splits, cos_t, sin_t, slots, hand_over, -1, nullptr, 0, 0, 0, nullptr, kHeadsPerBlock, stream);
 }

@@ -414,62 +414,102 @@ __global__ void __launch_bounds__(256) experts_sum_kernel(float* __restrict__ re
 }
 
 // ---- residual[t, :] += rmsnorm(sum of row t's slots) * w, rows[t, :] = the stream's new row in the activation type: the sum above with the
-// norm behind the mixture and the sum into the stream (a block per row; the sums wait in registers, or, in rows wider than a block keeps,
-// in `wide` [T, width]) ----
-template <typename TO>
-__global__ void __launch_bounds__(256) experts_sum_norm_kernel(float* __restrict__ residual, const float* __restrict__ y, const int32_t* __restrict__ slot_of,
-                                                               const float* __restrict__ w, float eps, TO* __restrict__ rows, float* __restrict__ wide, int T, int width,
-                                                               int top, int shared) {
-  __shared__ float scratch[4];
-  constexpr int kOwn = 16;      // values a thread keeps: rows up to 4,096 wide
+// norm behind the mixture and the sum into the stream (a block per row; a thread keeps the sums of its values). kVec values of a row a thread and
+// step: 4 where rows are 16-byte aligned, else 1; up to kAhead slots' values are on their way together. Rows wider than kOwn * kVec * kThreads
+// values keep the rest of their sums in `wide` [T, width]. ----
+template <int kVec>
+struct RowVec;
+template <>
+struct RowVec<4> {
+  float4 v;
+};
+template <>
+struct RowVec<1> {
+  float v;
+};
+template <int kVec>
+__device__ __forceinline__ void load_row(float (&out)[kVec], const float* p) {
+  const RowVec<kVec> x = *reinterpret_cast<const RowVec<kVec>*>(p);
+  if constexpr (kVec == 4) out[0] = x.v.x, out[1] = x.v.y, out[2] = x.v.z, out[3] = x.v.w;
+  else out[0] = x.v;
+}
+
+template <int kThreads, int kVec>
+__global__ void __launch_bounds__(kThreads) experts_sum_norm_kernel(float* __restrict__ residual, const float* __restrict__ y, const int32_t* __restrict__ slot_of,
+                                                                    const float* __restrict__ w, float eps, bf16_t* __restrict__ rows, float* __restrict__ wide, int T,
+                                                                    int width, int top, int shared) {
+  __shared__ float scratch[kThreads / kWave];
+  constexpr int kOwn = 2, kAhead = 5, kStep = kVec * kThreads;
   const int t = blockIdx.x;
   const int64_t at = static_cast<int64_t>(t) * width;
-  float own[kOwn];
-#pragma unroll
-  for (int i = 0; i < kOwn; ++i) own[i] = 0.f;
-  float ss = 0.f;
   const int parts = top + (shared ? 1 : 0);
-  if (width <= kOwn * 256) {      // (uniform over the launch)
-    for (int k = 0; k < parts; ++k) {
-      const int slot = k < top ? slot_of[t * top + k] : slot_of[T * top + t];
-      if (slot < 0) continue;      // (a choice without a slot)
-      const float* src = y + static_cast<int64_t>(slot) * width;
+  auto slot_at = [&](int k) { return k < top ? slot_of[t * top + k] : slot_of[T * top + t]; };
+  // the sum over the slots of kVec values from column c on, slots in ascending order
+  auto sum_at = [&](int c, float (&sum)[kVec]) {
 #pragma unroll
-      for (int i = 0; i < kOwn; ++i) {
-        const int c = threadIdx.x + i * 256;
-        if (c < width) own[i] += src[c];
+    for (int e = 0; e < kVec; ++e) sum[e] = 0.f;
+    for (int k0 = 0; k0 < parts; k0 += kAhead) {
+      float part[kAhead][kVec];
+      bool ok[kAhead];
+#pragma unroll
+      for (int a = 0; a < kAhead; ++a) {      // (every load is issued, from slot 0 where there is none to read)
+        const int slot = slot_at(k0 + a < parts ? k0 + a : parts - 1);
+        ok[a] = k0 + a < parts && slot >= 0;
+        load_row<kVec>(part[a], y + static_cast<int64_t>(ok[a] ? slot : 0) * width + c);
       }
+#pragma unroll
+      for (int a = 0; a < kAhead; ++a)
+#pragma unroll
+        for (int e = 0; e < kVec; ++e) sum[e] += ok[a] ? part[a][e] : 0.f;
     }
+  };
+  float own[kOwn][kVec], old[kOwn][kVec], weight[kOwn][kVec];
+  float ss = 0.f;
 #pragma unroll
-    for (int i = 0; i < kOwn; ++i) ss += own[i] * own[i];
-  } else {
-    for (int c = threadIdx.x; c < width; c += 256) {
-      float sum = 0.f;
-      for (int k = 0; k < parts; ++k) {
-        const int slot = k < top ? slot_of[t * top + k] : slot_of[T * top + t];
-        if (slot >= 0) sum += y[static_cast<int64_t>(slot) * width + c];
-      }
-      wide[at + c] = sum;      // (read back by the thread that wrote it)
-      ss += sum * sum;
+  for (int i = 0; i < kOwn; ++i) {
+    const int c = threadIdx.x * kVec + i * kStep;
+    if (c < width) {
+      load_row<kVec>(old[i], residual + at + c);
+      load_row<kVec>(weight[i], w + c);
+      sum_at(c, own[i]);
+#pragma unroll
+      for (int e = 0; e < kVec; ++e) ss += own[i][e] * own[i][e];
     }
   }
-  const float inv = 1.f / sqrtf(block_sum<float, 256>(ss, scratch) / static_cast<float>(width) + eps);
-  if (width <= kOwn * 256) {
+  for (int c = threadIdx.x * kVec + kOwn * kStep; c < width; c += kStep) {
+    float sum[kVec];
+    sum_at(c, sum);
 #pragma unroll
-    for (int i = 0; i < kOwn; ++i) {
-      const int c = threadIdx.x + i * 256;
-      if (c < width) {
-        const float now = residual[at + c] + own[i] * inv * w[c];
-        residual[at + c] = now;
-        if (rows) store_f32(rows + at + c, now);
-      }
+    for (int e = 0; e < kVec; ++e) {
+      wide[at + c + e] = sum[e];      // (read back by the thread that wrote it)
+      ss += sum[e] * sum[e];
     }
-  } else {
-    for (int c = threadIdx.x; c < width; c += 256) {
-      const float now = residual[at + c] + wide[at + c] * inv * w[c];
-      residual[at + c] = now;
-      if (rows) store_f32(rows + at + c, now);
+  }
+  const float inv = 1.f / sqrtf(block_sum<float, kThreads>(ss, scratch) / static_cast<float>(width) + eps);
+  auto put = [&](int c, const float (&now)[kVec]) {
+    if constexpr (kVec == 4) {
+      *reinterpret_cast<float4*>(residual + at + c) = make_float4(now[0], now[1], now[2], now[3]);
+      if (rows) *reinterpret_cast<uint2*>(rows + at + c) = uint2{pack_bf16x2(now[0], now[1]), pack_bf16x2(now[2], now[3])};
+    } else {
+      residual[at + c] = now[0];
+      if (rows) rows[at + c] = f32_to_bf16(now[0]);
     }
+  };
+#pragma unroll
+  for (int i = 0; i < kOwn; ++i) {
+    const int c = threadIdx.x * kVec + i * kStep;
+    if (c < width) {
+      float now[kVec];
+#pragma unroll
+      for (int e = 0; e < kVec; ++e) now[e] = old[i][e] + own[i][e] * inv * weight[i][e];
+      put(c, now);
+    }
+  }
+  for (int c = threadIdx.x * kVec + kOwn * kStep; c < width; c += kStep) {
+    float now[kVec];
+#pragma unroll
+    for (int e = 0; e < kVec; ++e) now[e] = residual[at + c + e] + wide[at + c + e] * inv * w[c + e];
+    put(c, now);
   }
 }
 
@@ -557,11 +597,19 @@ extern "C" int alofa_experts_sum(float* residual, const float* y, const int32_t*
   return check_launch("experts_sum");
 }
 
+// wide: room (float [T, width]) for the sums of rows of more values than a block keeps.
+extern "C" int alofa_experts_sum_norm_room(int width) { return width % 4 == 0 ? width > 4096 : width > 1024; }
+
 extern "C" int alofa_experts_sum_norm(float* residual, const float* y, const int32_t* slot_of, const float* w, float eps, void* rows, float* wide, int T, int width, int top,
                                       int shared, hipStream_t stream) {
   ALOFA_REQUIRE(T >= 0 && width > 0 && top > 0 && w && eps > 0.f, "experts_sum_norm: bad arguments");
-  ALOFA_REQUIRE(width <= 4096 || wide, "experts_sum_norm: rows of %d values need room for their sums", width);
+  ALOFA_REQUIRE(!alofa_experts_sum_norm_room(width) || wide, "experts_sum_norm: rows of %d values need room for their sums", width);
+  ALOFA_REQUIRE(width % 4 != 0 || (reinterpret_cast<uintptr_t>(residual) % 16 == 0 && reinterpret_cast<uintptr_t>(y) % 16 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0 &&
+                                   reinterpret_cast<uintptr_t>(rows) % 8 == 0 && reinterpret_cast<uintptr_t>(wide) % 16 == 0), "experts_sum_norm: operands must be 16-byte aligned");
   if (T == 0) return 0;
-  experts_sum_norm_kernel<bf16_t><<<static_cast<unsigned>(T), 256, 0, stream>>>(residual, y, slot_of, w, eps, static_cast<bf16_t*>(rows), wide, T, width, top, shared);
+  bf16_t* left = static_cast<bf16_t*>(rows);
+  const unsigned grid = static_cast<unsigned>(T);
+  if (width % 4 == 0) experts_sum_norm_kernel<512, 4><<<grid, 512, 0, stream>>>(residual, y, slot_of, w, eps, left, wide, T, width, top, shared);
+  else experts_sum_norm_kernel<512, 1><<<grid, 512, 0, stream>>>(residual, y, slot_of, w, eps, left, wide, T, width, top, shared);
   return check_launch("experts_sum_norm");
 }

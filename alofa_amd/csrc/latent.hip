@@ -30,31 +30,33 @@ struct LatentRows {
   int row_width;
 };
 
-// One wavefront per (row, latent): the keys' latents are the first `tokens` units, the queries' follow.
+// A block of four wavefronts per (row, latent): the keys' latents are the first `tokens` blocks, the queries' follow.
 template <typename T, typename Acc>
 __global__ void __launch_bounds__(256) latent_rows_kernel(const T* __restrict__ x, T* __restrict__ cq, T* __restrict__ k_cache, T* __restrict__ v_cache,
                                                           T* __restrict__ rows_out, int tokens, LatentRows a) {
-  const int64_t unit = static_cast<int64_t>(blockIdx.x) * 4 + threadIdx.x / kWave;
-  const int lane = threadIdx.x % kWave;
-  if (unit >= static_cast<int64_t>(tokens) * (a.q_rank > 0 ? 2 : 1)) return;
-  const bool of_keys = unit < tokens;
-  const int t = static_cast<int>(of_keys ? unit : unit - tokens);
+  __shared__ Acc scratch[4];
+  const bool of_keys = static_cast<int>(blockIdx.x) < tokens;
+  const int t = of_keys ? blockIdx.x : blockIdx.x - tokens, tid = threadIdx.x;
   const T* src = x + static_cast<int64_t>(t) * a.x_stride + (of_keys ? a.kv_at : a.q_at);
   const int width = of_keys ? a.r : a.q_rank;
-  constexpr int kOwn = 8;      // values a lane keeps (latents of up to 512 values; longer ones are read again)
-  float own[kOwn];
+  const float* w = of_keys ? a.kv_weight : a.q_weight;
+  // (what the stores below need is asked for with the row itself)
+  int64_t slot = 0;
+  const bool paged = of_keys && !rows_out;
+  if (paged) slot = a.slots[t];
+  const int64_t at = (paged && a.n > 0) ? static_cast<int64_t>(a.positions[t]) * (a.n / 2) : 0;
+  constexpr int kOwn = 4;      // values a thread keeps (latents of up to 1,024 values; longer ones are read again)
+  float own[kOwn], weight[kOwn];
   Acc ss = 0;
 #pragma unroll
   for (int i = 0; i < kOwn; ++i) {
-    const int c = lane + i * kWave;
+    const int c = tid + i * 256;
     own[i] = c < width ? load_f32(src + c) : 0.f;
+    weight[i] = c < width ? w[c] : 0.f;
     ss += static_cast<Acc>(own[i]) * static_cast<Acc>(own[i]);
   }
-  for (int c = lane + kOwn * kWave; c < width; c += kWave) ss += static_cast<Acc>(load_f32(src + c)) * static_cast<Acc>(load_f32(src + c));
-  ss = wave_sum(ss);
-  const Acc inv = static_cast<Acc>(1) / sqrt(ss / static_cast<Acc>(width) + static_cast<Acc>(of_keys ? a.kv_eps : a.q_eps));
-  const float* w = of_keys ? a.kv_weight : a.q_weight;
-  auto normed = [&](float v, int c) { return static_cast<float>(static_cast<Acc>(v) * inv * static_cast<Acc>(w[c])); };
+  for (int c = tid + kOwn * 256; c < width; c += 256) ss += static_cast<Acc>(load_f32(src + c)) * static_cast<Acc>(load_f32(src + c));
+  const Acc inv = static_cast<Acc>(1) / sqrt(block_sum<Acc, 256>(ss, scratch) / static_cast<Acc>(width) + static_cast<Acc>(of_keys ? a.kv_eps : a.q_eps));
   T *dst, *dst_v = nullptr;
   int64_t v_step = 0;
   int first = 0;
@@ -63,33 +65,27 @@ __global__ void __launch_bounds__(256) latent_rows_kernel(const T* __restrict__ 
   } else if (rows_out) {
     dst = rows_out + static_cast<int64_t>(t) * a.row_stride;
   } else {
-    const int64_t slot = a.slots[t], page = slot / a.block_size, place = slot % a.block_size;
+    const int64_t page = slot / a.block_size, place = slot % a.block_size;
     dst = k_cache + (page * a.block_size + place) * a.d;
     dst_v = v_cache + page * a.d * a.block_size + place;
     v_step = a.block_size;
     first = a.n;
   }
-#pragma unroll
-  for (int i = 0; i < kOwn; ++i) {
-    const int c = lane + i * kWave;
-    if (c < width) {
-      const float y = normed(own[i], c);
-      store_f32(dst + first + c, y);
-      if (dst_v) store_f32(dst_v + (first + c) * v_step, y);
-    }
-  }
-  for (int c = lane + kOwn * kWave; c < width; c += kWave) {
-    const float y = normed(load_f32(src + c), c);
+  auto put = [&](float v, float wc, int c) {
+    const float y = static_cast<float>(static_cast<Acc>(v) * inv * static_cast<Acc>(wc));
     store_f32(dst + first + c, y);
     if (dst_v) store_f32(dst_v + (first + c) * v_step, y);
-  }
+  };
+#pragma unroll
+  for (int i = 0; i < kOwn; ++i)
+    if (tid + i * 256 < width) put(own[i], weight[i], tid + i * 256);
+  for (int c = tid + kOwn * 256; c < width; c += 256) put(load_f32(src + c), w[c], c);
   if (!of_keys) return;
   if (rows_out) {
-    for (int c = lane; c < a.row_width - a.r; c += kWave) store_f32(dst + a.r + c, c < a.n ? load_f32(src + a.r + c) : 0.f);
+    for (int c = tid; c < a.row_width - a.r; c += 256) store_f32(dst + a.r + c, c < a.n ? load_f32(src + a.r + c) : 0.f);
     return;
   }
-  const int64_t at = a.n > 0 ? static_cast<int64_t>(a.positions[t]) * (a.n / 2) : 0;
-  for (int i = lane; i < a.n / 2; i += kWave) {
+  for (int i = tid; i < a.n / 2; i += 256) {
     const Acc u = static_cast<Acc>(load_f32(src + a.r + 2 * i)), v = static_cast<Acc>(load_f32(src + a.r + 2 * i + 1));
     const Acc cs = static_cast<Acc>(a.cos_t[at + i]), sn = static_cast<Acc>(a.sin_t[at + i]);
     store_f32(dst + 2 * i, static_cast<float>(u * cs - v * sn));
@@ -97,7 +93,7 @@ __global__ void __launch_bounds__(256) latent_rows_kernel(const T* __restrict__ 
     store_f32(dst_v + 2 * i * v_step, 0.f);
     store_f32(dst_v + (2 * i + 1) * v_step, 0.f);
   }
-  for (int c = a.n + a.r + lane; c < a.d; c += kWave) {
+  for (int c = a.n + a.r + tid; c < a.d; c += 256) {
     store_f32(dst + c, 0.f);
     store_f32(dst_v + c * v_step, 0.f);
   }
@@ -132,7 +128,7 @@ extern "C" int alofa_latent_rows(const void* x, int64_t x_stride, int dtype, int
   ALOFA_REQUIRE(!exact || dtype == kF32, "latent_rows: the exact path is float32");
   if (tokens == 0) return 0;
   LatentRows a{x_stride, q_at, q_rank, q_weight, q_eps, cq_stride, kv_at, r, n, kv_weight, kv_eps, positions, cos_t, sin_t, slots, block_size, d, row_stride, row_width};
-  const unsigned grid = static_cast<unsigned>((static_cast<int64_t>(tokens) * (q_rank > 0 ? 2 : 1) + 3) / 4);
+  const unsigned grid = static_cast<unsigned>(static_cast<int64_t>(tokens) * (q_rank > 0 ? 2 : 1));
 #define ALOFA_LATENT_ROWS(T, ACC) latent_rows_kernel<T, ACC><<<grid, 256, 0, stream>>>(static_cast<const T*>(x), static_cast<T*>(cq), static_cast<T*>(k_cache), static_cast<T*>(v_cache), static_cast<T*>(rows_out), tokens, a)
   if (exact) ALOFA_LATENT_ROWS(float, double);
   else if (dtype == kF32) ALOFA_LATENT_ROWS(float, float);

@@ -17,11 +17,11 @@ namespace alofa {
 // own bests, found by exchanges between lanes (value falling, index rising).
 constexpr int kMaxExperts = 512;
 
-template <typename Acc>
+// kOwn: products a lane holds (experts up to 64 * kOwn).
+template <typename Acc, int kOwn>
 __global__ void __launch_bounds__(256) route_top_kernel(const float* __restrict__ z, int64_t z_stride, float* __restrict__ dense, int32_t* __restrict__ chosen,
                                                         float* __restrict__ weights, float* __restrict__ shared_weight, int tokens, int experts, int top, float scale,
                                                         int renorm, int softmax) {
-  constexpr int kOwn = kMaxExperts / kWave;
   const int t = blockIdx.x * 4 + threadIdx.x / kWave, lane = threadIdx.x % kWave;
   if (t >= tokens) return;
   const float* row = z + static_cast<int64_t>(t) * z_stride;
@@ -34,9 +34,12 @@ __global__ void __launch_bounds__(256) route_top_kernel(const float* __restrict_
     const int e = lane + i * kWave;
     own[i] = e < experts ? row[e] : 0.f;
     taken[i] = e >= experts;
-    if (e < experts) d[e] = 0.f;
   }
-  Acc total = 0;
+  // pick k stays with lane k % 64 (its place k / 64) until the sum of all is known
+  Acc total = 0, score[kOwn];
+  int pick[kOwn];
+#pragma unroll
+  for (int i = 0; i < kOwn; ++i) score[i] = 0, pick[i] = -1;
   for (int k = 0; k < top; ++k) {
     float best = 0.f;
     int best_e = 1 << 30;
@@ -57,29 +60,45 @@ __global__ void __launch_bounds__(256) route_top_kernel(const float* __restrict_
         best_e = other_e;
       }
     }
-#pragma unroll
-    for (int i = 0; i < kOwn; ++i)
-      if (lane + i * kWave == best_e) taken[i] = true;
     if (k == 0) largest = best;
     const Acc s = softmax ? exp(static_cast<Acc>(best) - static_cast<Acc>(largest)) : static_cast<Acc>(1) / (static_cast<Acc>(1) + exp(-static_cast<Acc>(best)));
     total += s;
-    if (lane == 0) {
-      chosen[static_cast<int64_t>(t) * top + k] = best_e;
-      weights[static_cast<int64_t>(t) * top + k] = static_cast<float>(s);      // (made final below)
+#pragma unroll
+    for (int i = 0; i < kOwn; ++i) {
+      if (lane + i * kWave == best_e) taken[i] = true;
+      if (lane + i * kWave == k) score[i] = s, pick[i] = best_e;
     }
   }
-  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-  __builtin_amdgcn_wave_barrier();
-  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-  if (lane == 0) {
-    for (int k = 0; k < top; ++k) {
-      Acc w = static_cast<Acc>(weights[static_cast<int64_t>(t) * top + k]);
-      if (renorm || softmax) w /= total;
-      const float f = static_cast<float>(w * static_cast<Acc>(scale));
-      weights[static_cast<int64_t>(t) * top + k] = f;
-      d[chosen[static_cast<int64_t>(t) * top + k]] = f;
+  // what an expert gets: the final weight of the pick that named it (the lanes that hold the picks hand them round)
+  float out[kOwn], mine[kOwn];
+#pragma unroll
+  for (int i = 0; i < kOwn; ++i) {
+    mine[i] = 0.f;
+    Acc w = score[i];
+    if (renorm || softmax) w /= total;
+    out[i] = static_cast<float>(w * static_cast<Acc>(scale));
+    const int k = lane + i * kWave;
+    if (k < top) {
+      chosen[static_cast<int64_t>(t) * top + k] = pick[i];
+      weights[static_cast<int64_t>(t) * top + k] = out[i];
     }
   }
+  for (int k = 0; k < top; ++k) {
+    float w = 0.f;
+    int e = 0;
+#pragma unroll
+    for (int i = 0; i < kOwn; ++i)
+      if (k / kWave == i) {      // (uniform)
+        w = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(out[i]), k % kWave));
+        e = __builtin_amdgcn_readlane(pick[i], k % kWave);
+      }
+#pragma unroll
+    for (int i = 0; i < kOwn; ++i)
+      if (lane + i * kWave == e) mine[i] = w;
+  }
+#pragma unroll
+  for (int i = 0; i < kOwn; ++i)
+    if (lane + i * kWave < experts) d[lane + i * kWave] = mine[i];
 }
 
 // ---- the choice among experts in groups, by softmax scores with a correction -----------------------------------
@@ -250,8 +269,11 @@ extern "C" int alofa_route_top(const float* z, int64_t z_stride, float* dense, i
   ALOFA_REQUIRE(tokens >= 0 && experts > 0 && experts <= kMaxExperts && top > 0 && top <= experts, "route_top: bad sizes (tokens=%d experts=%d top=%d)", tokens, experts, top);
   if (tokens == 0) return 0;
   const unsigned grid = static_cast<unsigned>((tokens + 3) / 4);
-  if (exact) route_top_kernel<double><<<grid, 256, 0, stream>>>(z, z_stride, dense, chosen, weights, shared_weight, tokens, experts, top, scale, renorm, softmax);
-  else route_top_kernel<float><<<grid, 256, 0, stream>>>(z, z_stride, dense, chosen, weights, shared_weight, tokens, experts, top, scale, renorm, softmax);
+#define ALOFA_ROUTE(ACC, OWN) route_top_kernel<ACC, OWN><<<grid, 256, 0, stream>>>(z, z_stride, dense, chosen, weights, shared_weight, tokens, experts, top, scale, renorm, softmax)
+  if (exact) ALOFA_ROUTE(double, kMaxExperts / kWave);
+  else if (experts <= kWave) ALOFA_ROUTE(float, 1);
+  else ALOFA_ROUTE(float, kMaxExperts / kWave);
+#undef ALOFA_ROUTE
   return check_launch("route_top");
 }
 

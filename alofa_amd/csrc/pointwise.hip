@@ -578,9 +578,12 @@ __global__ void __launch_bounds__(256) rmsnorm_add_kernel(float* __restrict__ re
 // ---- out = x in the activation type (eight values a thread) ------------------------------------------------------------
 __global__ void __launch_bounds__(256) to_bf16_kernel(bf16_t* __restrict__ out, const float* __restrict__ x, int64_t elements) {
   const int64_t e = (static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x) * 8;
-#pragma unroll
-  for (int i = 0; i < 8; ++i)
-    if (e + i < elements) out[e + i] = f32_to_bf16(x[e + i]);
+  if (e + 8 <= elements) {
+    const float4 a = *reinterpret_cast<const float4*>(x + e), b = *reinterpret_cast<const float4*>(x + e + 4);
+    *reinterpret_cast<uint4*>(out + e) = make_uint4(pack_bf16x2(a.x, a.y), pack_bf16x2(a.z, a.w), pack_bf16x2(b.x, b.y), pack_bf16x2(b.z, b.w));
+    return;
+  }
+  for (int64_t i = e; i < elements; ++i) out[i] = f32_to_bf16(x[i]);
 }
 
 // ---- x = cap * tanh(x / cap) ---------------------------------------------------------------------------------------
@@ -689,7 +692,7 @@ extern "C" int alofa_rmsnorm_add(float* residual, const float* x, const float* w
 }
 
 extern "C" int alofa_to_bf16(void* out, const float* x, int64_t elements, hipStream_t stream) {
-  ALOFA_REQUIRE(elements >= 0, "to_bf16: bad sizes");
+  ALOFA_REQUIRE(elements >= 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0, "to_bf16: operands must be 16-byte aligned");
   if (elements == 0) return 0;
   to_bf16_kernel<<<blocks_of((elements + 7) / 8), 256, 0, stream>>>(static_cast<bf16_t*>(out), x, elements);
   return check_launch("to_bf16");

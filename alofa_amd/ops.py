@@ -531,6 +531,24 @@ def decode_waves(d: int) -> int:
 FORCED_DECODE_PARTS = int(os.environ.get("ALOFA_DECODE_PARTS", "0"))     # for measurements: so many parts whatever the sizes (0: the rule below)
 
 
+DECODE_BLOCK_HEADS = 16      # query heads of a key head that a block of the decode kernel serves at most
+HAND_OVER_MAX_FLOATS = 8192  # one wide key head: up to so many sums (parts x heads of a block x head size) the last block combines the parts, else a second kernel
+
+
+def decode_block_heads(tokens: int, heads: int, kv_heads: int, d: int) -> int:
+    """Query heads of a key head that a block of the decode kernel serves. All of them (up to 16) share the keys a block reads; but where ONE wide
+    key head serves many queries (attention over latents), what a block combines and hands over, heads x head size sums, takes longer than its
+    keys, so the heads are dealt out over blocks too while the tokens leave the chip room (16 heads of 256 channels at 550 keys: 10 us with two heads
+    a block and eight parts against 28 with sixteen, one token; 13 with four against 28, eight tokens; 22.8 with eight and two parts against 28, sixty-four)."""
+    group = heads // kv_heads
+    if kv_heads != 1 or d < 128 or group < 4:
+        return DECODE_BLOCK_HEADS
+    for n in (2, 4, 8):
+        if tokens * -(-group // n) <= 32:
+            return n
+    return 8 if tokens * -(-group // 8) <= compute_units() else DECODE_BLOCK_HEADS
+
+
 def decode_splits(tokens: int, heads: int, kv_heads: int, d: int, max_context: int) -> int:
     """Parts the keys of a (token, key head) are cut into beyond the waves of a block. A block reads
     its keys at the rate of one compute unit, so while the blocks are far fewer than the compute
@@ -560,10 +578,14 @@ _hand_over_known: dict = {}
 def _decode_splits_rule(tokens: int, heads: int, kv_heads: int, d: int, max_context: int) -> int:
     waves = decode_waves(d)
     step = 32 * waves
-    if max_context <= 2 * step:
+    narrow = decode_block_heads(tokens, heads, kv_heads, d) < DECODE_BLOCK_HEADS
+    if max_context <= 2 * step and not narrow:
         return 1
-    blocks = tokens * kv_heads * -(-(heads // kv_heads) // 16)
+    blocks = tokens * kv_heads * -(-(heads // kv_heads) // decode_block_heads(tokens, heads, kv_heads, d))
     by_chip = max(1, compute_units() // max(1, blocks))
+    if narrow:      # (few heads a block: what the parts hand over is little)
+        by_length = -(-max_context // step)
+        return max(1, min(64, by_length if by_length <= 8 else max(8, -(-max_context // (2 * step))), by_chip))
     if max_context <= 4 * step:
         return 4 if by_chip >= 4 else 1
     if max_context <= 8 * step and by_chip < 4:
@@ -583,13 +605,16 @@ def decode_hand_over(tokens: int, heads: int, kv_heads: int, d: int, n_splits: i
     second kernel."""
     if n_splits <= 1 or n_splits > HAND_OVER_MAX_PARTS:
         return False
+    block_heads = decode_block_heads(tokens, heads, kv_heads, d)
+    if block_heads < DECODE_BLOCK_HEADS and min(block_heads, heads // kv_heads) * n_splits * d > HAND_OVER_MAX_FLOATS:
+        return False
     key = (tokens, heads, kv_heads, d, n_splits)
     known = _hand_over_known.get(key)
     if known is None:      # (what fits the workspace does not change once it is there)
         _ensure_workspace(None)
         if len(_hand_over_known) > 1 << 16:
             _hand_over_known.clear()
-        known = _hand_over_known[key] = bool(load().alofa_attention_decode_can_hand_over(_I(tokens), _I(heads), _I(kv_heads), _I(d), _I(n_splits)))
+        known = _hand_over_known[key] = bool(load().alofa_attention_decode_can_hand_over(_I(tokens), _I(heads), _I(kv_heads), _I(d), _I(n_splits), _I(decode_block_heads(tokens, heads, kv_heads, d))))
     return known
 
 
@@ -673,7 +698,8 @@ def _sink_of(sink: Optional[torch.Tensor], heads: int) -> Optional[torch.Tensor]
 def attention_decode(out, q, k_cache, v_cache, block_table, req_of_token, positions, heads, kv_heads, d, window, scale,
                      max_context: int, scratch: Optional[torch.Tensor], rows: Optional[torch.Tensor] = None,
                      rope: Optional[tuple] = None, n_splits: Optional[int] = None, hand_over: Optional[bool] = None,
-                     v_head: Optional[int] = None, fine_weights: bool = False, all_value_heads: bool = False, sink: Optional[torch.Tensor] = None) -> None:
+                     v_head: Optional[int] = None, fine_weights: bool = False, all_value_heads: bool = False, sink: Optional[torch.Tensor] = None,
+                     block_heads: Optional[int] = None) -> None:
     """bfloat16 attention for tokens of requests that bring few tokens: every
     token of the batch, or the tokens ``rows`` (int32 indices into the batch).
     ``req_of_token`` None: every request brings one token and token i is request
@@ -690,7 +716,8 @@ def attention_decode(out, q, k_cache, v_cache, block_table, req_of_token, positi
     plane per value head, and a scratch buffer is sized with tokens x kv_heads for ``tokens``.
     ``out`` may be float32: the results are then stored unrounded. ``fine_weights``: every softmax weight meets the values as two bfloat16
     numbers, its rounding and what the rounding took away, so that sixteen bits of it count (twice the second product's instructions).
-    ``sink`` [heads] float32: exp(sink) joins the denominator of the head's rows."""
+    ``sink`` [heads] float32: exp(sink) joins the denominator of the head's rows. ``block_heads`` (default ``decode_block_heads``): how many heads of a
+    key head a block serves, 1 to 16."""
     planes = _value_planes(out, all_value_heads, v_head, kv_heads)
     T, bs = _attention_operands(out[0] if planes else out, q, k_cache, v_cache, block_table, heads, kv_heads, d)
     for n, t in (("req_of_token", req_of_token), ("positions", positions)):
@@ -721,12 +748,14 @@ def attention_decode(out, q, k_cache, v_cache, block_table, req_of_token, positi
             raise AlofaError("shape_mismatch", "one cache slot per token", f"slots={tuple(slots.shape)} T={T}")
     served = n_tok      # (the grid's first dimension: tokens, or (token, value head) pairs)
     n_tok *= max(planes, 1)
+    if block_heads is None:
+        block_heads = decode_block_heads(n_tok, heads, kv_heads, d)
     if n_splits is None:
         n_splits = decode_splits(n_tok, heads, kv_heads, d, min(max_context, window or max_context))
     if hand_over is None:
         hand_over = decode_hand_over(n_tok, heads, kv_heads, d, n_splits)
     elif hand_over and not (n_splits > 1 and _ensure_workspace(None) is None
-                            and load().alofa_attention_decode_can_hand_over(_I(n_tok), _I(heads), _I(kv_heads), _I(d), _I(n_splits))):
+                            and load().alofa_attention_decode_can_hand_over(_I(n_tok), _I(heads), _I(kv_heads), _I(d), _I(n_splits), _I(block_heads))):
         raise AlofaError("out_of_range", "the parts' states do not fit the library's workspace (or there is one part only)", f"tokens={n_tok} heads={heads} d={d} n_splits={n_splits}")
     floats = n_tok * heads * n_splits * (d + 2) if n_splits > 1 and not hand_over else 0
     if floats and (scratch is None or scratch.dtype is not torch.float32 or not scratch.is_cuda or scratch.numel() < floats or not scratch.is_contiguous()):
@@ -738,7 +767,7 @@ def attention_decode(out, q, k_cache, v_cache, block_table, req_of_token, positi
           _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _I(block_table.shape[1]), _ptr(req_of_token), _ptr(positions), _ptr(rows),
           _I(served), _I(heads), _I(kv_heads), _I(d), _I(bs), _I(int(window or 0)), _F(scale), _I(n_splits),
           _ptr(cos), _ptr(sin), _ptr(slots), _I(int(hand_over)), _I(-1 if v_head is None else v_head), _ptr(out if as32 else None), _I(int(fine_weights)),
-          _I(planes), _L(out.stride(0) if planes else 0), _ptr(_sink_of(sink, heads)), _stream())
+          _I(planes), _L(out.stride(0) if planes else 0), _ptr(_sink_of(sink, heads)), _I(block_heads), _stream())
 
 
 def can_fuse_rope_into_decode(d: int) -> bool:
@@ -1719,7 +1748,7 @@ def experts_up(act: torch.Tensor, x: torch.Tensor, w_up: torch.Tensor, rows: Exp
 def experts_sum_norm(residual: torch.Tensor, y: torch.Tensor, rows: ExpertRows, weight: torch.Tensor, eps: float, out: Optional[torch.Tensor] = None,
                      scratch=None) -> None:
     """residual[t] += rmsnorm(s) * weight with s the sum of row t's slots (``experts_sum``'s); ``out`` bfloat16 of the stream's shape: the stream's new rows are left
-    there too. ``scratch(name, shape, dtype)`` gives the room that rows of more than 4,096 values need."""
+    there too. ``scratch(name, shape, dtype)`` gives the room that rows of more values than a block keeps need."""
     _gpu("residual", residual, torch.float32, 2), _gpu("y", y, torch.float32, 2), _gpu("weight", weight, torch.float32, 1)
     _contig("residual", residual), _contig("y", y), _contig("weight", weight)
     T, h = residual.shape
@@ -1729,7 +1758,7 @@ def experts_sum_norm(residual: torch.Tensor, y: torch.Tensor, rows: ExpertRows, 
         _gpu("out", out, torch.bfloat16, 2), _contig("out", out)
         if out.shape != residual.shape:
             raise AlofaError("shape_mismatch", "the new rows do not fit the stream", f"out={tuple(out.shape)} residual={tuple(residual.shape)}")
-    wide = scratch("experts_wide_sum", (T, h), torch.float32) if h > 4096 else None
+    wide = scratch("experts_wide_sum", (T, h), torch.float32) if load().alofa_experts_sum_norm_room(_I(h)) else None
     _call("alofa_experts_sum_norm", _ptr(residual), _ptr(y), _ptr(rows.slot_of), _ptr(weight), _F(eps), _ptr(out), _ptr(wide), _I(T), _I(h), _I(rows.top), _I(int(rows.shared)), _stream())
 
 
