@@ -1338,6 +1338,53 @@ def linear_recurrence(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: to
     return used.value
 
 
+CHUNK_ROWS = 64           # rows of a chunk of ``chunked_recurrence``
+CHUNKED_FROM = 96         # rows of one request in a step from which a constant decay is taken in chunks
+USE_CHUNKS = os.environ.get("ALOFA_CHUNKED_RECURRENCE", "1") != "0"      # 0 (for measurements): every step goes row by row
+
+
+class Chunks:
+    """A step's rows in chunks of up to ``CHUNK_ROWS`` rows of one request, for ``chunked_recurrence``. ``spans``: (first row, rows) per request,
+    in the step's order."""
+
+    def __init__(self, spans: list, device):
+        chunks, of_request = [], []
+        for r, (row0, n) in enumerate(spans):
+            of_request.append((len(chunks), -(-n // CHUNK_ROWS)))
+            chunks += [(r, row0 + a, min(CHUNK_ROWS, n - a), 0) for a in range(0, n, CHUNK_ROWS)]
+        self.requests, self.count, self.rows = len(of_request), len(chunks), sum(n for _, n in spans)
+        both = torch.tensor([x for c in chunks for x in c] + [x for c in of_request for x in c], dtype=torch.int32, device=device)
+        self.chunks, self.of_request = both[:4 * self.count], both[4 * self.count:]
+
+
+def decay_powers(decay: torch.Tensor) -> torch.Tensor:
+    """g^0 .. g^CHUNK_ROWS of every head's decay: float32 [heads, CHUNK_ROWS + 1], formed in float64."""
+    return torch.pow(decay.double()[:, None], torch.arange(CHUNK_ROWS + 1, dtype=torch.float64, device=decay.device)[None, :]).float().contiguous()
+
+
+def can_chunk(q: torch.Tensor, k: torch.Tensor, dk: int, longest: int) -> bool:
+    """Whether a step whose longest portion has so many rows should take a constant decay in chunks, and the kernels take its rows."""
+    return USE_CHUNKS and longest >= CHUNKED_FROM and dk % 8 == 0 and _aligned_rows(q) and _aligned_rows(k)
+
+
+def chunked_recurrence(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Tensor, rows: RowsOfRequests, chunks: Chunks, heads: int,
+                       dk: int, dv: int, powers: torch.Tensor, added: torch.Tensor, q_scale: float = 1.0, k_scale: float = 1.0) -> None:
+    """``linear_recurrence`` with a constant decay per head (``powers`` = ``decay_powers`` of them), bfloat16 rows, in chunks: every chunk's own contribution and
+    read-outs side by side, and only the states in front of the chunks one after the other; all products in float32. ``out`` float32 [T, heads * dv]; ``added``
+    float32 [chunks, heads, dk, dv]: room for what the chunks add and then for the states in front of them."""
+    _gpu("out", out, torch.float32, 2), _contig("out", out), _gpu("q", q, torch.bfloat16, 2), _gpu("k", k, torch.bfloat16, 2), _gpu("v", v, torch.bfloat16, 2)
+    _gpu("state", state, torch.float32, 4), _contig("state", state), _gpu("powers", powers, torch.float32, 2), _contig("powers", powers), _gpu("added", added, torch.float32, 4), _contig("added", added)
+    T = q.shape[0]
+    if (tuple(q.shape) != (T, heads * dk) or tuple(k.shape) != (T, heads * dk) or tuple(v.shape) != (T, heads * dv) or tuple(out.shape) != (T, heads * dv)
+            or tuple(state.shape[1:]) != (heads, dk, dv) or T != rows.rows or T != chunks.rows or rows.requests != chunks.requests
+            or tuple(powers.shape) != (heads, CHUNK_ROWS + 1) or tuple(added.shape) != (chunks.count, heads, dk, dv)):
+        raise AlofaError("shape_mismatch", "recurrence operands do not fit", f"q={tuple(q.shape)} k={tuple(k.shape)} v={tuple(v.shape)} out={tuple(out.shape)} state={tuple(state.shape)} "
+                         f"heads={heads} dk={dk} dv={dv} rows={rows.rows} chunks={chunks.count} added={tuple(added.shape)}")
+    rows.fits("state", state)
+    _call("alofa_chunked_recurrence", _ptr(out), _L(_rows("out", out)), _ptr(q), _L(_rows("q", q)), _ptr(k), _L(_rows("k", k)), _ptr(v), _L(_rows("v", v)), _ptr(state), _ptr(rows.slots),
+          _ptr(chunks.chunks), _I(chunks.count), _ptr(chunks.of_request), _I(chunks.requests), _ptr(powers), _ptr(added), _I(heads), _I(dk), _I(dv), _F(q_scale), _F(k_scale), _stream())
+
+
 def gate_scan(gates: torch.Tensor, z: torch.Tensor, state: torch.Tensor, rows: RowsOfRequests, heads: int, cap: float) -> None:
     """Exponential gates kept in range by a running maximum m (``state`` float32 [slots, heads], read and left there), per request over
     its rows in order: with z [T, 2 * heads] float32 (input gates' then forget gates' products), i = cap tanh(zi / cap),

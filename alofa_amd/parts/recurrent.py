@@ -1,7 +1,7 @@
 """Mixers that keep a state of fixed size per request instead of keys: per head a matrix S [dk, dv] in float32 that
 every token decays and adds to, S_t = diag(w_t) S_(t-1) + k_t v_t^T, and reads out with its query. They differ in
 where the decay comes from and in the order of read-out and update; the recurrence itself is one kernel
-(``ops.linear_recurrence``), and so are the norm of every head's read-out with the gate (``ops.headnorm_gate``).
+(``ops.linear_recurrence``; with a constant decay and a long portion of a prompt, ``ops.chunked_recurrence``), and so are the norm of every head's read-out with the gate (``ops.headnorm_gate``).
 
 retention       w = a constant per head; rotary positions on q and k, or none; k scaled by dk^(-1/2); o_t = S_t^T q_t;
                 o / rms(o) per head, times silu(gate), output projection.
@@ -35,7 +35,7 @@ from ..errors import AlofaError
 from ..weights.loader import TensorRule
 from .attention import _padded_heads
 from .base import Mixer, StateNeed, TimeConv, build_part, part_class, register_part
-from .rows import rows_of_requests
+from .rows import chunks_of_requests, rows_of_requests
 
 
 def _stacked(rt, mats: list) -> torch.Tensor:
@@ -54,6 +54,7 @@ class RecurrentMixer(Mixer):
         self.hidden, self.heads, self.dk = int(p["hidden"]), int(p["heads"]), int(p["key_dim"])
         self.dv = int(p.get("value_dim") or self.dk)
         self.eps = float(p["eps"])
+        self.decay = self.powers = None      # (kinds with one constant decay per head set the first)
         if self.heads <= 0 or self.dv <= 0 or not 0 < self.dk <= ops.RECURRENCE_MAX_KEYS:
             raise AlofaError("unsupported", f"the recurrence kernel takes key sizes up to {ops.RECURRENCE_MAX_KEYS}", f"heads={self.heads} key_dim={self.dk} value_dim={self.dv}")
 
@@ -63,6 +64,19 @@ class RecurrentMixer(Mixer):
     def _readouts(self, ctx, rows: int):
         """Room for the read-outs of a step: float32 [parts, T, heads * dv]; a step of many rows may leave them in parts."""
         return ctx.scratch("recurrent_out", (ops.recurrence_max_parts(self.dk), rows, self.heads * self.dv), torch.float32)
+
+    def _constant_decay(self, ctx, where, o, q, k, v, k_scale: float = 1.0) -> int:
+        """The recurrence with one constant decay per head (``self.decay``), its read-outs left in ``o``; returns in how many parts. Steps that bring a long
+        portion of a prompt take it in chunks of rows, on the matrix cores; all others row by row."""
+        rows = rows_of_requests(ctx)
+        if ops.can_chunk(q, k, self.dk, ctx.max_q_len):
+            if self.powers is None:
+                self.powers = ops.decay_powers(self.decay)
+            chunks = chunks_of_requests(ctx)
+            added = ctx.scratch("recurrent_chunks", (chunks.count, self.heads, self.dk, self.dv), torch.float32)
+            ops.chunked_recurrence(o[0], q, k, v, ctx.state(where), rows, chunks, self.heads, self.dk, self.dv, self.powers, added, k_scale=k_scale)
+            return 1
+        return ops.linear_recurrence(o, q, k, v, ctx.state(where), rows, self.heads, self.dk, self.dv, ops.DECAY_PER_HEAD, self.decay, k_scale=k_scale)
 
     def _leave(self, ctx, o, parts, gate, weight, residual, out):
         """Head norm, gate and output projection of the read-outs ``o`` (float32 [P, T, heads * dv], the first ``parts`` to be added)."""
@@ -121,8 +135,7 @@ class Retention(RecurrentMixer):
         else:      # queries and keys alike: 2 * heads heads to rotate, nothing to write to pages
             ops.rope_kv_write(proj, table[0], table[1], ctx.positions, 2 * self.heads, 0, self.dk)
         o = self._readouts(ctx, T)
-        parts = ops.linear_recurrence(o, proj[:, :kd], proj[:, kd:2 * kd], proj[:, 2 * kd:2 * kd + vd], ctx.state(where), rows_of_requests(ctx),
-                                      self.heads, self.dk, self.dv, ops.DECAY_PER_HEAD, self.decay, k_scale=self.k_scale)
+        parts = self._constant_decay(ctx, where, o, proj[:, :kd], proj[:, kd:2 * kd], proj[:, 2 * kd:2 * kd + vd], self.k_scale)
         self._leave(ctx, o, parts, proj[:, 2 * kd + vd:], None, residual, out)
 
 
@@ -191,8 +204,7 @@ class LightningAttention(RecurrentMixer):
         qkv = proj[:, :2 * kd + vd]
         ops.activation(qkv, qkv, ops.SILU, exact=self.rt.exact)
         o = self._readouts(ctx, T)
-        parts = ops.linear_recurrence(o, proj[:, :kd], proj[:, kd:2 * kd], proj[:, 2 * kd:2 * kd + vd], ctx.state(where), rows_of_requests(ctx),
-                                      self.heads, self.dk, self.dv, ops.DECAY_PER_HEAD, self.decay)
+        parts = self._constant_decay(ctx, where, o, proj[:, :kd], proj[:, kd:2 * kd], proj[:, 2 * kd:2 * kd + vd])
         # (the heads together are one row to norm: a "head" of heads * dv channels)
         y = ctx.scratch("recurrent_gated", (T, vd), self.rt.dtype)
         ops.headnorm_gate(y, o, proj[:, 2 * kd + vd:], self.norm, 1, vd, self.eps, self.rt.exact, parts=parts, gate_kind="sigmoid")

@@ -10,6 +10,10 @@ def rows_of_requests(ctx) -> ops.RowsOfRequests:
     return ctx.memo("rows of requests", lambda: _build(ctx))
 
 
+def chunks_of_requests(ctx) -> ops.Chunks:
+    return ctx.memo("chunks of requests", lambda: ops.Chunks([(s.row0, s.n) for s in ctx.spans], ctx.device))
+
+
 def _build(ctx) -> ops.RowsOfRequests:
     n, n_slots = len(ctx.spans), ctx.fn.cache.max_requests
     if ctx.max_q_len == 1:      # every request brings one row: request r owns row r

@@ -256,17 +256,18 @@ class Pages:
 SINKS = (6.0, -40.0, 0.0, 2.0, 15.0, -1.0, 3.0)
 
 
-@pytest.mark.parametrize("heads, kv_heads, d", [(6, 1, 64), (7, 1, 96), (8, 1, 128), (20, 1, 48), (12, 2, 32), (4, 4, 64), (5, 1, 256), (3, 1, 16)])
+ALONE = [(6, 1, 64), (7, 1, 96), (8, 1, 128), (20, 1, 48), (12, 2, 32), (4, 4, 64), (5, 1, 256), (3, 1, 16)]
+SHARING = [(6, 1, 64), (7, 1, 96), (8, 1, 128), (20, 1, 48), (12, 2, 32), (7, 1, 16)]
+
+
+@pytest.mark.parametrize("heads, kv_heads, d, shared", [(*s, False) for s in ALONE] + [(*s, True) for s in SHARING])
 @pytest.mark.parametrize("window", [None, 1, 33, 64, 100])
-@pytest.mark.parametrize("shared", [False, True])
 def test_prompt_rows_with_a_sink(heads, kv_heads, d, window, shared):
     """The prefill kernel with sixteen bits of every weight, each head with blocks of its own and six to eight heads sharing their tiles."""
     from alofa_amd import ops
     group = heads // kv_heads
     chunks = -(-group // 8)
     share = -(-group // chunks) if shared else 0
-    if shared and (d > 128 or not 6 <= share <= 8):
-        pytest.skip("these heads do not share tiles")
     lengths, new = [150, 70, 200], [150, 20, 65]
     pages = Pages(lengths, kv_heads, d, 16, heads + d)
     rng = np.random.default_rng(3)
@@ -290,9 +291,11 @@ def test_prompt_rows_with_a_sink(heads, kv_heads, d, window, shared):
 
 @pytest.mark.parametrize("heads, kv_heads, d", [(6, 1, 64), (20, 1, 96), (16, 1, 256), (12, 2, 80), (4, 4, 32)])
 @pytest.mark.parametrize("window", [None, 1, 33, 300])
-@pytest.mark.parametrize("splits, hand_over", [(1, False), (3, False), (4, True), (20, False), (40, False)])
-def test_single_rows_with_a_sink(heads, kv_heads, d, window, splits, hand_over):
-    """The decode kernel: one part, parts that meet in the workspace, parts a second kernel combines: the sink counts once in each."""
+@pytest.mark.parametrize("splits, hand_over, block_heads", [(1, False, 16), (3, False, 16), (4, True, 16), (20, False, 16), (40, False, 16), (1, False, 4), (4, True, 2), (6, True, 4),
+                                                           (5, False, 8), (3, True, 3)])
+def test_single_rows_with_a_sink(heads, kv_heads, d, window, splits, hand_over, block_heads):
+    """The decode kernel: one part, parts that meet in the workspace, parts a second kernel combines: the sink counts once in each; and heads dealt out over
+    blocks."""
     from alofa_amd import ops
     lengths = [1, 40, 333, 700]
     pages = Pages(lengths, kv_heads, d, 16, heads + d)
@@ -301,8 +304,48 @@ def test_single_rows_with_a_sink(heads, kv_heads, d, window, splits, hand_over):
     out = torch.empty(4, heads * d, dtype=BF, device=DEV)
     room = torch.empty(4 * heads * splits * (d + 2), device=DEV)
     ops.attention_decode(out, dev(q, BF), pages.kc, pages.vc, pages.table, None, dev([n - 1 for n in lengths], torch.int32), heads, kv_heads, d, window, 0.3, 1024, room,
-                         n_splits=splits, hand_over=hand_over, fine_weights=True, sink=dev(sink))
+                         n_splits=splits, hand_over=hand_over, fine_weights=True, sink=dev(sink), block_heads=block_heads)
     got = back(out).reshape(4, heads, d)
     for r, n in enumerate(lengths):
         want = pages.attend(q[r].reshape(heads, d), r, n - 1, heads, window, 0.3, sink)
         assert np.abs(got[r] - want).max() <= 2.0 ** -7 * max(1.0, np.abs(want).max()), r
+
+
+# ---- the recurrence in chunks
+
+@pytest.mark.parametrize("heads, dk, dv", [(2, 16, 24), (3, 64, 64), (1, 128, 80), (5, 40, 7), (2, 200, 130)])
+@pytest.mark.parametrize("spans", [[64], [65], [1], [63, 1, 200], [130, 64, 2, 17], [700]])
+def test_a_constant_decay_in_chunks(heads, dk, dv, spans):
+    """Requests of unequal lengths in one call, twice (the second call goes on from the states the first left), against the recurrence row by row."""
+    from alofa_amd import ops
+    from test_recurrent_ops_gpu import rows_of
+    rng = np.random.default_rng(dk + sum(spans))
+    decay = np.array([0.5, 1.0, 0.999, 0.97, 0.0])[:heads].astype(np.float32)
+    T, slots = sum(spans), [4, 1, 3, 0][:len(spans)]
+    state = dev(rng.normal(0, 1, (6, heads, dk, dv)))
+    S = back(state)
+    untouched = S[[s for s in range(6) if s not in slots]].copy()
+    row0 = np.cumsum([0] + spans)
+    chunks = ops.Chunks(list(zip(row0[:-1].tolist(), spans)), DEV)
+    assert chunks.count == sum(-(-n // 64) for n in spans)
+    rows = rows_of(list(zip(slots, spans)), 6)
+    powers = ops.decay_powers(dev(decay))
+    for call in range(2):
+        proj = b16(rng.normal(0, 1, (T, heads * (2 * dk + dv) + 8)))
+        q, k, v = proj[:, :heads * dk], proj[:, heads * dk:2 * heads * dk], proj[:, 2 * heads * dk:2 * heads * dk + heads * dv]
+        wide = (proj.shape[1] + 7) // 8 * 8
+        p = torch.zeros(T, wide, dtype=BF, device=DEV)
+        p[:, :proj.shape[1]] = dev(proj, BF)
+        out, added = torch.full((T, heads * dv), 9.0, device=DEV), torch.empty(chunks.count, heads, dk, dv, device=DEV)
+        assert ops.can_chunk(p[:, :heads * dk], p[:, heads * dk:2 * heads * dk], dk, 1000)
+        ops.chunked_recurrence(out, p[:, :heads * dk], p[:, heads * dk:2 * heads * dk], p[:, 2 * heads * dk:2 * heads * dk + heads * dv], state, rows, chunks, heads, dk, dv, powers, added,
+                               q_scale=0.7, k_scale=dk ** -0.5)
+        want = np.zeros((T, heads, dv))
+        for r, (s, n) in enumerate(zip(slots, spans)):
+            for t in range(row0[r], row0[r] + n):
+                S[s] = decay.astype(np.float64)[:, None, None] * S[s] + dk ** -0.5 * k[t].reshape(heads, dk)[:, :, None] * v[t].reshape(heads, dv)[:, None, :]
+                want[t] = (S[s] * 0.7 * q[t].reshape(heads, dk)[:, :, None]).sum(axis=1)
+        err = np.abs(back(out) - want.reshape(T, -1)).max()
+        assert err <= 2e-5 * max(1.0, np.abs(want).max()), (call, err)
+        assert np.abs(back(state)[slots] - S[slots]).max() <= 2e-5 * max(1.0, np.abs(S[slots]).max())
+    assert (back(state)[[s for s in range(6) if s not in slots]] == untouched).all()
