@@ -444,7 +444,7 @@ __global__ void __launch_bounds__(64 * WPT * TEAMS, (RW == 32 && 64 * WPT * TEAM
   }
   if (row_ok && team == 0) {
     float inv = 1.f / l;
-    if (sink) {      // a number per head whose exponential joins the row's sum (no key, no value, not scaled)
+    if (sink) {      // a number per head whose exponential joins the row's sum and nothing else
       const float s2 = sink[head] * 1.44269504088896340736f, most = fmaxf(top, s2);
       const float shrink = __builtin_amdgcn_exp2f(top - most);
       inv = shrink / (l * shrink + __builtin_amdgcn_exp2f(s2 - most));

@@ -20,7 +20,7 @@ Optional, each chosen by a parameter:
              the last n rows of Wd x (not normed), turned likewise: the score is scale * (q_a . k_a + q'_a . k'). The key that all heads ask is then
              [k' | c], the query of a head [q'_a | Uk_a^T q_a]; what the pages hold beside c is k'. (Where the pages hold every head's keys, k' is
              a part of each.)
-  sink       a number per head whose exponential joins the softmax's denominator (no key, no value, not scaled).
+  sink       a number per head whose exponential joins the softmax's denominator and nothing else.
   window     a row sees itself and the window - 1 rows before it.
 With any of the first three, softmax weights meet the values with sixteen bits each on the matrix cores."""
 from __future__ import annotations

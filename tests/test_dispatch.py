@@ -67,6 +67,16 @@ def test_a_norm_behind_a_product_moves_it_to_the_kernel_that_adds_shares():
     assert not ops.norm_rides_on_shares(32, 8192, 4096)            # too many columns for the launch that adds shares
 
 
+def test_heads_of_one_wide_key_head_are_dealt_out_over_blocks(monkeypatch):
+    monkeypatch.setattr(ops, "_compute_units", 256)
+    for args in ((8, 14, 2, 64), (8, 28, 4, 128), (1, 16, 1, 64), (4, 3, 1, 256), (512, 32, 1, 256)):
+        assert ops.decode_block_heads(*args) == 16, args                             # several key heads, narrow ones, few queries, tokens enough
+    assert [ops.decode_block_heads(t, 16, 1, 256) for t in (1, 4, 8, 16, 64, 128, 256)] == [2, 2, 4, 8, 8, 8, 16]
+    assert [ops.decode_block_heads(t, 32, 1, 256) for t in (1, 2, 8, 64, 128)] == [2, 2, 8, 8, 16]
+    assert [ops.decode_splits(t, 16, 1, 256, 1024) for t in (1, 8, 64)] == [8, 8, 2] and ops.decode_splits(64, 32, 1, 256, 1024) == 1
+    assert ops.decode_splits(1, 16, 1, 256, 128) == 1 and ops.decode_splits(1, 16, 1, 256, 256) == 2
+
+
 def test_decode_splits_follow_the_context(monkeypatch):
     monkeypatch.setattr(ops, "_compute_units", 256)                                # the rule counts the chip's compute units: an MI355X's here
     assert ops.decode_splits(8, 14, 2, 64, 512) == 1                              # the waves of one block cover two steps each

@@ -364,16 +364,17 @@ def test_which_kernels_serve_which_layer(replayers, monkeypatch):
             calls[name] = calls.get(name, 0) + 1
             return real(*a, **k)
         return call
-    for name in ("attention_prefill", "attention_decode", "span_attention", "span_attention_mfma", "experts_up", "weighted_relu_squared"):
+    for name in ("attention_prefill", "attention_decode", "span_attention", "span_attention_mfma", "experts_up", "weighted_relu_squared", "chunked_recurrence", "linear_recurrence"):
         monkeypatch.setattr(ops, name, counted(name))
 
     def run(model, dtype, steps):
         calls.clear()
         collect(replayers(model, dtype), steps)
         return dict(calls)
-    assert run("C", "bfloat16", whole("m", ids_of("C", 70))) == {"attention_prefill": 3, "experts_up": 3}
-    assert run("C", "float32", whole("m", ids_of("C", 70))) == {"span_attention": 3, "weighted_relu_squared": 3}
-    assert run("C", "bfloat16", [{"step": 0, "entries": [{"id": "m", "tokens": [1], "want": []}], "end": ["m"]}]) == {"attention_decode": 3, "experts_up": 3}
+    assert run("C", "bfloat16", whole("m", ids_of("C", 70))) == {"attention_prefill": 3, "experts_up": 3, "linear_recurrence": 1}
+    assert run("C", "bfloat16", whole("m", ids_of("C", 100))) == {"attention_prefill": 3, "experts_up": 3, "chunked_recurrence": 1}      # (from 96 rows of one request on)
+    assert run("C", "float32", whole("m", ids_of("C", 70))) == {"span_attention": 3, "weighted_relu_squared": 3, "linear_recurrence": 1}
+    assert run("C", "bfloat16", [{"step": 0, "entries": [{"id": "m", "tokens": [1], "want": []}], "end": ["m"]}]) == {"attention_decode": 3, "experts_up": 3, "linear_recurrence": 1}
     # (D: heads of 80 channels take the window part's kernel; heads of 24 and 40 are widened to 48, and of 13 and 6 to 16)
     assert run("D", "bfloat16", whole("m", ids_of("D", 70))) == {"span_attention_mfma": 1, "attention_prefill": 2, "experts_up": 1}
 
