@@ -3,7 +3,8 @@ and slots for per-request state of fixed size.
 
 Mixers with the same need of history form a *group* with pages of its own: one
 group for mixers that keep every key, one per window length for mixers that
-see only the last ``window`` keys. Within a group one block id names a page of
+see only the last ``window`` keys (and, where they say so, the first few of the
+sequence, whose pages then stay). Within a group one block id names a page of
 every tensor of every mixer of the group, so a request has one table per group
 (src/alofa/engine/executor.mojo:117-127 for the one-table rule; groups are
 this engine's own). What a page holds is the mixer's business: it names its
@@ -41,8 +42,14 @@ def blocks_for(n_tokens: int, block_size: int) -> int:
 @dataclass
 class Group:
     window: Optional[int]
+    keep_first: int          # first tokens of a sequence whose pages stay when the window passes them
     entries: list            # run entries that own a cache in this group
     pool: BlockPool
+
+
+def window_and_kept(group) -> tuple:
+    """(window, kept first tokens) of a group's name: None, a window, or (window, kept first tokens)."""
+    return group if isinstance(group, tuple) else (group, 0)
 
 
 def _keyed(needs) -> dict:
@@ -58,37 +65,38 @@ class CacheManager:
     ``cache_needs`` and ``state_needs`` map an owner's key (any hashable: the
     model uses (run entry, mixer index)) to its need; a list stands for the keys
     0, 1, 2, ... with None where nothing is kept. ``n_blocks``: the pages of every
-    group's pool, or a dict from a group's window (None: the group that keeps every
-    key) to the pages of that group's pool; every owner's tensors have as many pages
+    group's pool, or a dict from a group's name (its window; None: the group that keeps every
+    key; (window, n) where the first n tokens stay) to the pages of that group's pool; every owner's tensors have as many pages
     as its group's pool, so a group that holds a window only can be given what its
     window needs (``pages_for``)."""
 
     @staticmethod
     def windows_of(cache_needs) -> list:
-        """The groups that these needs make, as their windows in group order (None: every key is kept)."""
+        """The groups that these needs make, by name in group order (None: every key is kept; a window; (window, kept first tokens))."""
         out: list = []
         for need in _keyed(cache_needs).values():
-            if need.window not in out:
-                out.append(need.window)
+            if need.group not in out:
+                out.append(need.group)
         return out
 
     @staticmethod
-    def held_tokens_of(window: Optional[int], step_tokens: int, block_size: int) -> int:
-        """The most tokens a request holds pages for at any time in a group with this window, when a step
+    def held_tokens_of(group, step_tokens: int, block_size: int) -> int:
+        """The most tokens a request holds pages for at any time in this group, when a step
         brings it at most ``step_tokens``: -1 for no bound (every key is kept), else the window plus the step
-        plus the two pages that the window's ends may lie in."""
-        return -1 if window is None else int(window) + int(step_tokens) + 2 * int(block_size)
+        plus the two pages that the window's ends may lie in, plus the pages of the first tokens that stay."""
+        window, keep = window_and_kept(group)
+        return -1 if window is None else int(window) + int(step_tokens) + 2 * int(block_size) + blocks_for(keep, block_size) * int(block_size)
 
     @staticmethod
-    def pages_for(window: Optional[int], requests: int, tokens: int, step_tokens: int, block_size: int) -> int:
-        """Pages that ``requests`` requests of up to ``tokens`` tokens hold at most in a group with this window."""
-        held = CacheManager.held_tokens_of(window, step_tokens, block_size)
+    def pages_for(group, requests: int, tokens: int, step_tokens: int, block_size: int) -> int:
+        """Pages that ``requests`` requests of up to ``tokens`` tokens hold at most in this group."""
+        held = CacheManager.held_tokens_of(group, step_tokens, block_size)
         return max(1, requests * blocks_for(tokens if held < 0 else min(tokens, held), block_size))
 
     @staticmethod
     def page_bytes(cache_needs, block_size: int, dtype=torch.bfloat16) -> dict:
         """Bytes that one page of every group takes on the device, summed over the group's mixers and their tensors:
-        {window: bytes}."""
+        {group's name: bytes}."""
         out: dict = {}
         for need in _keyed(cache_needs).values():
             n = 0
@@ -97,7 +105,7 @@ class CacheManager:
                 for d in t.page_shape(block_size):
                     count *= d
                 n += count * torch.empty((), dtype=t.dtype or dtype).element_size()
-            out[need.window] = out.get(need.window, 0) + n
+            out[need.group] = out.get(need.group, 0) + n
         return out
 
     def __init__(self, cache_needs, state_needs, n_blocks, block_size: int = 16,
@@ -111,10 +119,10 @@ class CacheManager:
         self.group_of_entry: dict = {}
         cache_needs, state_needs = _keyed(cache_needs), _keyed(state_needs)
         for i, need in cache_needs.items():
-            if need.window not in windows:
-                windows.append(need.window)
+            if need.group not in windows:
+                windows.append(need.group)
                 entries.append([])
-            g = windows.index(need.window)
+            g = windows.index(need.group)
             entries[g].append(i)
             self.group_of_entry[i] = g
         if isinstance(n_blocks, dict):
@@ -129,9 +137,9 @@ class CacheManager:
         if any(n <= 0 for n in pages):
             raise AlofaError("invalid_argument", "a pool needs at least one block", f"n_blocks={n_blocks}")
         self._lib = hostlib.lib()
-        self._h = ctypes.c_void_p(self._lib.alofa_cache_new(len(windows), hostlib.long_array([-1 if w is None else w for w in windows]),
-                                                             hostlib.long_array(pages), block_size, max_requests))
-        self.groups = [Group(w, entries[g], BlockPool(0, _borrowed=self._lib.alofa_cache_pool(self._h, g))) for g, w in enumerate(windows)]
+        self._h = ctypes.c_void_p(self._lib.alofa_cache_new(len(windows), hostlib.long_array([-1 if w is None else w for w, _ in map(window_and_kept, windows)]),
+                                                             hostlib.long_array([k for _, k in map(window_and_kept, windows)]), hostlib.long_array(pages), block_size, max_requests))
+        self.groups = [Group(*window_and_kept(w), entries[g], BlockPool(0, _borrowed=self._lib.alofa_cache_pool(self._h, g))) for g, w in enumerate(windows)]
         self.requests: dict = {}      # request key -> its slot
         self.needs = cache_needs
         self.state_needs = state_needs
@@ -264,7 +272,7 @@ class CacheManager:
         A model none of whose layers keeps pages has one rule, (1, 0): nothing is held, nothing binds."""
         if not self.groups:
             return [(1, 0)]
-        return [(g.pool.n_blocks, self.held_tokens_of(g.window, step_tokens, self.block_size)) for g in self.groups]
+        return [(g.pool.n_blocks, self.held_tokens_of((g.window, g.keep_first), step_tokens, self.block_size)) for g in self.groups]
 
     def step_width(self, slots: np.ndarray, n_tokens: np.ndarray) -> int:
         """How many blocks the longest request of a step will hold once the step's tokens are in:

@@ -64,6 +64,7 @@ class ModelSpec:
     final_norm: PartSpec
     head: PartSpec
     joins: tuple = ()        # PartSpec of the "join" family: what run entries name with ``join``
+    streams: int = 0         # copies of the residual stream that the blocks work on (0: one stream, and blocks that add to it)
 
 
 class ModelConfig:

@@ -64,6 +64,18 @@ struct RopeArgs {
   const int64_t* slots;
 };
 
+// The form for two maps per head (kMaps): a head's queries and keys are two halves of d / 2 channels, each with a softmax of its own over the same
+// values. Columns 2 j and 2 j + 1 of a block are head j's two maps (`heads` and a group count columns): a column's query stands in its own
+// half and zeros in the other, so that a key's two halves side by side serve all columns, and the second product shares the values. Keys lie in the cache as
+// [block, 2 kv_heads, slot, d / 2]. A head gives a1 - lambda a2 over its root mean square over d_true channels (plus eps), times gain, as
+// one head of d channels. In this form a window may keep the first keep_first (at most 64 pages of) tokens of a sequence in sight, and scores may be
+// capped, cap tanh(s / cap) (cap 0: as they are).
+struct MapsForm {
+  int keep_first;
+  float cap, lambda, gain, eps;
+  int d_true;
+};
+
 struct Pair8 {
   uint4 lo, hi;
 };
@@ -87,14 +99,15 @@ __device__ __forceinline__ Pair8 rotate8(uint4 lo, uint4 hi, float4 c_lo, float4
 
 // DT = d / 16; NW: waves per block. blockIdx.y = key head * chunks + chunk of up to `block_heads` (<= 16) heads of its group.
 // kSplit: a weight enters the second product as two bfloat16 numbers, its rounding and what the rounding took away: sixteen bits of every weight count.
-template <int DT, int NW, bool kRope, bool kSplit = false>
+template <int DT, int NW, bool kRope, bool kSplit = false, bool kMaps = false>
 __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
     bf16_t* __restrict__ out, int64_t out_stride, float* __restrict__ partial, const bf16_t* __restrict__ q,
     int64_t q_stride, bf16_t* __restrict__ k_cache, bf16_t* __restrict__ v_cache,
     const int32_t* __restrict__ block_table, int max_blocks, const int32_t* __restrict__ req_of_token,
     const int32_t* __restrict__ positions, const int32_t* __restrict__ rows, int heads, int kv_heads,
     int bs_shift, int window, float scale, RopeArgs rope, int* __restrict__ counters, int v_head, float* __restrict__ out32, int value_heads, int64_t plane,
-    const float* __restrict__ sink, int block_heads) {
+    const float* __restrict__ sink, int block_heads, MapsForm maps) {
+  static_assert(!kMaps || (kSplit && !kRope), "two maps: with split weights, queries turned beforehand");
   static_assert(!kRope || DT % 4 == 0, "the rotation needs a channel and its partner in the same lane: d a multiple of 64");
   constexpr int d = DT * 16;
   constexpr int DS = (d + 31) / 32;            // steps of 32 along d in the first product
@@ -124,7 +137,12 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
   const int p = positions[t];
   const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
   // the visible keys lo..p lie in the 16-key tiles first..last; a wave takes a contiguous run of tiles
-  const int first = lo >> 4, last = p >> 4;
+  // (kMaps: first the tiles of the kept tokens, then the window's; a tile's number counts along both, and from `kept_tiles` on `gap` leads to its place)
+  const int keep = kMaps && window > 0 ? (maps.keep_first < p + 1 ? maps.keep_first : p + 1) : 0;
+  const int kept_tiles = kMaps ? (keep + 15) >> 4 : 0;
+  const int window_first = kMaps && kept_tiles > (lo >> 4) ? kept_tiles : lo >> 4, gap = kMaps ? window_first - kept_tiles : 0;
+  const int first = kMaps ? 0 : lo >> 4, last = kMaps ? ((p >> 4) - gap > kept_tiles - 1 ? (p >> 4) - gap : kept_tiles - 1) : p >> 4;
+  auto tile_at = [&](int tile) { return kMaps && tile >= kept_tiles ? tile + gap : tile; };
   const int per_split = (last - first + 1 + n_splits - 1) / n_splits;
   const int tile_begin = first + split * per_split;
   const int tile_end = (tile_begin + per_split < last + 1) ? tile_begin + per_split : last + 1;
@@ -138,7 +156,11 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
   for (int ds = 0; ds < DS; ++ds) {
     uint4 v = make_uint4(0, 0, 0, 0);
     const int c = ds * 32 + g * 8;
-    if (head_ok && c < d) v = *reinterpret_cast<const uint4*>(q + static_cast<int64_t>(t) * q_stride + static_cast<int64_t>(head) * d + c);
+    if constexpr (kMaps) {
+      if (head_ok && c < d && (c >= d / 2) == (head & 1)) v = *reinterpret_cast<const uint4*>(q + static_cast<int64_t>(t) * q_stride + static_cast<int64_t>(head) * (d / 2) + c % (d / 2));
+    } else {
+      if (head_ok && c < d) v = *reinterpret_cast<const uint4*>(q + static_cast<int64_t>(t) * q_stride + static_cast<int64_t>(head) * d + c);
+    }
     qf[ds] = __builtin_bit_cast(bf16x8, v);
   }
 
@@ -170,11 +192,15 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
   for (int nt = 0; nt < DT; ++nt) o[nt] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = -FLT_MAX, l = 0.f;
   const float scale2 = scale * 1.44269504088896340736f;   // scores in units of log2(e)
+  const float cap2 = kMaps ? maps.cap * 1.44269504088896340736f : 0.f, cap_in = kMaps && maps.cap > 0.f ? 2.f * scale2 / maps.cap : 0.f;
 
   // lane x holds the page of logical block page_base + x; a step's keys lie within 64 pages of its first
   // (a share whose first step lies within the first 64 pages uses the pages that set out at the start)
-  int page_base = ((((tile_begin + 2) << 4) - 1) >> bs_shift) < 64 ? 0 : (tile_begin << 4) >> bs_shift;
+  const int start = tile_at(tile_begin >= kept_tiles ? tile_begin : kept_tiles);      // (kMaps: the first of the share's tiles in the window)
+  int page_base = ((((start + 2) << 4) - 1) >> bs_shift) < 64 ? 0 : (start << 4) >> bs_shift;
   const int last_page = p >> bs_shift;
+  int kept_page = my_page;      // (kMaps: the sequence's first 64 pages, among them those of all kept tokens)
+  if constexpr (kMaps) kept_page = (my_page < 0 || lane > last_page) ? 0 : my_page;
   // (pages that a window has passed read -1: they are never used, and 0 keeps every address inside the cache)
   if (page_base != 0) {     // uniform over the wave: a share that starts past the pages already on their way
     my_page = (tile_begin < tile_end && page_base + lane <= last_page) ? table[page_base + lane] : 0;
@@ -191,25 +217,36 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
   };
   const int lo4 = lo & ~3, p4 = p & ~3;
   auto fetch = [&](int tile, Step& s) __attribute__((always_inline)) {
-    if ((((((tile + 2) << 4) - 1)) >> bs_shift) - page_base >= 64 && (tile << 4) <= p) {     // uniform over the wave
-      page_base = (tile << 4) >> bs_shift;
+    const int tile1 = tile_at(tile + 1);
+    const bool in_window = !kMaps || tile + 1 >= kept_tiles;      // (kMaps: of the step's two tiles at least the second lies there)
+    const int from = kMaps && tile < kept_tiles ? tile1 : tile_at(tile);
+    if (in_window && ((((kMaps ? tile1 + 1 : tile + 2) << 4) - 1) >> bs_shift) - page_base >= 64 && (from << 4) <= p) {     // uniform over the wave
+      page_base = (from << 4) >> bs_shift;
       my_page = (page_base + lane <= last_page) ? table[page_base + lane] : 0;
       my_page = my_page < 0 ? 0 : my_page;
     }
 #pragma unroll
     for (int kt = 0; kt < 2; ++kt) {
       // the key of this lane's row of K, and the first of this lane's four keys of V^T, brought into lo..p
-      int key = ((tile + kt) << 4) + c16, key4 = ((tile + kt) << 4) + 4 * g;
-      key = key < lo ? lo : (key > p ? p : key);
-      key4 = key4 < lo4 ? lo4 : (key4 > p4 ? p4 : key4);
+      const int at16 = tile_at(tile + kt) << 4;
+      const bool kept = kMaps && tile + kt < kept_tiles;      // (a tile of kept tokens: its pages are all held, and it may hold tokens of the window too)
+      int key = at16 + c16, key4 = at16 + 4 * g;
+      key = (key < lo && !kept) ? lo : (key > p ? p : key);
+      key4 = (key4 < lo4 && !kept) ? lo4 : (key4 > p4 ? p4 : key4);
       // (a step past the end of the share may lie before the window of pages held in the lanes: its operands are not used)
-      const int kpage = (key >> bs_shift) - page_base, vpage = (key4 >> bs_shift) - page_base;
-      const int64_t kblk = __shfl(my_page, kpage < 0 ? 0 : (kpage > 63 ? 63 : kpage), 64);
-      const int64_t vblk = __shfl(my_page, vpage < 0 ? 0 : (vpage > 63 ? 63 : vpage), 64);
+      const int base = kept ? 0 : page_base, pages = kept ? kept_page : my_page;
+      const int kpage = (key >> bs_shift) - base, vpage = (key4 >> bs_shift) - base;
+      const int64_t kblk = __shfl(pages, kpage < 0 ? 0 : (kpage > 63 ? 63 : kpage), 64);
+      const int64_t vblk = __shfl(pages, vpage < 0 ? 0 : (vpage > 63 ? 63 : vpage), 64);
 #pragma unroll
       for (int ds = 0; ds < DS; ++ds) {
         const int c = ds * 32 + g * 8;
-        s.k[kt][ds] = *reinterpret_cast<const uint4*>(k_cache + ((((kblk * kv_heads + hk) << bs_shift) + (key & bs_mask)) * d) + (c < d ? c : 0));
+        if constexpr (kMaps) {
+          const int cc = c < d ? c : 0, m = cc >= d / 2;
+          s.k[kt][ds] = *reinterpret_cast<const uint4*>(k_cache + ((((kblk * 2 * kv_heads + 2 * hk + m) << bs_shift) + (key & bs_mask)) * (d / 2)) + cc - m * (d / 2));
+        } else {
+          s.k[kt][ds] = *reinterpret_cast<const uint4*>(k_cache + ((((kblk * kv_heads + hk) << bs_shift) + (key & bs_mask)) * d) + (c < d ? c : 0));
+        }
       }
 #pragma unroll
       for (int nt = 0; nt < DT; ++nt)
@@ -224,7 +261,9 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
     // Most steps of a long context touch neither end of the visible keys nor the new token: they skip the masks and
     // the new token's insertion (branches of the whole wave with no loads inside; the results are the same bits).
     const bool last_here = kRope && tile + 1 >= last;                                                   // the step holds the new token's tile
-    const bool inner = (tile << 4) >= lo && (((tile + 2) << 4) - 1) <= p && tile + 1 < tile_end;        // every key of the step is seen
+    const int at0 = tile_at(tile) << 4, at1 = tile_at(tile + 1) << 4;
+    auto tile_seen = [&](int at) { return at >= lo || (kMaps && at + 16 <= keep); };
+    const bool inner = tile_seen(at0) && (!kMaps || tile_seen(at1)) && at1 + 15 <= p && tile + 1 < tile_end;        // every key of the step is seen
     f32x4 s[2];
 #pragma unroll
     for (int kt = 0; kt < 2; ++kt) {
@@ -246,18 +285,25 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
     // scale, mask, running maximum; the four lanes of a head agree on the maximum
     float pw[8];
     float step_max = -FLT_MAX;
+    auto scored = [&](float x) {
+      if constexpr (kMaps) {
+        // (cap tanh(s / cap) = cap - 2 cap / (exp(2 s / cap) + 1), in units of log2 e)
+        if (maps.cap > 0.f) return __builtin_fmaf(-2.f * cap2, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(cap_in * x) + 1.f), cap2);
+      }
+      return x * scale2;
+    };
     if (inner) {
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
-        pw[i] = s[i / 4][i % 4] * scale2;
+        pw[i] = scored(s[i / 4][i % 4]);
         step_max = fmaxf(step_max, pw[i]);
       }
     } else {
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
-        const int key = ((tile + i / 4) << 4) + 4 * g + i % 4;
-        const bool seen = key >= lo && key <= p && tile + i / 4 < tile_end;
-        pw[i] = seen ? s[i / 4][i % 4] * scale2 : -FLT_MAX;
+        const int key = (i < 4 ? at0 : at1) + 4 * g + i % 4;
+        const bool seen = (key >= lo || (kMaps && key < keep)) && key <= p && tile + i / 4 < tile_end;
+        pw[i] = seen ? scored(s[i / 4][i % 4]) : -FLT_MAX;
         step_max = fmaxf(step_max, pw[i]);
       }
     }
@@ -285,7 +331,13 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
     if (!inner) {
 #pragma unroll
       for (int kt = 0; kt < 2; ++kt) {
-        const int key4 = ((tile + kt) << 4) + 4 * g;
+        const int key4 = (kt == 0 ? at0 : at1) + 4 * g;
+        if constexpr (kMaps) {
+          auto hidden = [&](int key) { return (key < lo && key >= keep) || key > p; };
+          keep_x[kt] = (hidden(key4) ? 0u : 0x0000ffffu) | (hidden(key4 + 1) ? 0u : 0xffff0000u);
+          keep_y[kt] = (hidden(key4 + 2) ? 0u : 0x0000ffffu) | (hidden(key4 + 3) ? 0u : 0xffff0000u);
+          continue;
+        }
         const int lo_e = lo - key4, hi_e = p - key4 + 1;       // elements lo_e .. hi_e - 1 are visible
         keep_x[kt] = ((0 < lo_e || 0 >= hi_e) ? 0u : 0x0000ffffu) | ((1 < lo_e || 1 >= hi_e) ? 0u : 0xffff0000u);
         keep_y[kt] = ((2 < lo_e || 2 >= hi_e) ? 0u : 0x0000ffffu) | ((3 < lo_e || 3 >= hi_e) ? 0u : 0xffff0000u);
@@ -384,6 +436,44 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
   }
   __syncthreads();
 
+  // kMaps: a wave makes the end of one head at a time from both its maps' sums (`sums`(column, channel): over all states of the column)
+  auto head_end = [&](auto&& sums) __attribute__((always_inline)) {
+    constexpr int kOwn = (d + 63) / 64;
+    for (int j = wave; 2 * j < block_heads && h0 + 2 * j < group; j += NW) {      // uniform over the wave
+      float y[kOwn], ss = 0.f;
+#pragma unroll
+      for (int n = 0; n < kOwn; ++n) {
+        const int c = lane + 64 * n;
+        y[n] = c < d ? sums(2 * j, c) - maps.lambda * sums(2 * j + 1, c) : 0.f;
+        ss += y[n] * y[n];
+      }
+      ss = wave_sum(ss);
+      const float f = maps.gain / sqrtf(ss / static_cast<float>(maps.d_true) + maps.eps);
+      const int64_t at = static_cast<int64_t>(t) * out_stride + static_cast<int64_t>((hk * group + h0) / 2 + j) * d;
+#pragma unroll
+      for (int n = 0; n < kOwn; ++n)
+        if (lane + 64 * n < d) store_f32(out + at + lane + 64 * n, y[n] * f);
+    }
+  };
+  if constexpr (kMaps) {
+    if (n_parts == 1) {
+      head_end([&](int i, int c) {
+        float big = state[0][i][0];
+#pragma unroll
+        for (int w = 1; w < NW; ++w) big = fmaxf(big, state[w][i][0]);
+        float total = 0.f, acc = 0.f;
+#pragma unroll
+        for (int w = 0; w < NW; ++w) {
+          const float e = __builtin_amdgcn_exp2f(state[w][i][0] - big);
+          total += state[w][i][1] * e;
+          acc += state[w][i][4 + c] * e;
+        }
+        return acc / total;
+      });
+      return;
+    }
+  }
+
   // the waves' states are combined in wave order; thread x takes channel x % d of head x / d
   for (int x = threadIdx.x; x < block_heads * d; x += 64 * NW) {
     const int i = x / d, c = x % d;
@@ -435,6 +525,33 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
   __syncthreads();
   if (!last_block) return;
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup");
+  if constexpr (kMaps) {
+    head_end([&](int i, int c) {
+      const float* src = partial + (static_cast<int64_t>(blockIdx.x) * heads + hk * group + h0 + i) * n_parts * (d + 2);
+      float big = -FLT_MAX, total = 0.f, acc = 0.f;
+      constexpr int kMost = 8;      // (parts that are handed over; their loads set out together)
+      float ms[kMost], ls[kMost], vs[kMost];
+#pragma unroll
+      for (int u = 0; u < kMost; ++u) {
+        const float* part = src + min(u, n_parts - 1) * (d + 2);
+        ms[u] = __hip_atomic_load(part, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        ls[u] = __hip_atomic_load(part + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        vs[u] = __hip_atomic_load(part + 2 + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      }
+#pragma unroll
+      for (int u = 0; u < kMost; ++u)
+        if (u < n_parts) big = fmaxf(big, ms[u]);
+#pragma unroll
+      for (int u = 0; u < kMost; ++u)
+        if (u < n_parts) {
+          const float e = __builtin_amdgcn_exp2f(ms[u] - big);
+          total += ls[u] * e;
+          acc += vs[u] * e;
+        }
+      return acc / total;
+    });
+    return;
+  }
   for (int x = threadIdx.x; x < block_heads * d; x += 64 * NW) {
     const int i = x / d, c = x % d;
     if (h0 + i >= group) break;
@@ -566,12 +683,14 @@ extern "C" int alofa_attention_decode_can_hand_over(int tokens, int heads, int k
 // v_head >= 0: every query head's weights meet the values of that one value head (its keys stay its own key head's);
 // out32: the results go there unrounded, as float rows of `out`'s shape and stride, and `out` is not written.
 // sink: a number per query head whose exponential joins the sum of its rows' weights (null: none). block_heads: how many heads of a key head a block serves.
+// two_maps and what follows: the form for two maps per head (MapsForm).
 extern "C" int alofa_attention_decode_v(void* out, int64_t out_stride, float* partial, const void* q, int64_t q_stride,
                                         void* k_cache, void* v_cache, const int32_t* block_table,
                                         int max_blocks, const int32_t* req_of_token, const int32_t* positions,
                                         const int32_t* rows, int tokens, int heads, int kv_heads, int d, int block_size, int window,
                                         float scale, int n_splits, const float* cos_t, const float* sin_t, const int64_t* slots,
-                                        int hand_over, int v_head, float* out32, int split, int value_heads, int64_t plane, const float* sink, int block_heads, hipStream_t stream) {
+                                        int hand_over, int v_head, float* out32, int split, int value_heads, int64_t plane, const float* sink, int block_heads,
+                                        int two_maps, int keep_first, float cap, float lambda, float gain, float eps, int d_true, hipStream_t stream) {
   ALOFA_REQUIRE(block_heads >= 1 && block_heads <= kHeadsPerBlock, "attention_decode: a block serves 1 to %d heads (%d)", kHeadsPerBlock, block_heads);
   ALOFA_REQUIRE(!split || !cos_t, "attention_decode: split weights and the rotary variant do not go together");
   // value_heads > 0: all of them in one launch, value head c's results in out32 + c * plane; `tokens` then counts (token, value head) pairs
@@ -596,6 +715,13 @@ extern "C" int alofa_attention_decode_v(void* out, int64_t out_stride, float* pa
   }
   ALOFA_REQUIRE(q_stride % 8 == 0 && reinterpret_cast<uintptr_t>(q) % 16 == 0, "attention_decode: q rows must be 16-byte aligned");
   ALOFA_REQUIRE(reinterpret_cast<uintptr_t>(k_cache) % 16 == 0 && reinterpret_cast<uintptr_t>(v_cache) % 8 == 0, "attention_decode: caches must be 16-byte aligned");
+  const MapsForm maps{keep_first, cap, lambda, gain, eps, d_true};
+  if (two_maps) {      // heads counts both maps of every head; parts that a second kernel combines leave both maps' sums as they are in out32 ([tokens, heads * d])
+    ALOFA_REQUIRE(split && !cos_t && !sink && v_head < 0 && value_heads == 0 && heads % (2 * kv_heads) == 0 && block_heads % 2 == 0 && d_true > 0 && d_true <= d,
+                  "attention_decode: two maps take split weights, an even count of columns a block (%d) and a key head (%d of %d), and neither turn, sink nor other value heads", block_heads, heads, kv_heads);
+    ALOFA_REQUIRE(keep_first >= 0 && keep_first <= 64 * block_size && cap >= 0.f, "attention_decode: keep_first=%d (at most 64 pages) cap=%g", keep_first, cap);
+    ALOFA_REQUIRE(n_splits == 1 || (hand_over && n_splits <= 8) || out32, "attention_decode: %d parts of two maps need room for both maps' sums", n_splits);
+  }
   const bool fused = cos_t != nullptr;
   ALOFA_REQUIRE(!fused || (sin_t && slots && d % 64 == 0 && q_stride >= static_cast<int64_t>(heads + 2 * kv_heads) * d),
                 "attention_decode: the rotary variant needs sin, slots, rows of queries, keys and values, and a head size in steps of 64 (d=%d)", d);
@@ -604,14 +730,18 @@ extern "C" int alofa_attention_decode_v(void* out, int64_t out_stride, float* pa
   const RopeArgs rope{cos_t, sin_t, slots};
   dim3 grid(tokens, kv_heads * ((group + block_heads - 1) / block_heads), n_splits);
 #define ALOFA_DECODE(DT, NW, ROPE)                                                                                        \
-  if (split && !ROPE) attention_decode_kernel<DT, NW, false, true><<<grid, 64 * NW, 0, stream>>>(                         \
+  if (two_maps && !ROPE) attention_decode_kernel<DT, NW, false, true, true><<<grid, 64 * NW, 0, stream>>>(                 \
       static_cast<bf16_t*>(out), out_stride, partial, static_cast<const bf16_t*>(q), q_stride,                            \
       static_cast<bf16_t*>(k_cache), static_cast<bf16_t*>(v_cache), block_table, max_blocks, req_of_token,                \
-      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane, sink, block_heads);       \
+      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane, sink, block_heads, maps); \
+  else if (split && !ROPE) attention_decode_kernel<DT, NW, false, true><<<grid, 64 * NW, 0, stream>>>(                         \
+      static_cast<bf16_t*>(out), out_stride, partial, static_cast<const bf16_t*>(q), q_stride,                            \
+      static_cast<bf16_t*>(k_cache), static_cast<bf16_t*>(v_cache), block_table, max_blocks, req_of_token,                \
+      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane, sink, block_heads, maps);       \
   else attention_decode_kernel<DT, NW, ROPE><<<grid, 64 * NW, 0, stream>>>(                                                    \
       static_cast<bf16_t*>(out), out_stride, partial, static_cast<const bf16_t*>(q), q_stride,                            \
       static_cast<bf16_t*>(k_cache), static_cast<bf16_t*>(v_cache), block_table, max_blocks, req_of_token,                \
-      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane, sink, block_heads)
+      positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane, sink, block_heads, maps)
   if (fused) {
     switch (d / 64) {
       case 1: ALOFA_DECODE(4, 8, true); break;
@@ -656,5 +786,5 @@ extern "C" int alofa_attention_decode(void* out, int64_t out_stride, float* part
                                       float scale, int n_splits, const float* cos_t, const float* sin_t, const int64_t* slots,
                                       int hand_over, hipStream_t stream) {
   return alofa_attention_decode_v(out, out_stride, partial, q, q_stride, k_cache, v_cache, block_table, max_blocks, req_of_token, positions, rows, tokens,
-                                  heads, kv_heads, d, block_size, window, scale, n_splits, cos_t, sin_t, slots, hand_over, -1, nullptr, 0, 0, 0, nullptr, kHeadsPerBlock, stream);
+                                  heads, kv_heads, d, block_size, window, scale, n_splits, cos_t, sin_t, slots, hand_over, -1, nullptr, 0, 0, 0, nullptr, kHeadsPerBlock, 0, 0, 0.f, 0.f, 0.f, 0.f, d, stream);
 }

@@ -44,6 +44,21 @@ template <typename T> __device__ __forceinline__ void store_f32(T* p, float v);
 template <> __device__ __forceinline__ void store_f32<float>(float* p, float v) { *p = v; }
 template <> __device__ __forceinline__ void store_f32<bf16_t>(bf16_t* p, float v) { *p = f32_to_bf16(v); }
 
+// ---- activations of gated feed-forwards -------------------------------------
+// silu(z) = z / (1 + exp(-z)); the tanh form of gelu, z/2 (1 + tanh(c (z + 0.044715 z^3))) with c = sqrt(2/pi), is z / (1 + exp(-2 c (z + 0.044715 z^3))).
+// A product's epilogue with gate and up of the same outputs, act(gate) * up, is number 2 with silu and number 4 with gelu in every product kernel.
+__host__ __device__ constexpr bool is_gated(int epilogue) { return epilogue == 2 || epilogue == 4; }
+template <bool kGelu>
+__device__ __forceinline__ float gate_of(float z) {
+  return z / (1.f + __expf(-(kGelu ? 1.5957691216057308f * (z + 0.044715f * z * z * z) : z)));
+}
+__device__ __forceinline__ double gate_of(double z, bool gelu) {
+  return z / (1.0 + exp(-(gelu ? 1.5957691216057307118 * (z + 0.044715 * z * z * z) : z)));
+}
+__device__ __forceinline__ float gate_of(float z, bool gelu) {
+  return z / (1.f + expf(-(gelu ? 1.5957691216057308f * (z + 0.044715f * z * z * z) : z)));
+}
+
 // ---- reductions ------------------------------------------------------------
 // Sums and maxima over the 64 lanes of a wavefront ride on data-parallel-primitive moves between
 // neighbouring lanes (no trip through LDS): a scan within each row of 16 lanes (shifts by 1, 2, 4, 8),

@@ -23,7 +23,7 @@
 //
 // Epilogues: store (+ bias), add to the float residual stream, and SwiGLU, for
 // which a block computes the gate and the up product of the same columns (its
-// W slab holds as many rows of each) and writes silu(gate) * up.
+// W slab holds as many rows of each) and writes silu(gate) * up (or the tanh form of gelu in silu's place).
 #include "common.h"
 
 #include <cstdlib>
@@ -33,7 +33,7 @@ namespace alofa {
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 
-enum MfmaEpilogue : int { kMfStore = 0, kMfResidual = 1, kMfSwiglu = 2, kMfArgmax = 3 };
+enum MfmaEpilogue : int { kMfStore = 0, kMfResidual = 1, kMfSwiglu = 2, kMfArgmax = 3, kMfGeglu = 4 };
 
 constexpr int TK = 64, PAD = 8;
 constexpr int kRow = TK + PAD;  // LDS row length in elements
@@ -104,7 +104,7 @@ __device__ __forceinline__ void tile_epilogue(f32x16 (&acc)[WTM][WTN], TO* __res
                                               const float* __restrict__ bias, int M, int N, int m0, int n0, int wm, int wn, int lane) {
   constexpr int kGateTiles = WTN / 2;
   const int col = lane % 32, row_base = (lane / 32) * 4;
-  constexpr int kOutTiles = (kEpilogue == kMfSwiglu) ? kGateTiles : WTN;
+  constexpr int kOutTiles = is_gated(kEpilogue) ? kGateTiles : WTN;
 #pragma unroll
   for (int i = 0; i < WTM; ++i) {
 #pragma unroll
@@ -133,7 +133,7 @@ __device__ __forceinline__ void tile_epilogue(f32x16 (&acc)[WTM][WTN], TO* __res
           store_f32(dst, old[e] + acc[i][j][e]);
         } else {
           const float g = acc[i][j][e];
-          store_f32(dst, g / (1.f + __expf(-g)) * acc[i][(j + kGateTiles) % WTN][e]);
+          store_f32(dst, gate_of<kEpilogue == kMfGeglu>(g) * acc[i][(j + kGateTiles) % WTN][e]);
         }
       }
     }
@@ -153,7 +153,7 @@ __global__ void __launch_bounds__(256) gemm_mfma_kernel(TO* __restrict__ out, in
   constexpr int TM = 64 * WTM, TN = 64 * WTN;
   // swiglu: the first half of a wave's column tiles are gate columns, the second half the up columns of the same outputs
   constexpr int kGateTiles = WTN / 2;
-  static_assert(kEpilogue != kMfSwiglu || WTN % 2 == 0, "the swiglu epilogue needs an even number of column tiles per wave");
+  static_assert(!is_gated(kEpilogue) || WTN % 2 == 0, "the swiglu epilogue needs an even number of column tiles per wave");
   __shared__ int last_block;
   const TilePlace place = place_tile(blockIdx.x, tiles_m, tiles_n, shares, by_die != 0);
   // this block's share of K: slabs [k_begin, K)
@@ -167,7 +167,7 @@ __global__ void __launch_bounds__(256) gemm_mfma_kernel(TO* __restrict__ out, in
   __shared__ __attribute__((aligned(16))) bf16_t Ws[TN * kRow];
   const int tid = threadIdx.x, wave = tid / 64, lane = tid % 64;
   const int wm = wave / 2, wn = wave % 2;
-  constexpr int kOutCols = (kEpilogue == kMfSwiglu) ? TN / 2 : TN;
+  constexpr int kOutCols = is_gated(kEpilogue) ? TN / 2 : TN;
   const int m0 = place.bm * TM, n0 = place.bn * kOutCols;
 
   // global -> register staging: 8 chunks of 16 bytes per slab row; a thread takes row (tid + 256 j) / 8
@@ -187,7 +187,7 @@ __global__ void __launch_bounds__(256) gemm_mfma_kernel(TO* __restrict__ out, in
     const int row = (tid + 256 * j) / 8;
     int n = n0 + row;
     const bf16_t* base = W;
-    if (kEpilogue == kMfSwiglu && row >= TN / 2) {  // slab rows below TN / 2: gate rows n0 ..; the others: up rows of the same columns
+    if (is_gated(kEpilogue) && row >= TN / 2) {  // slab rows below TN / 2: gate rows n0 ..; the others: up rows of the same columns
       n = n0 + row - TN / 2;
       base = W2;
     }
@@ -237,7 +237,7 @@ __global__ void __launch_bounds__(256) gemm_mfma_kernel(TO* __restrict__ out, in
 #pragma unroll
   for (int j = 0; j < WTN; ++j) {
     int row = wn * 32 * WTN + j * 32 + frag_row;
-    if (kEpilogue == kMfSwiglu)   // this wave's 32 kGateTiles output columns: their gate rows, then their up rows
+    if (is_gated(kEpilogue))   // this wave's 32 kGateTiles output columns: their gate rows, then their up rows
       row = (j < kGateTiles) ? wn * 32 * kGateTiles + j * 32 + frag_row : TN / 2 + wn * 32 * kGateTiles + (j - kGateTiles) * 32 + frag_row;
     w_off[j] = row * kRow + frag_k;
   }
@@ -370,7 +370,7 @@ __global__ void __launch_bounds__(256) gemm_dma_kernel(TO* __restrict__ out, int
   constexpr int kGateTiles = WTN / 2;
   // (swiglu with WTN = 1: the waves of column 0 take 32 gate columns, those of column 1 the up columns of the same
   // outputs, and the two meet in LDS after the last slab)
-  static_assert(kEpilogue != kMfSwiglu || WTN % 2 == 0 || WTN == 1, "the swiglu epilogue needs an even number of column tiles per wave, or one");
+  static_assert(!is_gated(kEpilogue) || WTN % 2 == 0 || WTN == 1, "the swiglu epilogue needs an even number of column tiles per wave, or one");
   constexpr int kRows = TM + TN;               // slab rows: A's, then W's
   constexpr int kStageBytes = kRows * 128;
   constexpr int kLoads = kRows / 32;           // fetch instructions per wave and slab (each brings eight rows)
@@ -379,7 +379,7 @@ __global__ void __launch_bounds__(256) gemm_dma_kernel(TO* __restrict__ out, int
   const TilePlace place = place_tile(blockIdx.x, tiles_m, tiles_n, kSplitK ? shares : 1, by_die != 0);
   const int tid = threadIdx.x, wave = tid / 64, lane = tid % 64;
   const int wm = wave / 2, wn = wave % 2;
-  constexpr int kOutCols = (kEpilogue == kMfSwiglu) ? TN / 2 : TN;
+  constexpr int kOutCols = is_gated(kEpilogue) ? TN / 2 : TN;
   // (own: the output columns a block owns of those its tile holds, all of them if 0: see launch_dma. The columns
   // beyond are fetched from the last owned one, which costs no memory traffic, and never stored.)
   const int owned = own > 0 ? own : kOutCols;
@@ -397,7 +397,7 @@ __global__ void __launch_bounds__(256) gemm_dma_kernel(TO* __restrict__ out, int
       const int row = r - TM;
       int n = n0 + row;
       const bf16_t* base = W;
-      if (kEpilogue == kMfSwiglu && row >= TN / 2) {   // slab rows below TN / 2: gate rows n0 ..; the others: up rows of the same columns
+      if (is_gated(kEpilogue) && row >= TN / 2) {   // slab rows below TN / 2: gate rows n0 ..; the others: up rows of the same columns
         n = n0 + row - TN / 2;
         base = W2;
       }
@@ -429,13 +429,13 @@ __global__ void __launch_bounds__(256) gemm_dma_kernel(TO* __restrict__ out, int
   // fragments: lane l reads row l % 32 of its 32-row group, chunk 2 q + l / 32 in step q of the slab's four
   const int sw = swz(lane % 32), half = lane / 32;
   const int a_row = (wm * 32 * WTM + lane % 32) * 128;
-  const int w_row = (TM + wn * 32 * (kEpilogue == kMfSwiglu ? (WTN == 1 ? 1 : kGateTiles) : WTN) + lane % 32) * 128;
+  const int w_row = (TM + wn * 32 * (is_gated(kEpilogue) ? (WTN == 1 ? 1 : kGateTiles) : WTN) + lane % 32) * 128;
   int place_of[4];
 #pragma unroll
   for (int q = 0; q < 4; ++q) place_of[q] = ((2 * q + half) ^ sw) * 16;
   auto w_group = [&](int j) {      // byte offset of this wave's j-th 32-row group of W within the slab's W rows
-    if (kEpilogue == kMfSwiglu && WTN == 1) return 0;
-    if (kEpilogue == kMfSwiglu) return (j < kGateTiles ? j * 32 : TN / 2 + (j - kGateTiles) * 32) * 128;
+    if (is_gated(kEpilogue) && WTN == 1) return 0;
+    if (is_gated(kEpilogue)) return (j < kGateTiles ? j * 32 : TN / 2 + (j - kGateTiles) * 32) * 128;
     return j * 32 * 128;
   };
 
@@ -484,7 +484,7 @@ __global__ void __launch_bounds__(256) gemm_dma_kernel(TO* __restrict__ out, int
     read(k);
     multiply();
   }
-  if constexpr (kEpilogue == kMfSwiglu && WTN == 1) {
+  if constexpr (is_gated(kEpilogue) && WTN == 1) {
     __syncthreads();      // every wave has read the last slab: the ring is free
     float* meet = reinterpret_cast<float*>(ring);     // [wm][i][e][lane]
     if (wn == 1) {
@@ -503,7 +503,7 @@ __global__ void __launch_bounds__(256) gemm_dma_kernel(TO* __restrict__ out, int
         for (int e = 0; e < 16; ++e) {
           const int m = m_first + 8 * (e / 4) + e % 4;
           const float g = acc[i][0][e], up = meet[((wm * WTM + i) * 16 + e) * 64 + lane];
-          if (m < M && n < n_end) store_f32(out + static_cast<int64_t>(m) * ldo + n, g / (1.f + __expf(-g)) * up);
+          if (m < M && n < n_end) store_f32(out + static_cast<int64_t>(m) * ldo + n, gate_of<kEpilogue == kMfGeglu>(g) * up);
         }
       }
     }
@@ -582,13 +582,13 @@ __global__ void __launch_bounds__(64 * WM * WN) gemm_wide_kernel(TO* __restrict_
   constexpr int kLoads = kRows / 16 / kWaves;        // fetch instructions per wave and slab (each brings sixteen rows)
   constexpr int TI = TM / 32 / WM, TJ = TN / 32 / WN;   // 32 x 32 tiles a wave
   static_assert(kRows % (16 * kWaves) == 0 && TM % (32 * WM) == 0 && TN % (32 * WN) == 0, "the tile must divide among the waves");
-  static_assert(kEpilogue != kMfSwiglu || TJ % 2 == 0, "the swiglu epilogue needs gate and up tiles in every wave");
+  static_assert(!is_gated(kEpilogue) || TJ % 2 == 0, "the swiglu epilogue needs gate and up tiles in every wave");
   constexpr int kGateTiles = TJ / 2;
   __shared__ __attribute__((aligned(1024))) char ring[S * kStageBytes];
   const TilePlace place = place_tile(blockIdx.x, tiles_m, tiles_n, 1, true);
   const int tid = threadIdx.x, wave = tid / 64, lane = tid % 64;
   const int wm = wave / WN, wn = wave % WN;
-  constexpr int kOutCols = (kEpilogue == kMfSwiglu) ? TN / 2 : TN;
+  constexpr int kOutCols = is_gated(kEpilogue) ? TN / 2 : TN;
   const int m0 = place.bm * TM, n0 = place.bn * kOutCols;
 
   // what this lane fetches: instruction j of this wave brings slab rows 16 (kWaves j + wave) .. + 15, lane l place l % 4 of row l / 4
@@ -602,7 +602,7 @@ __global__ void __launch_bounds__(64 * WM * WN) gemm_wide_kernel(TO* __restrict_
       const int row = r - TM;
       int n = n0 + row;
       const bf16_t* base = W;
-      if (kEpilogue == kMfSwiglu && row >= TN / 2) {
+      if (is_gated(kEpilogue) && row >= TN / 2) {
         n = n0 + row - TN / 2;
         base = W2;
       }
@@ -636,7 +636,7 @@ __global__ void __launch_bounds__(64 * WM * WN) gemm_wide_kernel(TO* __restrict_
 #pragma unroll
   for (int q = 0; q < 2; ++q) place_of[q] = ((2 * q + half) ^ sw) * 16;
   auto w_group = [&](int j) {      // byte offset of this wave's j-th 32-row group within the slab's W rows
-    if (kEpilogue == kMfSwiglu) return ((j < kGateTiles ? 0 : TN / 2) + (wn * kGateTiles + j % kGateTiles) * 32) * 64;
+    if (is_gated(kEpilogue)) return ((j < kGateTiles ? 0 : TN / 2) + (wn * kGateTiles + j % kGateTiles) * 32) * 64;
     return (wn * TJ + j) * 32 * 64;
   };
   auto step = [&](int slab) {
@@ -680,7 +680,7 @@ __global__ void __launch_bounds__(64 * WM * WN) gemm_wide_kernel(TO* __restrict_
 template <int kEpilogue, typename TO, int TM, int TN, int WM, int WN, int S>
 static int launch_wide(void* out, int64_t ldo, const void* A, int64_t lda, const void* W, int64_t ldw, const float* bias, int M, int N, int K,
                        hipStream_t stream, const void* W2 = nullptr) {
-  constexpr int kOutCols = (kEpilogue == kMfSwiglu) ? TN / 2 : TN;
+  constexpr int kOutCols = is_gated(kEpilogue) ? TN / 2 : TN;
   const int tiles_n = (N + kOutCols - 1) / kOutCols, tiles_m = (M + TM - 1) / TM;
   gemm_wide_kernel<kEpilogue, TO, TM, TN, WM, WN, S><<<tiles_n * tiles_m, 64 * WM * WN, 0, stream>>>(
       static_cast<TO*>(out), ldo, static_cast<const bf16_t*>(A), lda, static_cast<const bf16_t*>(W), static_cast<const bf16_t*>(W2), ldw, bias, M, N, K,
@@ -699,7 +699,7 @@ template <int kEpilogue>
 static bool wide_pays(int M, int N, int K) {
   static const bool switched_off = [] { const char* e = getenv("ALOFA_WIDE_TILES"); return e != nullptr && e[0] == '0'; }();     // (for measurements)
   if (switched_off || M <= 128 || K % 32 != 0 || K < 2048) return false;
-  constexpr int kOutCols = (kEpilogue == kMfSwiglu) ? 128 : 256;
+  constexpr int kOutCols = is_gated(kEpilogue) ? 128 : 256;
   const int64_t tiles = static_cast<int64_t>((M + 255) / 256) * ((N + kOutCols - 1) / kOutCols), units = compute_units();
   const int64_t rounds = (tiles + units - 1) / units;
   return tiles * 5 >= rounds * units * 4;
@@ -715,7 +715,7 @@ static int launch_tile(int tiles_n, int tiles_m, int shares, void* out, int64_t 
                   "gemm_mfma: %lld tiles in %d shares of K do not fit the workspace", static_cast<long long>(tiles), shares);
   }
   // operands beyond what the eight L2s hold together (4 MB each)
-  const int w_rows = (kEpilogue == kMfSwiglu) ? 2 * N : N;
+  const int w_rows = is_gated(kEpilogue) ? 2 * N : N;
   const int by_die = (static_cast<int64_t>(M) + w_rows) * K * 2 > (32 << 20);
   gemm_mfma_kernel<kEpilogue, TO, WTM, WTN, PF, kSplitK><<<tiles_n * tiles_m * shares, 256, 0, stream>>>(
       static_cast<TO*>(out), ldo, static_cast<const bf16_t*>(A), lda, static_cast<const bf16_t*>(W),
@@ -878,7 +878,7 @@ static int launch_dma_sliced(void* out, int64_t ldo, const void* A, int64_t lda,
 template <int kEpilogue, typename TO, int WTM, int WTN, int S>
 static int launch_dma(void* out, int64_t ldo, const void* A, int64_t lda, const void* W, int64_t ldw, const float* bias, int M, int N, int K,
                       hipStream_t stream, const void* W2 = nullptr, int own = 0) {
-  constexpr int kOutCols = (kEpilogue == kMfSwiglu) ? 32 * WTN : 64 * WTN;     // (gate and up rows of the same columns share a slab)
+  constexpr int kOutCols = is_gated(kEpilogue) ? 32 * WTN : 64 * WTN;     // (gate and up rows of the same columns share a slab)
   const int owned = (own > 0 && own < kOutCols) ? own : kOutCols;
   const int tiles_n = (N + owned - 1) / owned, tiles_m = (M + 64 * WTM - 1) / (64 * WTM);
   // (tiles dealt out die by die at every size: with weights that come from memory it is 3 to 9 % faster here than row
@@ -933,7 +933,7 @@ static int launch_mfma(void* out, int64_t ldo, const void* A, int64_t lda, const
       return check_launch("gemm_wide");
     }
   }
-  if constexpr (kEpilogue == kMfSwiglu) {
+  if constexpr (is_gated(kEpilogue)) {
     // A block computes gate and up of the same 64 columns. With K a multiple of 64 and tiles that do not fill the
     // chip twice over, the slabs go straight from memory into a ring in LDS (0.5B sizes, us against the kernel
     // that brings them in through registers with 128-row tiles, one slab ahead):
@@ -1068,15 +1068,15 @@ static int launch_mfma(void* out, int64_t ldo, const void* A, int64_t lda, const
       // N = 2,048, K = 11,008 at 128 rows 22.2 against 24.8)
       const int wide_tiles = ((N + 127) / 128) * tiles_m, all_slabs = K / TK;
       const int per_share = max(4, (all_slabs * wide_tiles + 255) / 256), slices = (all_slabs + per_share - 1) / per_share;
-      if (kEpilogue != kMfSwiglu && ring && long_k && (M <= 64 || (M <= 256 && !tall && K >= 3072)) && wide_tiles <= 36 && N % 4 == 0 && slices > 1 &&
+      if (!is_gated(kEpilogue) && ring && long_k && (M <= 64 || (M <= 256 && !tall && K >= 3072)) && wide_tiles <= 36 && N % 4 == 0 && slices > 1 &&
           static_cast<int64_t>(slices) * M * N <= workspace().tile_floats) {
-        if constexpr (kEpilogue != kMfSwiglu) {
+        if constexpr (!is_gated(kEpilogue)) {
           if (launch_dma_sliced<kEpilogue, TO, 2, 4>(out, ldo, A, lda, W, ldw, bias, M, N, K, slices, stream, then, then_done)) return 1;
         }
       } else
-      if (tall && kEpilogue != kMfSwiglu && ring && N % 4 == 0 &&
+      if (tall && !is_gated(kEpilogue) && ring && N % 4 == 0 &&
           static_cast<int64_t>(tall_shares) * M * N <= workspace().tile_floats) {
-        if constexpr (kEpilogue != kMfSwiglu) {
+        if constexpr (!is_gated(kEpilogue)) {
           if (launch_dma_sliced<kEpilogue, TO, 2, 3, 2>(out, ldo, A, lda, W, ldw, bias, M, N, K, tall_shares, stream, then, then_done)) return 1;
         }
       } else
@@ -1114,7 +1114,7 @@ static int launch_mfma(void* out, int64_t ldo, const void* A, int64_t lda, const
 using namespace alofa;
 
 // bfloat16 A [M, K] and W [N, K] (W2 for the swiglu epilogue); K a multiple of 8, rows 16-byte
-// aligned. Epilogues: 0 store (+ bias) as o_dtype, 1 add to the float residual, 2 swiglu.
+// aligned. Epilogues: 0 store (+ bias) as o_dtype, 1 add to the float residual, 2 swiglu, 4 the same with gelu.
 // then_w (may be null; residual epilogue only): an RMSNorm (then_w [N], then_eps) of the residual's new rows is
 // wanted in then_out (bfloat16 [M, then_ld]) afterwards. Where the product's last launch has whole rows in hand it
 // writes them and sets *then_done to 1; otherwise *then_done stays 0 and the norm is the caller's to run.
@@ -1144,6 +1144,10 @@ extern "C" int alofa_gemm_mfma(void* out, int o_dtype, int64_t ldo, const void* 
     ALOFA_REQUIRE(W2 != nullptr, "gemm_mfma: the swiglu epilogue needs the up matrix");
     return launch_mfma<kMfSwiglu, bf16_t>(out, ldo, A, lda, W, W2, ldw, nullptr, M, N, K, stream, kNoNorm, done);
   }
+  if (epilogue == kMfGeglu && o_dtype == kBF16) {
+    ALOFA_REQUIRE(W2 != nullptr, "gemm_mfma: the geglu epilogue needs the up matrix");
+    return launch_mfma<kMfGeglu, bf16_t>(out, ldo, A, lda, W, W2, ldw, nullptr, M, N, K, stream, kNoNorm, done);
+  }
   ALOFA_REQUIRE(false, "gemm_mfma: unsupported epilogue %d with out dtype %d", epilogue, o_dtype);
 }
 
@@ -1163,6 +1167,7 @@ extern "C" int alofa_gemm_wide(void* out, int o_dtype, int64_t ldo, const void* 
   else if (epilogue == kMfStore && o_dtype == kF32) failed = launch_wide<kMfStore, float, 256, 256, 4, 2, 4>(out, ldo, A, lda, W, ldw, bias, M, N, K, stream);
   else if (epilogue == kMfResidual && o_dtype == kF32) failed = launch_wide<kMfResidual, float, 256, 256, 4, 2, 4>(out, ldo, A, lda, W, ldw, nullptr, M, N, K, stream);
   else if (epilogue == kMfSwiglu && o_dtype == kBF16 && W2 != nullptr) failed = launch_wide<kMfSwiglu, bf16_t, 256, 256, 4, 2, 4>(out, ldo, A, lda, W, ldw, nullptr, M, N, K, stream, W2);
+  else if (epilogue == kMfGeglu && o_dtype == kBF16 && W2 != nullptr) failed = launch_wide<kMfGeglu, bf16_t, 256, 256, 4, 2, 4>(out, ldo, A, lda, W, ldw, nullptr, M, N, K, stream, W2);
   else ALOFA_REQUIRE(false, "gemm_wide: unsupported epilogue %d with out dtype %d", epilogue, o_dtype);
   if (failed) return 1;
   return check_launch("gemm_wide");

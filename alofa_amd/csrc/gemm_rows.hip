@@ -30,7 +30,7 @@ namespace alofa {
 
 typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
 
-enum RowsEpilogue : int { kRwStore = 0, kRwResidual = 1, kRwSwiglu = 2 };
+enum RowsEpilogue : int { kRwStore = 0, kRwResidual = 1, kRwSwiglu = 2, kRwGeglu = 4 };
 
 constexpr int kRowsMaxWaves = 12;     // runs of 512 along K, one per wave
 constexpr int kRowsMaxK = kRowsMaxWaves * 512;
@@ -102,7 +102,7 @@ __global__ void __launch_bounds__(64 * kMaxWaves) gemm_rows_kernel(
     TO* __restrict__ out, int64_t ldo, const void* __restrict__ A, int64_t lda, const bf16_t* __restrict__ W,
     const bf16_t* __restrict__ W2, int64_t ldw, const float* __restrict__ bias, int M, int N, int K,
     const float* __restrict__ norm_w, float eps) {
-  constexpr int kMats = (kEpilogue == kRwSwiglu) ? 2 : 1;
+  constexpr int kMats = is_gated(kEpilogue) ? 2 : 1;
   constexpr int V = C * MR;                                // partial sums per lane and matrix
   __shared__ float red[kMaxWaves][kMats][V];
   __shared__ float ssq[kNorm ? kMaxWaves : 1][MR];
@@ -206,7 +206,7 @@ __global__ void __launch_bounds__(64 * kMaxWaves) gemm_rows_kernel(
   if (!finisher) return;
   float sum = red[0][0][threadIdx.x], up = 0.f;
   for (int w = 1; w < n_waves; ++w) sum += red[w][0][threadIdx.x];
-  if constexpr (kEpilogue == kRwSwiglu) {
+  if constexpr (is_gated(kEpilogue)) {
     up = red[0][1][threadIdx.x];
     for (int w = 1; w < n_waves; ++w) up += red[w][1][threadIdx.x];
   }
@@ -224,7 +224,7 @@ __global__ void __launch_bounds__(64 * kMaxWaves) gemm_rows_kernel(
   } else if (kEpilogue == kRwResidual) {
     store_f32(dst, add + sum);
   } else {
-    store_f32(dst, sum / (1.f + __expf(-sum)) * up);
+    store_f32(dst, gate_of<kEpilogue == kRwGeglu>(sum) * up);
   }
 }
 
@@ -315,7 +315,7 @@ static int launch_rows(void* out, int64_t ldo, const void* A, int64_t lda, const
   const int waves = (K + 511) / 512;
   const dim3 grid((N + C - 1) / C);
   if (waves > kRowsMaxWaves) {
-    if constexpr (!kNorm && kEpilogue != kRwSwiglu && MR <= 8) {
+    if constexpr (!kNorm && !is_gated(kEpilogue) && MR <= 8) {
       gemm_rows_long_kernel<MR, C, kEpilogue, TO><<<grid, 64 * rows_long_waves(MR), 0, stream>>>(
           static_cast<TO*>(out), ldo, static_cast<const bf16_t*>(A), lda, static_cast<const bf16_t*>(W), ldw, bias, M, N, K);
       return check_launch("gemm_rows (long K)");
@@ -341,11 +341,11 @@ static int dispatch_rows(void* out, int64_t ldo, const void* A, int64_t lda, con
                          const float* bias, int M, int N, int K, const float* norm_w, float eps, hipStream_t stream) {
   // (gate and up: eight columns of either, so that the rows, which every block reads and, with a norm, converts,
   // are read half as often where the blocks are many)
-  constexpr int C = (kEpilogue == kRwSwiglu) ? 8 : 4;
+  constexpr int C = is_gated(kEpilogue) ? 8 : 4;
   if (M <= 1) return launch_rows<1, C, kEpilogue, TO, kNorm>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, norm_w, eps, stream);
   if (M <= 2) return launch_rows<2, C, kEpilogue, TO, kNorm>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, norm_w, eps, stream);
   if (M <= 4) return launch_rows<4, C, kEpilogue, TO, kNorm>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, norm_w, eps, stream);
-  if constexpr (!kNorm && kEpilogue != kRwSwiglu) {
+  if constexpr (!kNorm && !is_gated(kEpilogue)) {
     if (M > 8) return launch_rows<16, C, kEpilogue, TO, kNorm>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, norm_w, eps, stream);
   }
   return launch_rows<8, C, kEpilogue, TO, kNorm>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, norm_w, eps, stream);
@@ -369,7 +369,7 @@ extern "C" int alofa_gemm_rows_fits(int M, int N, int K, int plain) {
 extern "C" int alofa_gemm_rows(void* out, int o_dtype, int64_t ldo, const void* A, int64_t lda, const void* W,
                                const void* W2, int64_t ldw, const float* bias, int M, int N, int K, int epilogue,
                                const float* norm_w, float eps, hipStream_t stream) {
-  ALOFA_REQUIRE(alofa_gemm_rows_fits(M, N, K, norm_w == nullptr && epilogue != kRwSwiglu),
+  ALOFA_REQUIRE(alofa_gemm_rows_fits(M, N, K, norm_w == nullptr && !is_gated(epilogue)),
                 "gemm_rows: M=%d (1..8; to 16 for plain products of K up to 6,144) N=%d K=%d (a multiple of 8; beyond %d with the store and residual epilogues of bfloat16 rows only)", M, N, K, kRowsMaxK);
   ALOFA_REQUIRE(ldw % 8 == 0 && reinterpret_cast<uintptr_t>(W) % 16 == 0 && (W2 == nullptr || reinterpret_cast<uintptr_t>(W2) % 16 == 0),
                 "gemm_rows: rows of W must be 16-byte aligned");
@@ -379,6 +379,7 @@ extern "C" int alofa_gemm_rows(void* out, int o_dtype, int64_t ldo, const void* 
   if (norm_w != nullptr) {
     if (epilogue == kRwStore && o_dtype == kBF16) return dispatch_rows<kRwStore, bf16_t, true>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, norm_w, eps, stream);
     if (epilogue == kRwSwiglu && o_dtype == kBF16 && W2) return dispatch_rows<kRwSwiglu, bf16_t, true>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, norm_w, eps, stream);
+    if (epilogue == kRwGeglu && o_dtype == kBF16 && W2) return dispatch_rows<kRwGeglu, bf16_t, true>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, norm_w, eps, stream);
     ALOFA_REQUIRE(false, "gemm_rows: the norm goes with the bfloat16 store and swiglu epilogues only");
     return 1;
   }
@@ -386,6 +387,7 @@ extern "C" int alofa_gemm_rows(void* out, int o_dtype, int64_t ldo, const void* 
   if (epilogue == kRwStore && o_dtype == kF32) return dispatch_rows<kRwStore, float, false>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, nullptr, 0.f, stream);
   if (epilogue == kRwResidual && o_dtype == kF32) return dispatch_rows<kRwResidual, float, false>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, nullptr, 0.f, stream);
   if (epilogue == kRwSwiglu && o_dtype == kBF16 && W2) return dispatch_rows<kRwSwiglu, bf16_t, false>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, nullptr, 0.f, stream);
+  if (epilogue == kRwGeglu && o_dtype == kBF16 && W2) return dispatch_rows<kRwGeglu, bf16_t, false>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, nullptr, 0.f, stream);
   ALOFA_REQUIRE(false, "gemm_rows: no kernel for epilogue %d with output type %d", epilogue, o_dtype);
   return 1;
 }

@@ -83,13 +83,13 @@ __global__ void __launch_bounds__(256) gemm_simple_kernel(TO* __restrict__ out, 
   }
 }
 
-// out[m, n] = silu(A Wg^T)[m, n] * (A Wu^T)[m, n]: both products are rounded to
-// float first, then x / (1 + exp(-x)) * u in Acc.
+// out[m, n] = act(A Wg^T)[m, n] * (A Wu^T)[m, n] with silu or the tanh form of gelu: both products are rounded to
+// float first, then the activation and the product in Acc.
 template <typename TA, typename TW, typename TO, typename Acc>
 __global__ void __launch_bounds__(256) gemm_swiglu_simple_kernel(TO* __restrict__ out, int64_t ldo,
                                                                  const TA* __restrict__ A, int64_t lda,
                                                                  const TW* __restrict__ Wg, const TW* __restrict__ Wu,
-                                                                 int64_t ldw, int M, int N, int K) {
+                                                                 int64_t ldw, int M, int N, int K, int gelu) {
   __shared__ Acc As[BK][BM + 1];
   __shared__ Acc Gs[BK][BN + 1];
   __shared__ Acc Us[BK][BN + 1];
@@ -138,7 +138,7 @@ __global__ void __launch_bounds__(256) gemm_swiglu_simple_kernel(TO* __restrict_
       if (n >= N) continue;
       const Acc gv = static_cast<Acc>(static_cast<float>(g[i][j]));
       const Acc uv = static_cast<Acc>(static_cast<float>(u[i][j]));
-      store_f32(out + static_cast<int64_t>(m) * ldo + n, static_cast<float>(gv / (Acc(1) + exp(-gv)) * uv));
+      store_f32(out + static_cast<int64_t>(m) * ldo + n, static_cast<float>(gate_of(gv, gelu != 0) * uv));
     }
   }
 }
@@ -158,10 +158,10 @@ static int launch_gemm(void* out, int64_t ldo, const void* A, int64_t lda, const
 
 template <typename TA, typename TW, typename TO, typename Acc>
 static int launch_gemm_swiglu(void* out, int64_t ldo, const void* A, int64_t lda, const void* Wg, const void* Wu,
-                              int64_t ldw, int M, int N, int K, hipStream_t stream) {
+                              int64_t ldw, int M, int N, int K, int gelu, hipStream_t stream) {
   dim3 grid((N + BN - 1) / BN, (M + BM - 1) / BM);
   gemm_swiglu_simple_kernel<TA, TW, TO, Acc><<<grid, 256, 0, stream>>>(static_cast<TO*>(out), ldo, static_cast<const TA*>(A), lda,
-                                                                       static_cast<const TW*>(Wg), static_cast<const TW*>(Wu), ldw, M, N, K);
+                                                                       static_cast<const TW*>(Wg), static_cast<const TW*>(Wu), ldw, M, N, K, gelu);
   return check_launch("gemm_swiglu_simple");
 }
 
@@ -195,18 +195,18 @@ extern "C" int alofa_gemm_simple(void* out, int o_dtype, int64_t ldo, const void
 
 extern "C" int alofa_gemm_swiglu_simple(void* out, int o_dtype, int64_t ldo, const void* A, int a_dtype, int64_t lda,
                                         const void* Wg, const void* Wu, int w_dtype, int64_t ldw, int M, int N,
-                                        int K, int exact, hipStream_t stream) {
+                                        int K, int gelu, int exact, hipStream_t stream) {
   ALOFA_REQUIRE(M > 0 && N > 0 && K > 0, "gemm_swiglu: M=%d N=%d K=%d must be positive", M, N, K);
   ALOFA_REQUIRE(lda >= K && ldw >= K && ldo >= N, "gemm_swiglu: a leading dimension is shorter than its row");
   if (exact) {
     ALOFA_REQUIRE(a_dtype == kF32 && w_dtype == kF32 && o_dtype == kF32, "gemm_swiglu: the exact path takes float operands only");
-    return launch_gemm_swiglu<float, float, float, double>(out, ldo, A, lda, Wg, Wu, ldw, M, N, K, stream);
+    return launch_gemm_swiglu<float, float, float, double>(out, ldo, A, lda, Wg, Wu, ldw, M, N, K, gelu, stream);
   }
   if (a_dtype == kBF16 && w_dtype == kBF16 && o_dtype == kBF16)
-    return launch_gemm_swiglu<bf16_t, bf16_t, bf16_t, float>(out, ldo, A, lda, Wg, Wu, ldw, M, N, K, stream);
+    return launch_gemm_swiglu<bf16_t, bf16_t, bf16_t, float>(out, ldo, A, lda, Wg, Wu, ldw, M, N, K, gelu, stream);
   if (a_dtype == kBF16 && w_dtype == kF32 && o_dtype == kBF16)
-    return launch_gemm_swiglu<bf16_t, float, bf16_t, float>(out, ldo, A, lda, Wg, Wu, ldw, M, N, K, stream);
+    return launch_gemm_swiglu<bf16_t, float, bf16_t, float>(out, ldo, A, lda, Wg, Wu, ldw, M, N, K, gelu, stream);
   if (a_dtype == kF32 && w_dtype == kF32 && o_dtype == kF32)
-    return launch_gemm_swiglu<float, float, float, float>(out, ldo, A, lda, Wg, Wu, ldw, M, N, K, stream);
+    return launch_gemm_swiglu<float, float, float, float>(out, ldo, A, lda, Wg, Wu, ldw, M, N, K, gelu, stream);
   ALOFA_REQUIRE(false, "gemm_swiglu: unsupported dtype mix a=%d w=%d o=%d", a_dtype, w_dtype, o_dtype);
 }

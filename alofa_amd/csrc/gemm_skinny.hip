@@ -36,7 +36,7 @@ namespace alofa {
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
-enum SkinnyEpilogue : int { kSkStore = 0, kSkResidual = 1, kSkSwiglu = 2 };
+enum SkinnyEpilogue : int { kSkStore = 0, kSkResidual = 1, kSkSwiglu = 2, kSkGeglu = 4 };
 
 
 // A partial sum leaves for the workspace at device scope: written through to memory, past this
@@ -113,9 +113,9 @@ __global__ void __launch_bounds__(kWaves * 64) gemm_skinny_kernel(
   bool w_ok[NT];
 #pragma unroll
   for (int nt = 0; nt < NT; ++nt) {
-    const int n = (kEpilogue == kSkSwiglu) ? n0 + r : n0 + nt * 16 + r;
+    const int n = is_gated(kEpilogue) ? n0 + r : n0 + nt * 16 + r;
     w_ok[nt] = n < N && n - n0 < cols;
-    const bf16_t* base = (kEpilogue == kSkSwiglu && nt == 1) ? W2 : W;
+    const bf16_t* base = (is_gated(kEpilogue) && nt == 1) ? W2 : W;
     w_row[nt] = base + static_cast<int64_t>(w_ok[nt] ? n : 0) * ldw;
   }
 
@@ -127,7 +127,7 @@ __global__ void __launch_bounds__(kWaves * 64) gemm_skinny_kernel(
 
   // What the epilogue adds (the bias, or the residual stream's old values) sets out now and has arrived when
   // the sums are ready: this wave finishes tiles wave, wave + kWaves, ...
-  constexpr int kOutTiles = (kEpilogue == kSkSwiglu) ? MT : MT * NT;
+  constexpr int kOutTiles = is_gated(kEpilogue) ? MT : MT * NT;
   constexpr int kMyTiles = (kOutTiles + kWaves - 1) / kWaves;
   // With so few output tiles that they would leave most waves without work at the end (one or two), and K not
   // shared out over blocks, every thread finishes one output instead (`flat` below): thread x the x-th float of
@@ -135,8 +135,8 @@ __global__ void __launch_bounds__(kWaves * 64) gemm_skinny_kernel(
   constexpr bool kFlatTail = kOutTiles * 4 <= kWaves;
   const bool flat = kFlatTail && gridDim.y == 1;
   const int f_tile = threadIdx.x >> 8, f_r = (threadIdx.x >> 2) & 15, f_g = (threadIdx.x >> 6) & 3, f_i = threadIdx.x & 3;
-  const int f_mt = (kEpilogue == kSkSwiglu) ? f_tile : f_tile / NT, f_nt = (kEpilogue == kSkSwiglu) ? 0 : f_tile % NT;
-  const int f_m = f_mt * 16 + f_g * 4 + f_i, f_n = (kEpilogue == kSkSwiglu) ? n0 + f_r : n0 + f_nt * 16 + f_r;
+  const int f_mt = is_gated(kEpilogue) ? f_tile : f_tile / NT, f_nt = is_gated(kEpilogue) ? 0 : f_tile % NT;
+  const int f_m = f_mt * 16 + f_g * 4 + f_i, f_n = is_gated(kEpilogue) ? n0 + f_r : n0 + f_nt * 16 + f_r;
   const bool f_ok = flat && f_tile < kOutTiles && f_m < M && f_n < N && f_n - n0 < cols;
   float f_add = 0.f;
   if (f_ok) {
@@ -148,8 +148,8 @@ __global__ void __launch_bounds__(kWaves * 64) gemm_skinny_kernel(
 #pragma unroll
   for (int it = 0; it < kMyTiles; ++it) {
     const int tile = wave + it * kWaves;
-    const int mt = (kEpilogue == kSkSwiglu) ? tile : tile / NT, nt = (kEpilogue == kSkSwiglu) ? 0 : tile % NT;
-    const int n = (kEpilogue == kSkSwiglu) ? n0 + r : n0 + nt * 16 + r;
+    const int mt = is_gated(kEpilogue) ? tile : tile / NT, nt = is_gated(kEpilogue) ? 0 : tile % NT;
+    const int n = is_gated(kEpilogue) ? n0 + r : n0 + nt * 16 + r;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int m = mt * 16 + g * 4 + i;
@@ -290,7 +290,7 @@ __global__ void __launch_bounds__(kWaves * 64) gemm_skinny_kernel(
     float sum = shares[at], up = 0.f;
 #pragma unroll
     for (int w = 1; w < kWaves; ++w) sum += shares[w * (MT * NT * 256) + at];
-    if (kEpilogue == kSkSwiglu) {
+    if (is_gated(kEpilogue)) {
       up = shares[at + 256];
 #pragma unroll
       for (int w = 1; w < kWaves; ++w) up += shares[w * (MT * NT * 256) + at + 256];
@@ -309,7 +309,7 @@ __global__ void __launch_bounds__(kWaves * 64) gemm_skinny_kernel(
     } else if (kEpilogue == kSkResidual) {
       store_f32(dst, f_add + sum);
     } else {
-      store_f32(dst, sum / (1.f + __expf(-sum)) * up);
+      store_f32(dst, gate_of<kEpilogue == kSkGeglu>(sum) * up);
     }
     return;
   }
@@ -348,8 +348,8 @@ __global__ void __launch_bounds__(kWaves * 64) gemm_skinny_kernel(
   for (int it = 0; it < kMyTiles; ++it) {
     const int tile = wave + it * kWaves;
     if (tile >= kOutTiles) break;
-    const int mt = (kEpilogue == kSkSwiglu) ? tile : tile / NT;
-    const int nt = (kEpilogue == kSkSwiglu) ? 0 : tile % NT;
+    const int mt = is_gated(kEpilogue) ? tile : tile / NT;
+    const int nt = is_gated(kEpilogue) ? 0 : tile % NT;
     f32x4 sum, up = f32x4{0.f, 0.f, 0.f, 0.f};
     if (k_splits > 1) {
       // (all the splits' loads on their way together, two, four or eight: they come from memory, and one after
@@ -372,13 +372,13 @@ __global__ void __launch_bounds__(kWaves * 64) gemm_skinny_kernel(
       sum = red[0][mt * NT + nt][lane];
 #pragma unroll
       for (int w = 1; w < kWaves; ++w) sum += red[w][mt * NT + nt][lane];
-      if (kEpilogue == kSkSwiglu) {
+      if (is_gated(kEpilogue)) {
         up = red[0][mt * NT + 1][lane];
 #pragma unroll
         for (int w = 1; w < kWaves; ++w) up += red[w][mt * NT + 1][lane];
       }
     }
-    const int n = (kEpilogue == kSkSwiglu) ? n0 + r : n0 + nt * 16 + r;
+    const int n = is_gated(kEpilogue) ? n0 + r : n0 + nt * 16 + r;
     if (n >= N || n - n0 >= cols) continue;
     if constexpr (kNorm) {
       // rows 4 g .. 4 g + 3 of the tile: their factors 1 / sqrt(mean of squares + eps)
@@ -405,7 +405,7 @@ __global__ void __launch_bounds__(kWaves * 64) gemm_skinny_kernel(
         store_f32(dst, add[it][i] + sum[i]);
       } else {
         const float gv = sum[i];
-        store_f32(dst, gv / (1.f + __expf(-gv)) * up[i]);
+        store_f32(dst, gate_of<kEpilogue == kSkGeglu>(gv) * up[i]);
       }
     }
   }
@@ -430,10 +430,10 @@ struct NormArgs {
 // the compute units, 11.0); 2,560 x 2,048 against 64 rows stays whole (13.5; eight parts 18.0).
 template <int MT, int NT, int kWaves, int kEpilogue>
 static int skinny_splits(int M, int N, int K) {
-  constexpr int cols = (kEpilogue == kSkSwiglu) ? 16 : 16 * NT;
+  constexpr int cols = is_gated(kEpilogue) ? 16 : 16 * NT;
   const int col_tiles = (N + cols - 1) / cols;
   const Workspace& g_ws = workspace();
-  if (kEpilogue == kSkSwiglu || g_ws.tiles == nullptr || col_tiles > kGemmCounters) return 1;
+  if (is_gated(kEpilogue) || g_ws.tiles == nullptr || col_tiles > kGemmCounters) return 1;
   const int steps = (K + 31) / 32, units = compute_units();
   const int64_t block_bytes = static_cast<int64_t>(M + cols) * K * 2;
   auto cost = [&](int parts) {
@@ -451,7 +451,7 @@ static int skinny_splits(int M, int N, int K) {
 template <int MT, int NT, int kWaves, int kEpilogue, typename TO>
 static int launch_skinny(void* out, int64_t ldo, const void* A, int64_t lda, const void* W, const void* W2, int64_t ldw,
                          const float* bias, int M, int N, int K, NormArgs norm, hipStream_t stream, int* splits_only) {
-  constexpr int cols = (kEpilogue == kSkSwiglu) ? 16 : 16 * NT;
+  constexpr int cols = is_gated(kEpilogue) ? 16 : 16 * NT;
   const int col_tiles = (N + cols - 1) / cols;
   const Workspace& g_ws = workspace();
   if (splits_only) {
@@ -475,7 +475,7 @@ static int launch_skinny(void* out, int64_t ldo, const void* A, int64_t lda, con
       // 0.930 against 0.938 ms).
       int own = cols;
       {
-        const int64_t row_bytes = static_cast<int64_t>(M) * K * 4, col_bytes = static_cast<int64_t>(kEpilogue == kSkSwiglu ? 2 : 1) * K * 2;
+        const int64_t row_bytes = static_cast<int64_t>(M) * K * 4, col_bytes = static_cast<int64_t>(is_gated(kEpilogue) ? 2 : 1) * K * 2;
         auto reads = [&](int c) {
           const int64_t blocks = (N + c - 1) / c, each = (blocks + compute_units() - 1) / compute_units();
           return each * (c * col_bytes + row_bytes);
@@ -507,9 +507,9 @@ static int dispatch_skinny(void* out, int64_t ldo, const void* A, int64_t lda, c
                            const float* bias, int M, int N, int K, NormArgs norm, hipStream_t stream, int* splits_only = nullptr) {
   // few columns: one 16-column tile per block and eight waves along K keep more of the chip busy;
   // many columns and many rows: four column tiles per block, so that the rows are read less often
-  const bool narrow = (kEpilogue != kSkSwiglu) && N <= 4096;
+  const bool narrow = (!is_gated(kEpilogue)) && N <= 4096;
 #define ALOFA_SKINNY(MT, WIDE)                                                                                        \
-  if (kEpilogue == kSkSwiglu)                                                                                         \
+  if (is_gated(kEpilogue))                                                                                         \
     return launch_skinny<MT, 2, (MT >= 4 ? 4 : 8), kEpilogue, TO>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, norm, stream, splits_only); \
   if (narrow) return launch_skinny<MT, 1, 8, kEpilogue, TO>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, norm, stream, splits_only);     \
   return launch_skinny<MT, WIDE, 4, kEpilogue, TO>(out, ldo, A, lda, W, W2, ldw, bias, M, N, K, norm, stream, splits_only);
@@ -559,6 +559,10 @@ extern "C" int alofa_gemm_skinny(void* out, int o_dtype, int64_t ldo, const void
   if (epilogue == kSkSwiglu && o_dtype == kBF16) {
     ALOFA_REQUIRE(W2 != nullptr, "gemm_skinny: the swiglu epilogue needs the up matrix");
     return dispatch_skinny<kSkSwiglu, bf16_t>(out, ldo, A, lda, W, W2, ldw, nullptr, M, N, K, norm, stream);
+  }
+  if (epilogue == kSkGeglu && o_dtype == kBF16) {
+    ALOFA_REQUIRE(W2 != nullptr, "gemm_skinny: the geglu epilogue needs the up matrix");
+    return dispatch_skinny<kSkGeglu, bf16_t>(out, ldo, A, lda, W, W2, ldw, nullptr, M, N, K, norm, stream);
   }
   ALOFA_REQUIRE(false, "gemm_skinny: unsupported epilogue %d with out dtype %d", epilogue, o_dtype);
 }

@@ -75,7 +75,8 @@ struct Pool {
 // ----------------------------------------------------------------------- cache
 
 struct Group {
-  int64_t window;  // -1: every key stays visible
+  int64_t window;      // -1: every key stays visible
+  int64_t keep_first;  // a window passes over this many of a sequence's first keys without letting go of them
   Pool pool;
 };
 
@@ -83,7 +84,7 @@ struct Request {
   bool live = false;
   int64_t length = 0;
   std::vector<std::vector<int>> tables;  // per group: logical block -> physical or -1
-  std::vector<int> first_held;
+  std::vector<int> first_held;           // per group: the first block that a window has not passed yet
 };
 
 struct Cache {
@@ -395,12 +396,13 @@ int alofa_pool_n_blocks(void* p) { return static_cast<Pool*>(p)->n_blocks; }
 
 // ---- cache
 // n_blocks: the pages of every group's own pool
-void* alofa_cache_new(int n_groups, const int64_t* windows, const int64_t* n_blocks, int block_size, int max_requests) {
+// keep_first: how many of a sequence's first keys stay although a group's window has passed them (0: none)
+void* alofa_cache_new(int n_groups, const int64_t* windows, const int64_t* keep_first, const int64_t* n_blocks, int block_size, int max_requests) {
   if (n_groups < 0 || block_size <= 0 || max_requests <= 0) return nullptr;
   for (int g = 0; g < n_groups; ++g)
-    if (n_blocks[g] <= 0 || n_blocks[g] > INT32_MAX) return nullptr;
+    if (n_blocks[g] <= 0 || n_blocks[g] > INT32_MAX || keep_first[g] < 0) return nullptr;
   Cache* c = new Cache{block_size, max_requests, {}, {}, {}};
-  for (int g = 0; g < n_groups; ++g) c->groups.push_back(Group{windows[g], Pool(static_cast<int>(n_blocks[g]))});
+  for (int g = 0; g < n_groups; ++g) c->groups.push_back(Group{windows[g], keep_first[g], Pool(static_cast<int>(n_blocks[g]))});
   c->reqs.resize(max_requests);
   for (int s = max_requests - 1; s >= 0; --s) c->free_slots.push_back(s);
   return c;
@@ -416,7 +418,8 @@ int alofa_cache_admit(void* cv) {  // takes the lowest free request slot
   r.live = true;
   r.length = 0;
   r.tables.assign(c->groups.size(), {});
-  r.first_held.assign(c->groups.size(), 0);
+  r.first_held.clear();
+  for (const Group& g : c->groups) r.first_held.push_back(static_cast<int>(blocks_for(g.keep_first, c->block_size)));      // (the pages before these are never let go of)
   return slot;
 }
 int alofa_cache_drop(void* cv, int slot) {  // the request ends: every page and its slot are given back

@@ -206,7 +206,7 @@ __global__ void __launch_bounds__(256) route_groups_kernel(const float* __restri
     for (int k = 0; k < top; ++k) {
       const int e = chosen[static_cast<int64_t>(t) * top + k];
       Acc w = static_cast<Acc>(weights[static_cast<int64_t>(t) * top + k]);
-      if (renorm) w /= total;
+      if (renorm) w /= total + static_cast<Acc>(1e-20f);      // (scores that are all next to nothing stay numbers)
       const float f = static_cast<float>(w * static_cast<Acc>(scale));
       weights[static_cast<int64_t>(t) * top + k] = f;
       if (e >= 0 && e < real) d[e] = f;

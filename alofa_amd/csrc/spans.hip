@@ -9,7 +9,8 @@
 //                     the pages hold them, in pages of their own (one place per P tokens of a page).
 //   span_attention    the always-valid kernel, a wavefront per (row, head): softmax over the tokens of the window and the
 //                     blocks wholly behind it, scores plus a bias by distance, exp(sink) in the denominator, a sigmoid gate
-//                     per channel or per head.
+//                     per channel or per head. The first tokens of a sequence may stay in sight behind the window, scores may be
+//                     capped, and neighbouring key heads may share a value head.
 //
 // Cache layout (that of the other attention kernels): keys [page, kv_head, slot, d], values transposed [page, kv_head, dv, slot].
 // Pooled: keys [page, kv_head, place, d], values [page, kv_head, dv, place], block b at page table[(b P) / S], place ((b P) % S) / P.
@@ -169,6 +170,10 @@ struct SpanArgs {
   int bias_len;
   const float* sink;           // [heads] (nullptr: none)
   int gate_kind;               // 0 none, 1 a gate per channel [T, heads * dv], 2 a gate per head [T, heads]
+  int keep_first;              // that many of a sequence's first tokens are seen although the window has passed them
+  float cap;                   // scores become cap tanh(score / cap) (0: as they are)
+  int maps;                    // so many neighbouring key heads share a value head, and as many neighbouring query heads are one head's maps of them
+  float* out32;                // results go here unrounded, and `out` is not written (nullptr: to out)
 };
 
 template <typename T, typename Acc>
@@ -180,12 +185,14 @@ __global__ void __launch_bounds__(256) span_attention_kernel(T* __restrict__ out
   const int64_t unit = static_cast<int64_t>(blockIdx.x) * 4 + wave;
   if (unit >= static_cast<int64_t>(a.tokens) * a.heads) return;
   const int t = static_cast<int>(unit / a.heads), h = static_cast<int>(unit % a.heads);
-  const int g = h / (a.heads / a.kv_heads);
+  const int g = h / (a.heads / a.kv_heads * a.maps) * a.maps + h % a.maps;      // (heads that share values lie map by map, and so do their key heads)
   const int d = a.d, dv = a.dv, S = a.block_size;
   const int p = a.positions[t];
   const int r = a.req_of_token ? a.req_of_token[t] : t;
   const int lo = (a.window > 0 && p - a.window + 1 > 0) ? p - a.window + 1 : 0;
-  const int n_tok = p - lo + 1;
+  const int n_keep = a.keep_first < lo ? a.keep_first : lo;      // kept tokens behind the window
+  const int n_tok = n_keep + p - lo + 1;
+  const int gv = g / a.maps, value_heads = a.kv_heads / a.maps;
   const int n_blk = (a.pool_table != nullptr && a.window > 0 && p - a.window + 1 >= a.P) ? (p - a.window + 1) / a.P : 0;
   const int n_all = n_tok + n_blk;
   const int32_t* tab = a.table + static_cast<int64_t>(r) * a.max_blocks;
@@ -194,12 +201,13 @@ __global__ void __launch_bounds__(256) span_attention_kernel(T* __restrict__ out
   for (int c = lane; c < d; c += kWave) myq[c] = load_f32(q + static_cast<int64_t>(t) * a.q_stride + static_cast<int64_t>(h) * d + c);
   wave_lds_sync();
 
-  // entry e of the row's list: the window's tokens in ascending order, then the blocks behind it in ascending order
+  // entry e of the row's list: the kept tokens behind the window, its own tokens, both in ascending order, then the pooled blocks in ascending order
+  auto token_of = [&](int e) { return e < n_keep ? e : lo + e - n_keep; };
   auto score = [&](int e) -> Acc {
     const T* k;
     Acc b = 0;
     if (e < n_tok) {
-      const int j = lo + e;
+      const int j = token_of(e);
       k = k_cache + ((static_cast<int64_t>(tab[j / S]) * a.kv_heads + g) * S + j % S) * static_cast<int64_t>(d);
       if (a.bias) {
         const int dist = p - j;
@@ -211,7 +219,9 @@ __global__ void __launch_bounds__(256) span_attention_kernel(T* __restrict__ out
     }
     Acc acc = 0;
     for (int c = 0; c < d; ++c) acc += static_cast<Acc>(myq[c]) * static_cast<Acc>(load_f32(k + c));
-    return acc * static_cast<Acc>(a.scale) + b;
+    acc *= static_cast<Acc>(a.scale);
+    if (a.cap > 0.f) acc = static_cast<Acc>(a.cap) * tanh(acc / static_cast<Acc>(a.cap));
+    return acc + b;
   };
 
   Acc m = -DBL_MAX, l = 0;
@@ -245,8 +255,8 @@ __global__ void __launch_bounds__(256) span_attention_kernel(T* __restrict__ out
       const T* v;
       int64_t step;
       if (ee < n_tok) {
-        const int j = lo + ee;
-        v = v_cache + (static_cast<int64_t>(tab[j / S]) * a.kv_heads + g) * static_cast<int64_t>(dv) * S + j % S;
+        const int j = token_of(ee);
+        v = v_cache + (static_cast<int64_t>(tab[j / S]) * value_heads + gv) * static_cast<int64_t>(dv) * S + j % S;
         step = S;
       } else {
         const int first = (ee - n_tok) * a.P;
@@ -272,7 +282,9 @@ __global__ void __launch_bounds__(256) span_attention_kernel(T* __restrict__ out
       const Acc z = static_cast<Acc>(load_f32(gate + static_cast<int64_t>(t) * a.gate_stride + at));
       y = y / (static_cast<Acc>(1) + exp(-z));
     }
-    store_f32(out + static_cast<int64_t>(t) * a.out_stride + static_cast<int64_t>(h) * dv + c, static_cast<float>(y));
+    const int64_t at = static_cast<int64_t>(t) * a.out_stride + static_cast<int64_t>(h) * dv + c;
+    if (a.out32) a.out32[at] = static_cast<float>(y);
+    else store_f32(out + at, static_cast<float>(y));
   }
 }
 
@@ -590,7 +602,10 @@ extern "C" int alofa_pool_blocks(const void* k_cache, const void* v_cache, void*
 extern "C" int alofa_span_attention(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* k_cache, const void* v_cache, const void* pk, const void* pv,
                                     int dtype, const int32_t* table, int max_blocks, const int32_t* pool_table, int pool_max_blocks, const int32_t* req_of_token,
                                     const int32_t* positions, int tokens, int heads, int kv_heads, int d, int dv, int block_size, int window, int P, int places, float scale,
-                                    const float* bias, int bias_len, const float* sink, const void* gate, int64_t gate_stride, int gate_kind, int exact, hipStream_t stream) {
+                                    const float* bias, int bias_len, const float* sink, const void* gate, int64_t gate_stride, int gate_kind, int keep_first, float cap, int maps,
+                                    float* out32, int exact, hipStream_t stream) {
+  ALOFA_REQUIRE(keep_first >= 0 && cap >= 0.f && maps >= 1 && kv_heads % maps == 0, "span_attention: keep_first=%d cap=%g maps=%d (of %d key heads)", keep_first, cap, maps, kv_heads);
+  ALOFA_REQUIRE(pool_table == nullptr || (keep_first == 0 && maps == 1), "span_attention: pooled blocks go with neither kept tokens nor shared value heads");
   ALOFA_REQUIRE(tokens >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0, "span_attention: tokens=%d heads=%d kv_heads=%d (kv_heads must divide heads)", tokens, heads, kv_heads);
   ALOFA_REQUIRE(d > 0 && d <= 256 && dv > 0 && dv <= 256, "span_attention: head sizes %d and %d (up to 256 channels)", d, dv);
   ALOFA_REQUIRE(block_size > 0 && max_blocks > 0 && window >= 0, "span_attention: block_size=%d max_blocks=%d window=%d", block_size, max_blocks, window);
@@ -600,7 +615,7 @@ extern "C" int alofa_span_attention(void* out, int64_t out_stride, const void* q
   ALOFA_REQUIRE(!exact || dtype == kF32, "span_attention: the exact path is float32");
   if (tokens == 0) return 0;
   SpanArgs a{out_stride, q_stride, gate_stride, table, max_blocks, pool_table, pool_max_blocks, req_of_token, positions, tokens, heads, kv_heads, d, dv, block_size, window,
-             P, places, scale, bias, bias_len, sink, gate_kind};
+             P, places, scale, bias, bias_len, sink, gate_kind, keep_first, cap, maps, out32};
   const unsigned grid = static_cast<unsigned>((static_cast<int64_t>(tokens) * heads + 3) / 4);
 #define ALOFA_SPAN(T, ACC) span_attention_kernel<T, ACC><<<grid, 256, 0, stream>>>(static_cast<T*>(out), static_cast<const T*>(q), static_cast<const T*>(k_cache), static_cast<const T*>(v_cache), \
     static_cast<const T*>(pk), static_cast<const T*>(pv), static_cast<const T*>(gate), a)

@@ -14,6 +14,7 @@ from .config.base import ModelSpec
 from .config.registry import load_config
 from .errors import AlofaError
 from .parts.base import Runtime, build_part, part_class, tensors_of
+from .parts.streams import StreamRead
 from .weights.loader import load_weights
 
 DTYPES = {"float32": torch.float32, "bfloat16": torch.bfloat16, "fp32": torch.float32, "bf16": torch.bfloat16}
@@ -56,6 +57,11 @@ class Model:
         self.head = build_part("head", spec.head, weights, rt, embedding=self.embedding)
         self.joins = [build_part("join", j, weights, rt) for j in spec.joins]
         self.order = list(spec.order)
+        self.streams = int(spec.streams)
+        if any(b.on_streams != bool(self.streams) for b in self.blocks) or (self.streams and self.joins):
+            raise AlofaError("unsupported", "blocks on copies of the stream go with a model that keeps copies, and with no joins", f"streams={self.streams}")
+        # what leaves the last layer of a model that keeps copies of the stream: their sum
+        self.sum_of_streams = StreamRead(torch.ones(self.streams, dtype=torch.float32, device=rt.device), last=True) if self.streams else None
 
     # What the cache manager has to provide. The blocks answer; an owner's key is (run entry, index
     # of the mixer within its block).
@@ -119,24 +125,33 @@ class Model:
             first = ctx.scratch("hidden_first", tuple(hidden.shape), torch.float32)
             first.copy_(hidden)
         watch = getattr(ctx, "watch", None)      # (for tests and debugging: called with the stream after every run entry)
+        stream = hidden
+        if self.streams:      # the copies: spread, and read for the first block, in one launch
+            stream = ctx.scratch("streams", (rows, self.streams, hidden.shape[1]), torch.float32)
+            read = self.blocks[self.order[0].layer].wants_normed(rows)
+            normed = ctx.scratch("normed", tuple(hidden.shape), self.rt.dtype)
+            ops.streams_step(stream, source=hidden, w_in=read.weights, norm=read.norm, out=normed, exact=self.rt.exact)
         for i, e in enumerate(self.order):
             block = self.blocks[e.layer]
             if e.join is not None:
                 self.joins[e.join].forward(ctx, hidden, first)
                 normed = None
             if not block.takes_normed or watch is not None:
-                block.forward(ctx, i, hidden)
+                block.forward(ctx, i, stream)
                 normed = None
+                if self.streams:
+                    ops.streams_step(stream, w_in=self.sum_of_streams.weights, out=hidden, write=False, exact=self.rt.exact)
                 if watch is not None:
                     watch(i, hidden)
                 continue
             # the norm the next block starts with may be left by this block's last product (a launch less)
             nxt = self.blocks[self.order[i + 1].layer] if i + 1 < len(self.order) and self.order[i + 1].join is None else None
             norm = nxt.wants_normed(rows) if nxt is not None and nxt.takes_normed else None
-            leaves = norm is not None and (norm.as_rmsnorm() is not None or (norm.as_layernorm() is not None and getattr(block, "leaves_layernorm", False))
-                                         or (norm.identity and getattr(block, "leaves_rows", False)))
+            leaves = norm is not None and block.can_leave(norm)
             then = (norm, ctx.scratch("normed", tuple(hidden.shape), self.rt.dtype)) if leaves else None
-            normed = then[1] if block.forward(ctx, i, hidden, normed, then) else None
+            if self.streams and nxt is None:
+                then = (self.sum_of_streams, hidden)
+            normed = then[1] if block.forward(ctx, i, stream, normed, then) else None
         return hidden
 
     def logits(self, ctx, hidden: torch.Tensor, rows: torch.Tensor) -> torch.Tensor:

@@ -2,6 +2,7 @@
 from ..config.registry import register_architecture
 from .lalepel import LalepelConfig
 from .ludelorn import LudelornConfig
+from .nodopel import NodopelConfig
 from .qwen2 import Qwen2Config
 from .rerupel import RerupelConfig
 from .retotar import RetotarConfig
@@ -13,5 +14,6 @@ register_architecture(RerupelConfig.architecture, RerupelConfig)
 register_architecture(RetotarConfig.architecture, RetotarConfig)
 register_architecture(LudelornConfig.architecture, LudelornConfig)
 register_architecture(LalepelConfig.architecture, LalepelConfig)
+register_architecture(NodopelConfig.architecture, NodopelConfig)
 
-__all__ = ["LalepelConfig", "LudelornConfig", "Qwen2Config", "RerupelConfig", "RetotarConfig", "TugalixConfig"]
+__all__ = ["LalepelConfig", "LudelornConfig", "NodopelConfig", "Qwen2Config", "RerupelConfig", "RetotarConfig", "TugalixConfig"]

@@ -145,7 +145,7 @@ def rmsnorm(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, eps: float, exa
 # ------------------------------------------------------------ matrix product
 
 SKINNY_MAX_ROWS = 64
-SWIGLU = 2
+GATED = {"silu": 2, "gelu_tanh": 4}      # epilogues of the products of gate and up together, by activation
 
 
 ROWS_MAX_M, ROWS_MAX_K = 8, 6144      # what the vector-unit kernel for very few rows takes (longer rows: plain products only)
@@ -415,8 +415,10 @@ def gemm(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, bias: Optional[tor
 
 
 def gemm_swiglu(out: torch.Tensor, a: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor, exact: bool = False,
-                kernel: Optional[str] = None, norm: Optional[tuple] = None) -> None:
-    """out = silu(a @ w_gate.T) * (a @ w_up.T). ``kernel`` and ``norm`` as for ``gemm``."""
+                kernel: Optional[str] = None, norm: Optional[tuple] = None, act: str = "silu") -> None:
+    """out = act(a @ w_gate.T) * (a @ w_up.T), act "silu" or "gelu_tanh". ``kernel`` and ``norm`` as for ``gemm``."""
+    if act not in GATED:
+        raise AlofaError("unsupported", "no such activation of a gate", f"act={act}")
     _gpu("out", out, None, 2), _gpu("a", a, None, 2), _gpu("w_gate", w_gate, None, 2), _gpu("w_up", w_up, None, 2)
     M, K = a.shape
     N = w_gate.shape[0]
@@ -428,17 +430,17 @@ def gemm_swiglu(out: torch.Tensor, a: torch.Tensor, w_gate: torch.Tensor, w_up: 
         if exact or not can_fuse_norm(M, w_gate, out.dtype, swiglu=True, kernel=kernel) or w_up.data_ptr() % 16:
             raise AlofaError("unsupported", "no kernel takes a norm with this product", f"a={tuple(a.shape)} gate={tuple(w_gate.shape)} out={out.dtype}")
         _call(_product_entry(kernel, M, 2 * N, K, True, normed=True), _ptr(out), _I(BF16), _L(_rows("out", out)), _ptr(a), _L(_rows("a", a)), _ptr(w_gate), _ptr(w_up),
-              _L(_rows("w_gate", w_gate)), _ptr(None), _I(M), _I(N), _I(K), _I(SWIGLU), *_norm_operands(a, norm, K), _stream())
+              _L(_rows("w_gate", w_gate)), _ptr(None), _I(M), _I(N), _I(K), _I(GATED[act]), *_norm_operands(a, norm, K), _stream())
         return
     if not exact and out.dtype is torch.bfloat16 and _mfma_operands(a, w_gate) and _mfma_operands(a, w_up):
         _ensure_workspace(a.device)
         entry = _product_entry(kernel, M, 2 * N, K, True)
         more = (_ptr(None), _F(0.0)) if entry != "alofa_gemm_mfma" else (_ptr(None), _F(0.0), _ptr(None), _L(0), _ptr(None))
         _call(entry, _ptr(out), _I(BF16), _L(_rows("out", out)), _ptr(a), _L(_rows("a", a)), _ptr(w_gate), _ptr(w_up),
-              _L(_rows("w_gate", w_gate)), _ptr(None), _I(M), _I(N), _I(K), _I(SWIGLU), *more, _stream())
+              _L(_rows("w_gate", w_gate)), _ptr(None), _I(M), _I(N), _I(K), _I(GATED[act]), *more, _stream())
         return
     _call("alofa_gemm_swiglu_simple", _ptr(out), _I(dtype_code(out)), _L(_rows("out", out)), _ptr(a), _I(dtype_code(a)), _L(_rows("a", a)),
-          _ptr(w_gate), _ptr(w_up), _I(dtype_code(w_gate)), _L(_rows("w_gate", w_gate)), _I(M), _I(N), _I(K), _I(int(exact)), _stream())
+          _ptr(w_gate), _ptr(w_up), _I(dtype_code(w_gate)), _L(_rows("w_gate", w_gate)), _I(M), _I(N), _I(K), _I(int(act == "gelu_tanh")), _I(int(exact)), _stream())
 
 
 def swiglu(out: torch.Tensor, gate: torch.Tensor, up: torch.Tensor, exact: bool = False) -> None:
@@ -767,7 +769,7 @@ def attention_decode(out, q, k_cache, v_cache, block_table, req_of_token, positi
           _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _I(block_table.shape[1]), _ptr(req_of_token), _ptr(positions), _ptr(rows),
           _I(served), _I(heads), _I(kv_heads), _I(d), _I(bs), _I(int(window or 0)), _F(scale), _I(n_splits),
           _ptr(cos), _ptr(sin), _ptr(slots), _I(int(hand_over)), _I(-1 if v_head is None else v_head), _ptr(out if as32 else None), _I(int(fine_weights)),
-          _I(planes), _L(out.stride(0) if planes else 0), _ptr(_sink_of(sink, heads)), _I(block_heads), _stream())
+          _I(planes), _L(out.stride(0) if planes else 0), _ptr(_sink_of(sink, heads)), _I(block_heads), _I(0), _I(0), _F(0.0), _F(0.0), _F(0.0), _F(0.0), _I(d), _stream())
 
 
 def can_fuse_rope_into_decode(d: int) -> bool:
@@ -1932,18 +1934,21 @@ def pool_blocks(k_cache: torch.Tensor, v_cache: torch.Tensor, pk: torch.Tensor, 
 def span_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor, req_of_token: Optional[torch.Tensor],
                    positions: torch.Tensor, heads: int, kv_heads: int, d: int, dv: int, window: Optional[int], scale: float, exact: bool = False,
                    pooled: Optional[tuple] = None, bias: Optional[torch.Tensor] = None, sink: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
-                   gate_kind: int = GATE_NONE) -> None:
+                   gate_kind: int = GATE_NONE, keep_first: int = 0, softcap: Optional[float] = None, maps: int = 1) -> None:
     """The always-valid attention over a window: out[t, h] = (sum_e w_e v_e) * sigmoid(gate), the softmax weights w over the tokens row t may see (its request's, up to its
     position; the last ``window``) and, with ``pooled`` = (keys, values, table, pool), over the blocks of ``pool`` tokens that lie wholly behind the window (their mean keys
     and values, as ``pool_blocks`` left them); scores are scale * q . k, plus ``bias`` [heads, n] float32 by distance (the last entry for every distance from n - 1 on);
     ``sink`` [heads] float32 adds exp(sink) to the head's denominator. ``gate``: [T, heads * dv] (GATE_CHANNEL) or [T, heads] (GATE_HEAD). Rows ``q`` [T, heads * d],
-    ``out`` [T, heads * dv] (row strides allowed)."""
-    _gpu("out", out, None, 2), _gpu("q", q, out.dtype, 2), _gpu("k_cache", k_cache, out.dtype, 4), _gpu("v_cache", v_cache, out.dtype, 4)
+    ``out`` [T, heads * dv] (row strides allowed; float32 beside bfloat16 operands: the results are left unrounded). ``keep_first``: the first so many tokens of the
+    sequence are seen too when the window has passed them. ``softcap``: scores become softcap tanh(score / softcap) (the bias comes after). ``maps``: so many
+    neighbouring key heads share a value head, and query head h reads key head h % maps of its group's (heads and key heads lie map by map); the value pages then hold kv_heads / maps heads of dv channels, in whatever cut the tensor names."""
+    _gpu("out", out, None, 2), _gpu("q", q, None if out.dtype is torch.float32 else out.dtype, 2), _gpu("k_cache", k_cache, q.dtype, 4), _gpu("v_cache", v_cache, q.dtype, 4)
     _contig("k_cache", k_cache), _contig("v_cache", v_cache), _gpu("block_table", block_table, torch.int32, 2), _contig("block_table", block_table)
     _gpu("positions", positions, torch.int32, 1), _contig("positions", positions)
     T, block = q.shape[0], k_cache.shape[2]
-    if (tuple(q.shape) != (T, heads * d) or tuple(out.shape) != (T, heads * dv) or tuple(k_cache.shape[1:]) != (kv_heads, block, d)
-            or tuple(v_cache.shape) != (k_cache.shape[0], kv_heads, dv, block) or positions.shape[0] != T):
+    if (tuple(q.shape) != (T, heads * d) or tuple(out.shape) != (T, heads * dv) or tuple(k_cache.shape[1:]) != (kv_heads, block, d) or positions.shape[0] != T
+            or v_cache.shape[0] != k_cache.shape[0] or v_cache.shape[3] != block or maps < 1 or kv_heads % maps or v_cache.shape[1] * v_cache.shape[2] != kv_heads // maps * dv
+            or (maps == 1 and v_cache.shape[1] != kv_heads)):
         raise AlofaError("shape_mismatch", "attention operands do not fit", f"out={tuple(out.shape)} q={tuple(q.shape)} k={tuple(k_cache.shape)} v={tuple(v_cache.shape)} heads={heads} kv_heads={kv_heads} d={d} dv={dv}")
     pk = pv = pool_table = None
     pool = places = 0
@@ -1964,15 +1969,18 @@ def span_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_
         _gpu("sink", sink, torch.float32, 1), _contig("sink", sink)
         if sink.shape[0] != heads:
             raise AlofaError("shape_mismatch", "one sink per head", f"sink={tuple(sink.shape)}")
+    if keep_first < 0 or (keep_first and pooled is not None) or (softcap is not None and not softcap > 0):
+        raise AlofaError("invalid_argument", "kept tokens do not go with pooled blocks; a cap of scores is positive", f"keep_first={keep_first} softcap={softcap}")
+    as32 = out.dtype is torch.float32 and q.dtype is not torch.float32
     if gate_kind != GATE_NONE:
-        _gpu("gate", gate, out.dtype, 2)
+        _gpu("gate", gate, q.dtype, 2)
         if tuple(gate.shape) != (T, heads * dv if gate_kind == GATE_CHANNEL else heads):
             raise AlofaError("shape_mismatch", "the gate does not fit its kind", f"gate={tuple(gate.shape)} kind={gate_kind}")
-    _call("alofa_span_attention", _ptr(out), _L(_rows("out", out)), _ptr(q), _L(_rows("q", q)), _ptr(k_cache), _ptr(v_cache), _ptr(pk), _ptr(pv), _I(dtype_code(out)),
+    _call("alofa_span_attention", _ptr(None if as32 else out), _L(_rows("out", out)), _ptr(q), _L(_rows("q", q)), _ptr(k_cache), _ptr(v_cache), _ptr(pk), _ptr(pv), _I(dtype_code(q)),
           _ptr(block_table), _I(block_table.shape[1]), _ptr(pool_table), _I(pool_table.shape[1] if pool_table is not None else 0), _ptr(req_of_token), _ptr(positions),
           _I(T), _I(heads), _I(kv_heads), _I(d), _I(dv), _I(block), _I(int(window or 0)), _I(int(pool)), _I(places), _F(scale), _ptr(bias),
           _I(bias.shape[1] if bias is not None else 0), _ptr(sink), _ptr(gate if gate_kind != GATE_NONE else None),
-          _L(_rows("gate", gate) if gate_kind != GATE_NONE else 0), _I(gate_kind), _I(int(exact)), _stream())
+          _L(_rows("gate", gate) if gate_kind != GATE_NONE else 0), _I(gate_kind), _I(int(keep_first)), _F(softcap or 0.0), _I(int(maps)), _ptr(out if as32 else None), _I(int(exact)), _stream())
 
 
 def head_gate(x: torch.Tensor, gate: torch.Tensor, heads: int, dv: int, per_head: bool, dv_stored: Optional[int] = None) -> None:
@@ -2173,3 +2181,154 @@ def ssd_step(xbc: torch.Tensor, raw: torch.Tensor, w: torch.Tensor, bias: Option
     _call("alofa_ssd_step", _ptr(xbc), _L(_rows("xbc", xbc)), _ptr(raw), _L(_rows("raw", raw)), _I(dtype_code(raw)), _ptr(w), _ptr(bias), _ptr(state if taps > 1 else None),
           _ptr(rows.slots), _I(taps), _ptr(qf), _ptr(kf), _ptr(vf), _ptr(decay), _ptr(dt_raw), _L(_rows("dt_raw", dt_raw)), _ptr(dt_bias), _ptr(a_log), _L(T), _I(heads),
           _I(groups), _I(n_state), _I(dv), _I(int(exact)), _stream())
+
+
+# ------------------------------------------------------------- several copies of the residual stream
+
+MAX_STREAMS = 16
+
+
+def streams_step(x: torch.Tensor, source: Optional[torch.Tensor] = None, y: Optional[torch.Tensor] = None, mix: Optional[torch.Tensor] = None,
+                 w_out: Optional[torch.Tensor] = None, w_in: Optional[torch.Tensor] = None, norm: Optional[tuple] = None, out: Optional[torch.Tensor] = None,
+                 write: bool = True, exact: bool = False) -> None:
+    """Copies of the stream, x [T, S, h] float32. With ``y`` [T, h] float32, ``mix`` [S, S] (from, to) and ``w_out`` [S]:
+    x[t, v] becomes sum_s mix[s, v] x[t, s] + w_out[v] y[t], all copies from the old ones. With ``out`` [T, h] and ``w_in`` [S]: out[t] = sum_v w_in[v] x[t, v] of
+    the new copies, through an RMSNorm where ``norm`` = (weight, eps) is given. ``source`` [T, h] float32: every copy is source[t] at the start.
+    ``write`` False: the new copies are not stored (nobody reads them again)."""
+    _gpu("x", x, torch.float32, 3), _contig("x", x)
+    T, S, h = x.shape
+    if not 1 <= S <= MAX_STREAMS:
+        raise AlofaError("unsupported", f"one to {MAX_STREAMS} copies of the stream", f"streams={S}")
+    for n, t in (("source", source), ("y", y)):
+        if t is not None:
+            _gpu(n, t, torch.float32, 2), _contig(n, t)
+            if tuple(t.shape) != (T, h):
+                raise AlofaError("shape_mismatch", "rows do not fit the copies of the stream", f"operand={n} shape={tuple(t.shape)} x={tuple(x.shape)}")
+    for n, t, shape, needed in (("mix", mix, (S, S), y is not None), ("w_out", w_out, (S,), y is not None), ("w_in", w_in, (S,), out is not None)):
+        if needed:
+            _gpu(n, t, torch.float32), _contig(n, t)
+            if tuple(t.shape) != shape:
+                raise AlofaError("shape_mismatch", "weights do not fit the copies of the stream", f"operand={n} shape={tuple(t.shape)} streams={S}")
+    weight, eps = norm if norm is not None else (None, 0.0)
+    if out is not None:
+        _gpu("out", out, None, 2), _contig("out", out)
+        if tuple(out.shape) != (T, h) or (exact and out.dtype is not torch.float32):
+            raise AlofaError("shape_mismatch", "what is read does not fit the copies of the stream", f"out={tuple(out.shape)} dtype={out.dtype} x={tuple(x.shape)}")
+        if weight is not None:
+            _gpu("norm weight", weight, torch.float32, 1), _contig("norm weight", weight)
+            if weight.shape[0] != h:
+                raise AlofaError("shape_mismatch", "norm width does not fit", f"weight={tuple(weight.shape)} h={h}")
+    _call("alofa_streams_step", _ptr(out), _I(dtype_code(out) if out is not None else F32), _ptr(x), _ptr(source), _ptr(y), _ptr(mix if y is not None else None),
+          _ptr(w_out if y is not None else None), _ptr(w_in if out is not None else None), _ptr(weight if out is not None else None), _F(eps), _I(T), _I(S), _I(h),
+          _I(int(write)), _I(int(exact)), _stream())
+
+
+# ------------------------------------------------------------- two maps per head over the same values
+
+MAPS_HEAD_DIMS = (16, 32, 48, 64, 96, 128, 192, 256)      # value head sizes (and both halves of a key head together) the matrix-core kernels are built for
+MAPS_MAX_KEPT_PAGES = 64                                   # first tokens of a sequence that stay in sight: what the decode kernel holds the pages of
+
+
+class HeadEnd:
+    """How a head of two maps ends: (a1 - lam a2) over its root mean square over ``true_d`` channels (plus eps), times ``gain``."""
+
+    def __init__(self, lam: float, gain: float, eps: float, true_d: int):
+        self.lam, self.gain, self.eps, self.true_d = float(lam), float(gain), float(eps), int(true_d)
+
+    def arguments(self) -> tuple:
+        return _F(self.lam), _F(self.gain), _F(self.eps)
+
+
+def maps_attention_fast(d: int, map_d: int, block_size: int, keep_first: int, dtype) -> bool:
+    """Whether the matrix-core kernels take these sizes."""
+    return (dtype is torch.bfloat16 and d in MAPS_HEAD_DIMS and 2 * map_d == d and block_size >= MIN_FAST_PAGE and block_size & (block_size - 1) == 0
+            and keep_first <= MAPS_MAX_KEPT_PAGES * block_size)
+
+
+def combine_maps(out: torch.Tensor, a: torch.Tensor, heads: int, d: int, end: HeadEnd, exact: bool = False,
+                 rows: Optional[torch.Tensor] = None) -> None:
+    """out[t, h] = the end (``HeadEnd``) of head h, whose maps' sums are a[t, 2 h] and a[t, 2 h + 1] (float32 rows of 2 heads * d values), for all rows t or
+    for ``rows`` (int32)."""
+    _gpu("out", out, None, 2), _gpu("a", a, torch.float32, 2)
+    T = out.shape[0]
+    if tuple(out.shape) != (T, heads * d) or tuple(a.shape) != (T, 2 * heads * d) or not 0 < end.true_d <= d <= MAX_HEAD_DIM:
+        raise AlofaError("shape_mismatch", "the maps' sums do not fit the heads", f"out={tuple(out.shape)} a={tuple(a.shape)} heads={heads} d={d} true_d={end.true_d}")
+    if rows is not None:
+        _gpu("rows", rows, torch.int32, 1), _contig("rows", rows)
+        T = rows.shape[0]
+    _call("alofa_combine_maps", _ptr(out), _L(_rows("out", out)), _I(dtype_code(out)), _ptr(a), _L(_rows("a", a)), _ptr(rows), _I(T), _I(heads), _I(d), _I(end.true_d), *end.arguments(),
+          _I(int(exact)), _stream())
+
+
+def _maps_operands(out, q, k_cache, v_cache, block_table, heads, kv_heads, d, window, keep_first, softcap, end):
+    _gpu("out", out, torch.bfloat16, 2), _gpu("q", q, torch.bfloat16, 2)
+    T = q.shape[0]
+    if kv_heads <= 0 or heads % kv_heads or tuple(out.shape) != (T, heads * d) or q.shape[1] < heads * d:
+        raise AlofaError("shape_mismatch", "attention rows do not fit", f"out={tuple(out.shape)} q={tuple(q.shape)} heads={heads} kv_heads={kv_heads} d={d}")
+    bs = check_caches(k_cache, v_cache, 2 * kv_heads, d // 2)
+    if k_cache.dtype is not torch.bfloat16 or not maps_attention_fast(d, d // 2, bs, keep_first, q.dtype) or keep_first < 0 or not 0 < end.true_d <= d:
+        raise AlofaError("unsupported", "no kernel for two maps takes these sizes", f"d={d} page={bs} keep_first={keep_first} true_d={end.true_d}")
+    if softcap is not None and not softcap > 0:
+        raise AlofaError("invalid_argument", "a cap of scores is positive", f"softcap={softcap}")
+    _gpu("block_table", block_table, torch.int32, 2), _contig("block_table", block_table)
+    if _rows("q", q) % 8 or q.data_ptr() % 16 or _rows("out", out) % 4 or out.data_ptr() % 8:
+        raise AlofaError("alignment", "attention rows must be 16-byte aligned", f"q_stride={_rows('q', q)} out_stride={_rows('out', out)}")
+    return T, bs
+
+
+def maps_prefill(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor, tiles: torch.Tensor, heads: int, kv_heads: int, d: int,
+                 window: Optional[int], keep_first: int, scale: float, softcap: Optional[float], end: HeadEnd) -> None:
+    """bfloat16 attention of two maps per head for portions of prompts, from turned queries to the heads' ends in one launch. ``q`` [T, >= heads * d]: head by head
+    map 1 and map 2, d / 2 channels each; ``k_cache`` [pages, 2 kv_heads, page, d / 2] likewise; ``v_cache`` [pages, 2 kv_heads, d / 2, page], which holds [kv_heads, d] channels;
+    ``tiles`` int32 [n, 4]: (request index, first row, rows <= 64, position of the first row). ``window`` and ``keep_first``: row i sees j <= i with i - j < window or
+    j < keep_first. Every softmax weight counts with sixteen bits."""
+    T, bs = _maps_operands(out, q, k_cache, v_cache, block_table, heads, kv_heads, d, window, keep_first, softcap, end)
+    _gpu("tiles", tiles, torch.int32, 2), _contig("tiles", tiles)
+    if tiles.shape[1] != 4 or tiles.shape[0] == 0:
+        raise AlofaError("shape_mismatch", "tiles must be [n, 4]", f"tiles={tuple(tiles.shape)}")
+    _call("alofa_maps_prefill", _ptr(out), _L(_rows("out", out)), _ptr(q), _L(_rows("q", q)), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _I(block_table.shape[1]),
+          _ptr(tiles), _I(tiles.shape[0]), _I(heads), _I(kv_heads), _I(d), _I(end.true_d), _I(bs), _I(int(window or 0)), _I(int(keep_first)), _F(scale), _F(softcap or 0.0),
+          *end.arguments(), _stream())
+
+
+def maps_decode_plan(tokens: int, heads: int, kv_heads: int, d: int, max_context: int, window: Optional[int], keep_first: int) -> tuple:
+    """(parts, whether the last block combines them, floats of scratch) of ``maps_decode`` for these sizes."""
+    n = decode_splits(tokens, 2 * heads, kv_heads, d, min(max_context, window + keep_first if window else max_context))
+    hand_over = decode_hand_over(tokens, 2 * heads, kv_heads, d, n)
+    # (parts that a second kernel combines: their states, and both maps' sums)
+    return n, hand_over, tokens * 2 * heads * n * (d + 2) if n > 1 and not hand_over else 0
+
+
+def maps_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor, req_of_token: Optional[torch.Tensor],
+                positions: torch.Tensor, heads: int, kv_heads: int, d: int, window: Optional[int], keep_first: int, scale: float, softcap: Optional[float], end: HeadEnd,
+                max_context: int, scratch: Optional[torch.Tensor] = None, sums: Optional[torch.Tensor] = None, rows: Optional[torch.Tensor] = None, plan: Optional[tuple] = None) -> None:
+    """The same for tokens of requests that bring few tokens: all of the batch, or the tokens ``rows``; all heads of a key head with both their maps
+    share the keys and values a block reads. ``req_of_token`` None: token i is the one token of request i. ``scratch`` and ``sums`` (float32 [T, 2 heads * d]): needed
+    where ``maps_decode_plan`` asks for floats of scratch (a second kernel then combines the parts and ``combine_maps`` ends the heads). ``plan``: that
+    function's answer, if another is wanted."""
+    T, bs = _maps_operands(out, q, k_cache, v_cache, block_table, heads, kv_heads, d, window, keep_first, softcap, end)
+    _gpu("positions", positions, torch.int32, 1), _contig("positions", positions)
+    if req_of_token is not None:
+        _gpu("req_of_token", req_of_token, torch.int32, 1), _contig("req_of_token", req_of_token)
+    if positions.shape[0] != T or (req_of_token is not None and req_of_token.shape[0] != T):
+        raise AlofaError("shape_mismatch", "one request index and one position per token")
+    if req_of_token is None and (rows is not None or block_table.shape[0] < T):
+        raise AlofaError("invalid_argument", "without request indices every request brings one token, in table order", f"tokens={T} table_rows={block_table.shape[0]}")
+    n_tok = T
+    if rows is not None:
+        _gpu("rows", rows, torch.int32, 1), _contig("rows", rows)
+        n_tok = rows.shape[0]
+    n_splits, hand_over, floats = plan or maps_decode_plan(n_tok, heads, kv_heads, d, max_context, window, keep_first)
+    if floats:
+        _gpu("scratch", scratch, torch.float32), _contig("scratch", scratch), _gpu("sums", sums, torch.float32, 2), _contig("sums", sums)
+        if scratch.numel() < floats or tuple(sums.shape) != (T, 2 * heads * d):
+            raise AlofaError("invalid_argument", "parts need room for their states and for both maps' sums", f"floats={floats} scratch={scratch.numel()} sums={tuple(sums.shape)}")
+    # (where a second kernel combines parts its rows are the sums', and the heads' end is a third)
+    stride = 2 * heads * d if floats else _rows("out", out)
+    _call("alofa_attention_decode_v", _ptr(None if floats else out), _L(stride), _ptr(scratch if floats else None), _ptr(q), _L(_rows("q", q)),
+          _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _I(block_table.shape[1]), _ptr(req_of_token), _ptr(positions), _ptr(rows),
+          _I(n_tok), _I(2 * heads), _I(kv_heads), _I(d), _I(bs), _I(int(window or 0)), _F(scale), _I(n_splits), _ptr(None), _ptr(None), _ptr(None), _I(int(hand_over)), _I(-1),
+          _ptr(sums if floats else None), _I(1), _I(0), _L(0), _ptr(None), _I(decode_block_heads(n_tok, 2 * heads, kv_heads, d)),
+          _I(1), _I(int(keep_first)), _F(softcap or 0.0), *end.arguments(), _I(end.true_d), _stream())
+    if floats:
+        combine_maps(out, sums, heads, d, end, rows=rows)

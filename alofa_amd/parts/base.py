@@ -14,7 +14,7 @@ dtype, ``residual`` the float32 residual stream):
   feed_forward  forward(ctx, x, residual)                         residual += ff(x); capturable
   block         built from a LayerSpec; layer_tensors(layer); mixers() (the parts that may keep
                 a cache or state, in a fixed order); cache_needs(), state_needs(), capturable,
-                prepare(n_positions); forward(ctx, entry, hidden)  one layer on the stream
+                prepare(n_positions); forward(ctx, entry, hidden)  one layer on the stream (or on its copies [T,S,h]: on_streams)
   embedding     forward(ctx, ids) -> hidden[T,h] f32; state_need() -> StateNeed | None (kept under the key ("embedding", 0))
   join          forward(ctx, hidden[T,h] f32, first[T,h] f32)     the stream, replaced by a function of itself and the embedding's output
   head          forward(ctx, y[S,h]) -> logits[S,V] f32
@@ -100,9 +100,17 @@ class CacheTensor:
 class CacheNeed:
     """What a mixer keeps per token in pages: any number of named tensors. ``window`` None: every
     earlier token stays visible; else only the last ``window`` ones, and pages the window has
-    passed go back to the pool. Mixers with the same window share block tables (a group)."""
+    passed go back to the pool. ``keep_first``: that many of a sequence's first tokens stay visible although the
+    window has passed them, and their pages are held for good. Mixers with the same window and the same kept
+    tokens share block tables (a group)."""
     tensors: tuple
     window: Optional[int] = None
+    keep_first: int = 0
+
+    @property
+    def group(self):
+        """What names the group: None (every key), a window, or (window, kept first tokens)."""
+        return self.window if self.window is None or not self.keep_first else (self.window, self.keep_first)
 
     @staticmethod
     def keys_and_values(kv_heads: int, head_dim: int, window: Optional[int] = None) -> "CacheNeed":
@@ -261,9 +269,15 @@ class Block(Part):
     # many rows (or None), ``forward`` takes the rows so normed as ``normed`` and, with ``then=(norm, rows)``,
     # leaves the next block's. Blocks that know nothing of this take (ctx, entry, hidden) alone.
     takes_normed = False
+    # True: the block works on several copies of the stream, [T, S, h] (``ModelSpec.streams``), instead of one [T, h]
+    on_streams = False
 
     def wants_normed(self, rows: int):
         return None
+
+    def can_leave(self, norm) -> bool:
+        """Whether this block's last launch can leave what the next block asks for (its ``wants_normed``)."""
+        return norm.as_rmsnorm() is not None
 
     def forward(self, ctx, entry: int, hidden: torch.Tensor) -> None:
         raise NotImplementedError

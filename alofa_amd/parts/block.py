@@ -279,7 +279,9 @@ class SandwichBlock(Block):
             ops.add_scaled(hidden, apart, 1.0, exact=self.rt.exact)
 
     takes_normed = True
-    leaves_layernorm = True      # the launch that adds this block's last result can leave the next block's layer norm
+
+    def can_leave(self, norm):
+        return norm.as_rmsnorm() is not None or norm.as_layernorm() is not None      # (the launch that adds the last result can leave the next block's layer norm)
 
     def wants_normed(self, rows):
         return self.norms[0]
@@ -345,7 +347,9 @@ class PostNormBlock(Block):
         return self.mixer.stateful_parts()
 
     takes_normed = True
-    leaves_rows = True      # the launch that adds this block's last result can leave the stream's rows in the activation dtype
+
+    def can_leave(self, norm):
+        return norm.as_rmsnorm() is not None or norm.identity      # (the launch that adds the last result can leave the stream's rows in the activation dtype)
 
     def wants_normed(self, rows):
         return None if self.rt.dtype is torch.float32 else self.front      # (float32: the sub-layers read the stream where it lies)

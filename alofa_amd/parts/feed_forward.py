@@ -1,6 +1,6 @@
 """Dense feed-forwards.
 
-SwiGLU: down(silu(gate(x)) * up(x)), no biases; silu is
+SwiGLU: down(silu(gate(x)) * up(x)), no biases (or the tanh form of gelu in silu's place); silu is
 x / (1 + exp(-x)) (src/alofa/kernels/cpu/scalar.mojo:219-231,
 src/alofa/engine/executor.mojo:806-837). Gate and up run as one kernel that
 applies the activation before anything is written.
@@ -22,7 +22,7 @@ from .base import FeedForward, register_part
 
 
 class SwiGLU(FeedForward):
-    """params: prefix, hidden, intermediate; optional: names (tensor names after the prefix for gate, up, down, default the *_proj ones), init (the rule
+    """params: prefix, hidden, intermediate; optional: activation ("silu", the default, or "gelu_tanh"), names (tensor names after the prefix for gate, up, down, default the *_proj ones), init (the rule
     random weights are drawn by). ``forward(..., out=)``: the result is stored there (float32, the stream's shape) and the stream left alone."""
     NAMES = {"gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
     capturable = True   # native kernels on the current stream only: a decode step may be graph-captured
@@ -38,6 +38,9 @@ class SwiGLU(FeedForward):
         super().__init__(spec, weights, rt)
         p = spec.params
         self.hidden, self.intermediate = int(p["hidden"]), int(p["intermediate"])
+        self.activation = p.get("activation", "silu")
+        if self.activation not in ops.GATED:
+            raise AlofaError("unsupported", "no such activation of a gate is built", f"activation={self.activation}")
         pre, n = p["prefix"], {**self.NAMES, **p.get("names", {})}
         gate, up = weights[pre + n["gate"]], weights[pre + n["up"]]
         if gate.dtype is not up.dtype:
@@ -54,9 +57,9 @@ class SwiGLU(FeedForward):
     def forward(self, ctx, x, residual, norm=None, then=None, out=None):
         act = ctx.scratch("ff_act", (residual.shape[0], self.intermediate), self.rt.dtype)
         if norm is not None:      # the norm before the feed-forward rides on the gate/up product
-            ops.gemm_swiglu(act, residual, self.w_gate, self.w_up, norm=norm.as_rmsnorm())
+            ops.gemm_swiglu(act, residual, self.w_gate, self.w_up, norm=norm.as_rmsnorm(), act=self.activation)
         else:
-            ops.gemm_swiglu(act, x, self.w_gate, self.w_up, exact=self.rt.exact)
+            ops.gemm_swiglu(act, x, self.w_gate, self.w_up, exact=self.rt.exact, act=self.activation)
         if out is not None:
             ops.gemm(out, act, self.w_down, exact=self.rt.exact)
             return

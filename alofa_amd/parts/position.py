@@ -24,7 +24,9 @@ class Rotary(PositionEncoding):
     stretched linearly; default 1), stretch ({factor, original, fast, slow}: frequencies stretched by wavelength: with
     dim(t) = dims ln(original / (2 pi t)) / (2 ln theta), lo = max(floor(dim(fast)), 0), hi = min(ceil(dim(slow)), dims - 1) and
     ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1), pair i turns at f_i / factor * ramp_i + f_i (1 - ramp_i), and cos and sin
-    are multiplied by 0.1 ln(factor) + 1), frequencies ("reciprocal": 1 / float32(theta^(2i/dims)) in float32, the default;
+    are multiplied by 0.1 ln(factor) + 1), blend ({factor, original, low, high}: frequencies slowed down by how often they turn within
+    ``original`` tokens, n = original f / (2 pi): f where n > high, f / factor where n < low, and in between, with s = (n - low) / (high - low),
+    (1 - s) f / factor + s f; cos and sin keep their size), frequencies ("reciprocal": 1 / float32(theta^(2i/dims)) in float32, the default;
     "direct": theta^(-2i/dims) formed in float64 and rounded once).
 
     The kernels pair channel j with j + head_dim/2. With dims < head_dim the table holds the angle zero for the pairs
@@ -52,6 +54,12 @@ class Rotary(PositionEncoding):
             if not (st["factor"] > 0 and st["original"] > 0 and st["fast"] > 0 and st["slow"] > 0 and self.theta > 1):
                 raise AlofaError("invalid_argument", "a stretch by wavelength takes positive numbers and a base above one", f"stretch={self.stretch} theta={self.theta}")
             self.stretch = st
+        self.blend = spec.params.get("blend")
+        if self.blend is not None:
+            b = {k: float(self.blend[k]) for k in ("factor", "original", "low", "high")}
+            if not (b["factor"] > 0 and b["original"] > 0 and 0 < b["low"] <= b["high"]) or self.stretch is not None or not self.direct:
+                raise AlofaError("invalid_argument", "a blend by turns takes positive numbers, low at most high, direct frequencies and no stretch", f"blend={self.blend}")
+            self.blend = b
         if self.head_dim <= 0 or self.head_dim % 2:
             raise AlofaError("unsupported", "head dimension must be positive and even", f"head_dim={self.head_dim}")
 
@@ -75,7 +83,7 @@ class Rotary(PositionEncoding):
         return cos.astype(np.float32), sin.astype(np.float32)
 
     def _frequency(self, i: int) -> float:
-        """Pair i's frequency in float64, with the linear factor and the stretch by wavelength."""
+        """Pair i's frequency in float64, with the linear factor and the stretch or the blend by wavelength."""
         f = math.pow(self.theta, -2.0 * i / self.dims) / self.factor
         st = self.stretch
         if st is not None:
@@ -85,6 +93,14 @@ class Rotary(PositionEncoding):
             hi = min(math.ceil(dim_of(st["slow"])), self.dims - 1)
             ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
             f = f / st["factor"] * ramp + f * (1.0 - ramp)
+        b = self.blend
+        if b is not None:
+            turns = b["original"] * f / (2.0 * math.pi)
+            if turns < b["low"]:
+                f = f / b["factor"]
+            elif turns <= b["high"] and b["high"] > b["low"]:
+                s = (turns - b["low"]) / (b["high"] - b["low"])
+                f = (1.0 - s) * f / b["factor"] + s * f
         return f
 
     def channel_order(self):
@@ -106,7 +122,7 @@ class Rotary(PositionEncoding):
         """One table per (theta, head size) serves every layer of the model (kept on the runtime).
         A table that has to grow is replaced; the old one is kept alive, since a captured graph
         may still read it (for positions it covers)."""
-        key = ("rotary", self.theta, self.head_dim, self.dims, self.factor, self.direct, tuple(sorted(self.stretch.items())) if self.stretch else None)
+        key = ("rotary", self.theta, self.head_dim, self.dims, self.factor, self.direct, tuple(sorted(self.stretch.items())) if self.stretch else None, tuple(sorted(self.blend.items())) if self.blend else None)
         have = self.rt.shared.get(key)
         if have is None or have[0].shape[0] < n_positions:
             n = max(n_positions, 2 * have[0].shape[0] if have else 0)
