@@ -141,7 +141,7 @@ class NodopelConfig(ModelConfig):
         r, shared = mlp["router"], mlp["shared"]
         return PartSpec("routed_experts", {
             "prefix": pre, "hidden": self.width, "experts": r["experts"], "top": r["top"], "score": "softmax", "correction": "correction", "passing": r["identity"], "renormalize": True,
-            "expert": {"intermediate": mlp["expert"]["ff"]}, "shared": None if shared is None else {"intermediate": shared["ff"]}, "activation": "silu_glu", "router_init": "decisive",
+            "expert": {"intermediate": mlp["expert"]["ff"]}, "shared": None if shared is None else {"intermediate": shared["ff"]}, "activation": "silu_glu",
             "names": {"router": "router", "expert": "e{}", "shared": "shared", "gate": "gate", "up": "up", "down": "down"}})
 
     def _order(self) -> tuple:

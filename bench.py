@@ -28,8 +28,8 @@ context of 4,096) through the same engine and print their own line;
 ``--config 1.5b``, ``3b`` and ``14b`` run the continuous batch at those sizes.
 ``--sweep batch`` and ``--sweep context`` take any of the configurations.
 
-``--design tugalix``, ``--design rerupel``, ``--design retotar``, ``--design ludelorn`` and ``--design lalepel`` measure another design beside Qwen2 (Retotar and Ludelorn: beside
-Tugalix; Lalepel: beside Rerupel) at equal sizes: prefill of one prompt and
+``--design tugalix``, ``--design rerupel``, ``--design retotar``, ``--design ludelorn``, ``--design lalepel`` and ``--design nodopel`` measure another design beside Qwen2 (Retotar and Ludelorn: beside
+Tugalix; Lalepel: beside Rerupel; Nodopel: beside both Rerupel and Qwen2) at equal sizes: prefill of one prompt and
 decode steps at batch 1, 8 and 64, at a few widths (``--sizes``), a line per point and model."""
 import argparse
 import json
@@ -584,8 +584,24 @@ def lalepel_sizes(width, heads, dim, ff, layers, vocab=32000):
     return lal, rerupel_sizes(width, heads, dim, ff, layers, vocab)[0]
 
 
-DESIGN_MODELS = {"tugalix": tugalix_sizes, "rerupel": rerupel_sizes, "retotar": retotar_sizes, "ludelorn": ludelorn_sizes, "lalepel": lalepel_sizes}
-DESIGN_BESIDE = {"retotar": "tugalix", "ludelorn": "tugalix", "lalepel": "rerupel"}      # the model a design is measured beside, where that is not Qwen2
+def nodopel_sizes(width, heads, dim, ff, layers, vocab=32000):
+    """A Nodopel model of ``layers`` layers on four copies of the stream (heads of two maps of half a head's size over values of a head's size, a window of 1,024
+    keys that keeps the first 64, capped scores; the first layer with a dense feed-forward, the others with sixteen experts and four identity experts of which a token takes four,
+    and one that every token takes; all layers but the first in a loop that is passed once), beside it the closest other designs: Rerupel (the same experts, one latent
+    key head) at equal width, heads, layers and feed-forward, and Qwen2 within the same window (grouped-query attention with biases at equal head counts and sizes) with as many
+    feed-forward channels as a token's five experts."""
+    expert = max(64, ff // 8 // 64 * 64)
+    mixer = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": dim // 2, "vdim": dim, "scale": (dim // 2) ** -0.5, "softcap": 50.0, "diff": 0.3, "mask": {"size": 1024, "keep_first": 64},
+             "rot": {"dims": dim // 2, "base": 500000.0, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    moe = {"kind": "moe", "router": {"experts": 16, "top": 4, "identity": 4}, "expert": {"ff": expert}, "shared": {"ff": expert}}
+    nod = {"architecture": "Nodopel", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "streams": 4, "loop": {"start": 1, "stop": layers, "times": 1},
+           "layers": [{"type": "attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": ff} if i == 0 else moe} for i in range(layers)]}
+    rer, qwen = rerupel_sizes(width, heads, dim, ff, layers, vocab)
+    return nod, rer, dict(qwen, use_sliding_window=True, sliding_window=1024, max_window_layers=0)
+
+
+DESIGN_MODELS = {"tugalix": tugalix_sizes, "rerupel": rerupel_sizes, "retotar": retotar_sizes, "ludelorn": ludelorn_sizes, "lalepel": lalepel_sizes, "nodopel": nodopel_sizes}
+DESIGN_BESIDE = {"retotar": ("tugalix",), "ludelorn": ("tugalix",), "lalepel": ("rerupel",), "nodopel": ("rerupel", "qwen2")}      # the models a design is measured beside, where that is not Qwen2 alone
 DESIGN_SIZES = {"256": (256, 4, 64, 1024, 4), "1k": (1024, 16, 64, 4096, 8), "2k": (2048, 16, 128, 8192, 8), "4k": (4096, 32, 128, 14336, 4)}
 DESIGN_DEFAULT = ("1k", "2k", "4k")      # ("256": a small one, for a quick look)
 
@@ -598,7 +614,7 @@ def designs(args):
         if size not in DESIGN_SIZES:
             print(f"no such size: {size} (known: {','.join(DESIGN_SIZES)})")
             return 2
-        for name, cfg in zip((args.design, DESIGN_BESIDE.get(args.design, "qwen2")), DESIGN_MODELS[args.design](*DESIGN_SIZES[size])):
+        for name, cfg in zip((args.design, *DESIGN_BESIDE.get(args.design, ("qwen2",))), DESIGN_MODELS[args.design](*DESIGN_SIZES[size])):
             if args.only and name != args.only:
                 continue
             cfg = dict(cfg, vocab_size=cfg.get("vocab_size", cfg.get("vocab")))      # (the points draw their tokens by this key)

@@ -154,3 +154,10 @@ def lalepel_dirs(tmp_path_factory):
         write_random_model(cfg, d, seed={"A": 5, "B": 4, "C": 6067, "D": 6, "E": 5}[name])
         out[name] = d
     return out
+
+
+@pytest.fixture(scope="session")
+def nodopel_dirs(tmp_path_factory):
+    """Model folders of the small Nodopel configurations."""
+    from nodopel_cases import NODOPEL, SEEDS, write_model
+    return {name: write_model(cfg, tmp_path_factory.mktemp(f"nodopel_{name}"), SEEDS[name]) for name, cfg in NODOPEL.items()}

@@ -233,8 +233,8 @@ def greedy(W, cfg, prompt, n_new) -> list:
 
 def router_margins(W, cfg, ids) -> np.ndarray:
     """Per position the smallest gap, over all passes of layers with a router, between the last choice score that is taken and the
-    first that is not, in units of the scores' spread at that position (infinite where nothing is left out). Positions with a small
-    gap are the ones where rounding may change which experts a token takes."""
+    first that is not, in units of the two experts' softmax scores (what moves a score by rounding is proportional to it; infinite where nothing
+    is left out). Positions with a small gap are the ones where rounding may change which experts a token takes."""
     out = np.full(len(ids), np.inf)
     X, eps = np.repeat(W["embed"][np.asarray(ids)][:, None, :], cfg["streams"], axis=1), cfg["norm"]["eps"]
     for i in order(cfg):
@@ -245,8 +245,13 @@ def router_margins(W, cfg, ids) -> np.ndarray:
             mid = write_streams(X, differential_attention(u, W, p + "mix.", l["mixer"], eps), W[p + "hc1.mix"], W[p + "hc1.out"])
             z = rms_norm(read_streams(mid, W[p + "hc2.in"]), W[p + "norm2"], eps) @ W[p + "mlp.router"].T
             s = np.exp(z - z.max(axis=-1, keepdims=True))
-            c = np.sort(s / s.sum(axis=-1, keepdims=True) + W[p + "mlp.correction"], axis=-1)[:, ::-1]
+            s = s / s.sum(axis=-1, keepdims=True)
+            by = np.argsort(-(s + W[p + "mlp.correction"]), axis=-1, kind="stable")
+            c = np.take_along_axis(s + W[p + "mlp.correction"], by, axis=-1)
+            s = np.take_along_axis(s, by, axis=-1)
             top = mlp["router"]["top"]
-            out = np.minimum(out, (c[:, top - 1] - c[:, top]) / (c.std(axis=-1) + 1e-30))
+            # (any expert that is left out may be the one that comes in)
+            gap = (c[:, top - 1:top] - c[:, top:]) / (s[:, top - 1:top] + s[:, top:] + 1e-30)
+            out = np.minimum(out, gap.min(axis=-1))
         X = layer(X, W, cfg, i)
     return out
