@@ -107,8 +107,8 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
     const int32_t* __restrict__ positions, const int32_t* __restrict__ rows, int heads, int kv_heads,
     int bs_shift, int window, float scale, RopeArgs rope, int* __restrict__ counters, int v_head, float* __restrict__ out32, int value_heads, int64_t plane,
     const float* __restrict__ sink, int block_heads, MapsForm maps) {
-  static_assert(!kMaps || (kSplit && !kRope), "two maps: with split weights, queries turned beforehand");
-  static_assert(!kRope || DT % 4 == 0, "the rotation needs a channel and its partner in the same lane: d a multiple of 64");
+  static_assert(!kMaps || kSplit, "two maps: with split weights");
+  static_assert(!kRope || DT % (kMaps ? 8 : 4) == 0, "the rotation needs a channel and its partner in the same lane: d (of one map: d / 2) a multiple of 64");
   constexpr int d = DT * 16;
   constexpr int DS = (d + 31) / 32;            // steps of 32 along d in the first product
   // per wave and head: maximum, sum of weights, (two unused,) weighted value sums of the wave's share
@@ -167,21 +167,22 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
   // the new token's key (this lane's channel slices, rotated) and value (channels 16 nt + c16), kRope only
   uint4 new_k[DS];
   uint32_t new_v[DT];
-  float4 cs[kRope ? DS / 2 : 1][2], sn[kRope ? DS / 2 : 1][2];
+  constexpr int kPairs = !kRope ? 1 : kMaps ? DS / 4 : DS / 2;      // slices of pairs' first channels; a pair's second lies kPairs slices on (kMaps: in either map's half)
+  float4 cs[kPairs][2], sn[kPairs][2];
   int64_t new_slot = 0;
   if constexpr (kRope) {
     new_slot = rope.slots[t];
     const bf16_t* row = q + static_cast<int64_t>(t) * q_stride;
-    const bf16_t* k_row = row + static_cast<int64_t>(heads + hk) * d;
-    const bf16_t* v_row = row + static_cast<int64_t>(heads + kv_heads + hk) * d;
+    const bf16_t* k_row = row + static_cast<int64_t>((kMaps ? heads / 2 : heads) + hk) * d;
+    const bf16_t* v_row = row + static_cast<int64_t>((kMaps ? heads / 2 : heads) + kv_heads + hk) * d;
 #pragma unroll
     for (int ds = 0; ds < DS; ++ds) new_k[ds] = *reinterpret_cast<const uint4*>(k_row + ds * 32 + g * 8);
 #pragma unroll
     for (int nt = 0; nt < DT; ++nt) new_v[nt] = v_row[nt * 16 + c16];
     // (cos and sin of the pairs (c, c + d / 2): slices ds and ds + DS / 2 of this lane)
 #pragma unroll
-    for (int ds = 0; ds < DS / 2; ++ds) {
-      const int64_t at = static_cast<int64_t>(p) * (d / 2) + ds * 32 + g * 8;
+    for (int ds = 0; ds < kPairs; ++ds) {
+      const int64_t at = static_cast<int64_t>(p) * (32 * kPairs) + ds * 32 + g * 8;
       cs[ds][0] = *reinterpret_cast<const float4*>(rope.cos_t + at), cs[ds][1] = *reinterpret_cast<const float4*>(rope.cos_t + at + 4);
       sn[ds][0] = *reinterpret_cast<const float4*>(rope.sin_t + at), sn[ds][1] = *reinterpret_cast<const float4*>(rope.sin_t + at + 4);
     }
@@ -376,24 +377,28 @@ __global__ void __launch_bounds__(64 * NW) attention_decode_kernel(
   // The rotation comes after the first keys and values have set out: it needs cos and sin only, which were
   // asked for before them.
   if constexpr (kRope) {
-    // pairs (c, c + d / 2): slices ds and ds + DS / 2 of this lane
+    // pairs (c, c + d / 2) (kMaps: of either map, (c, c + d / 4)): slices a and b of this lane
 #pragma unroll
-    for (int ds = 0; ds < DS / 2; ++ds) {
+    for (int i = 0; i < DS / 2; ++i) {
+      const int ds = i % kPairs, a = i / kPairs * 2 * kPairs + ds, b = a + kPairs;
       const float4 c_lo = cs[ds][0], c_hi = cs[ds][1], s_lo = sn[ds][0], s_hi = sn[ds][1];
-      const Pair8 rq = rotate8(__builtin_bit_cast(uint4, qf[ds]), __builtin_bit_cast(uint4, qf[ds + DS / 2]), c_lo, c_hi, s_lo, s_hi);
-      qf[ds] = __builtin_bit_cast(bf16x8, rq.lo);
-      qf[ds + DS / 2] = __builtin_bit_cast(bf16x8, rq.hi);
-      const Pair8 rk = rotate8(new_k[ds], new_k[ds + DS / 2], c_lo, c_hi, s_lo, s_hi);
-      new_k[ds] = rk.lo;
-      new_k[ds + DS / 2] = rk.hi;
+      const Pair8 rq = rotate8(__builtin_bit_cast(uint4, qf[a]), __builtin_bit_cast(uint4, qf[b]), c_lo, c_hi, s_lo, s_hi);
+      qf[a] = __builtin_bit_cast(bf16x8, rq.lo);
+      qf[b] = __builtin_bit_cast(bf16x8, rq.hi);
+      const Pair8 rk = rotate8(new_k[a], new_k[b], c_lo, c_hi, s_lo, s_hi);
+      new_k[a] = rk.lo;
+      new_k[b] = rk.hi;
     }
     // the wave that owns the last tile of keys (in the first chunk of heads) writes the token's cache slot
     if (h0 == 0 && tile_begin <= last && last < tile_end) {
       const int64_t blk = new_slot >> bs_shift, off = new_slot & bs_mask;
       if (c16 == 0) {
 #pragma unroll
-        for (int ds = 0; ds < DS; ++ds)
-          *reinterpret_cast<uint4*>(k_cache + ((((blk * kv_heads + hk) << bs_shift) + off) * d) + ds * 32 + g * 8) = new_k[ds];
+        for (int ds = 0; ds < DS; ++ds) {
+          const int c = ds * 32 + g * 8, m = kMaps && c >= d / 2;
+          if constexpr (kMaps) *reinterpret_cast<uint4*>(k_cache + ((((blk * 2 * kv_heads + 2 * hk + m) << bs_shift) + off) * (d / 2)) + c - m * (d / 2)) = new_k[ds];
+          else *reinterpret_cast<uint4*>(k_cache + ((((blk * kv_heads + hk) << bs_shift) + off) * d) + c) = new_k[ds];
+        }
       }
       if (g == 0) {
 #pragma unroll
@@ -692,7 +697,7 @@ extern "C" int alofa_attention_decode_v(void* out, int64_t out_stride, float* pa
                                         int hand_over, int v_head, float* out32, int split, int value_heads, int64_t plane, const float* sink, int block_heads,
                                         int two_maps, int keep_first, float cap, float lambda, float gain, float eps, int d_true, hipStream_t stream) {
   ALOFA_REQUIRE(block_heads >= 1 && block_heads <= kHeadsPerBlock, "attention_decode: a block serves 1 to %d heads (%d)", kHeadsPerBlock, block_heads);
-  ALOFA_REQUIRE(!split || !cos_t, "attention_decode: split weights and the rotary variant do not go together");
+  ALOFA_REQUIRE(!split || !cos_t || two_maps, "attention_decode: split weights and the rotary variant go together in the form for two maps only");
   // value_heads > 0: all of them in one launch, value head c's results in out32 + c * plane; `tokens` then counts (token, value head) pairs
   // wherever it sizes scratch, workspace and grid
   ALOFA_REQUIRE(value_heads == 0 || (value_heads == kv_heads && out32 && v_head < 0 && !cos_t && plane > 0), "attention_decode: all %d value heads in one launch need float rows and no value head named", kv_heads);
@@ -717,20 +722,20 @@ extern "C" int alofa_attention_decode_v(void* out, int64_t out_stride, float* pa
   ALOFA_REQUIRE(reinterpret_cast<uintptr_t>(k_cache) % 16 == 0 && reinterpret_cast<uintptr_t>(v_cache) % 8 == 0, "attention_decode: caches must be 16-byte aligned");
   const MapsForm maps{keep_first, cap, lambda, gain, eps, d_true};
   if (two_maps) {      // heads counts both maps of every head; parts that a second kernel combines leave both maps' sums as they are in out32 ([tokens, heads * d])
-    ALOFA_REQUIRE(split && !cos_t && !sink && v_head < 0 && value_heads == 0 && heads % (2 * kv_heads) == 0 && block_heads % 2 == 0 && d_true > 0 && d_true <= d,
-                  "attention_decode: two maps take split weights, an even count of columns a block (%d) and a key head (%d of %d), and neither turn, sink nor other value heads", block_heads, heads, kv_heads);
+    ALOFA_REQUIRE(split && (!cos_t || d % 128 == 0) && !sink && v_head < 0 && value_heads == 0 && heads % (2 * kv_heads) == 0 && block_heads % 2 == 0 && d_true > 0 && d_true <= d,
+                  "attention_decode: two maps take split weights, an even count of columns a block (%d) and a key head (%d of %d), and neither sink nor other value heads (turned here: sizes in steps of 128)", block_heads, heads, kv_heads);
     ALOFA_REQUIRE(keep_first >= 0 && keep_first <= 64 * block_size && cap >= 0.f, "attention_decode: keep_first=%d (at most 64 pages) cap=%g", keep_first, cap);
     ALOFA_REQUIRE(n_splits == 1 || (hand_over && n_splits <= 8) || out32, "attention_decode: %d parts of two maps need room for both maps' sums", n_splits);
   }
   const bool fused = cos_t != nullptr;
-  ALOFA_REQUIRE(!fused || (sin_t && slots && d % 64 == 0 && q_stride >= static_cast<int64_t>(heads + 2 * kv_heads) * d),
+  ALOFA_REQUIRE(!fused || (sin_t && slots && d % 64 == 0 && q_stride >= static_cast<int64_t>((two_maps ? heads / 2 : heads) + 2 * kv_heads) * d),
                 "attention_decode: the rotary variant needs sin, slots, rows of queries, keys and values, and a head size in steps of 64 (d=%d)", d);
   ALOFA_REQUIRE(!fused || (reinterpret_cast<uintptr_t>(cos_t) % 16 == 0 && reinterpret_cast<uintptr_t>(sin_t) % 16 == 0), "attention_decode: cos and sin must be 16-byte aligned");
   const int group = heads / kv_heads;
   const RopeArgs rope{cos_t, sin_t, slots};
   dim3 grid(tokens, kv_heads * ((group + block_heads - 1) / block_heads), n_splits);
 #define ALOFA_DECODE(DT, NW, ROPE)                                                                                        \
-  if (two_maps && !ROPE) attention_decode_kernel<DT, NW, false, true, true><<<grid, 64 * NW, 0, stream>>>(                 \
+  if (two_maps) attention_decode_kernel<DT, NW, ROPE && DT % 8 == 0, true, true><<<grid, 64 * NW, 0, stream>>>(                 \
       static_cast<bf16_t*>(out), out_stride, partial, static_cast<const bf16_t*>(q), q_stride,                            \
       static_cast<bf16_t*>(k_cache), static_cast<bf16_t*>(v_cache), block_table, max_blocks, req_of_token,                \
       positions, rows, heads, kv_heads, bs_shift, window, scale, rope, counters, v_head, out32, value_heads, plane, sink, block_heads, maps); \

@@ -109,26 +109,25 @@ __global__ void __launch_bounds__(256) route_top_kernel(const float* __restrict_
 // first when `renorm`). Outputs: chosen, weights [T, top] in order of falling c; dense [T, E - pass] the weights at the taken
 // experts with matrices, 0 elsewhere; pass_weight [T] the sum of the weights of taken experts without.
 // A wavefront per token; lane l holds the experts l, l + 64, ...
-template <typename Acc>
+// kOwn: experts a lane holds (experts up to 64 * kOwn). With one group there is nothing to compare before the picks.
+template <typename Acc, int kOwn>
 __global__ void __launch_bounds__(256) route_groups_kernel(const float* __restrict__ z, const float* __restrict__ correction, float* __restrict__ dense,
                                                            int32_t* __restrict__ chosen, float* __restrict__ weights, float* __restrict__ pass_weight,
                                                            int tokens, int experts, int pass, int top, int groups, int keep, float scale, int renorm) {
-  constexpr int kOwn = kMaxExperts / kWave;
-  __shared__ float group_best[4][kMaxExperts], all_scores[4][kMaxExperts];
+  __shared__ float group_best[4][kOwn * kWave], all_scores[4][kOwn * kWave];
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const int t = blockIdx.x * 4 + wave;
   if (t >= tokens) return;      // (no block-wide barrier below: a wavefront is on its own)
   const float* row = z + static_cast<int64_t>(t) * experts;
   const int real = experts - pass, size = experts / groups;
-  float* d = dense + static_cast<int64_t>(t) * real;
-  float zs[kOwn];
+  float zs[kOwn], extra[kOwn];
   float top_z = -3.402823466e+38f;
 #pragma unroll
   for (int i = 0; i < kOwn; ++i) {
     const int e = lane + i * kWave;
     zs[i] = e < experts ? row[e] : -3.402823466e+38f;
+    extra[i] = (correction && e < experts) ? correction[e] : 0.f;
     top_z = fmaxf(top_z, zs[i]);
-    if (e < real) d[e] = 0.f;
   }
   top_z = wave_max(top_z);
   Acc ex[kOwn], sum = 0;
@@ -140,43 +139,53 @@ __global__ void __launch_bounds__(256) route_groups_kernel(const float* __restri
   }
   sum = wave_sum(sum);
   float s[kOwn], c[kOwn];
-  bool taken[kOwn];
-  float* best = group_best[wave];
-  float* all = all_scores[wave];
+  bool out_of_it[kOwn], taken[kOwn];
 #pragma unroll
   for (int i = 0; i < kOwn; ++i) {
     const int e = lane + i * kWave;
     s[i] = static_cast<float>(ex[i] / sum);
-    c[i] = e < experts ? static_cast<float>(static_cast<Acc>(s[i]) + static_cast<Acc>(correction ? correction[e] : 0.f)) : 0.f;
-    if (e < experts) all[e] = c[i];
+    c[i] = e < experts ? static_cast<float>(static_cast<Acc>(s[i]) + static_cast<Acc>(extra[i])) : 0.f;
+    out_of_it[i] = e >= experts;
+    taken[i] = false;
   }
-  wave_lds_sync();
-  for (int g = lane; g < groups; g += kWave) {      // a group's score: the largest of its members' (a lane a group)
-    float m = all[g * size];
-    for (int o = 1; o < size; ++o) m = fmaxf(m, all[g * size + o]);
-    best[g] = m;
-  }
-  wave_lds_sync();
+  if (groups > 1) {      // (uniform)
+    float* best = group_best[wave];
+    float* all = all_scores[wave];
 #pragma unroll
-  for (int i = 0; i < kOwn; ++i) {
-    const int e = lane + i * kWave;
-    taken[i] = true;
-    if (e < experts) {
-      const int g = e / size;
-      const float mine = best[g];
-      int ahead = 0;      // groups that come before this one: a larger best, or an equal one with a lower index
-      for (int o = 0; o < groups; ++o) ahead += (best[o] > mine || (best[o] == mine && o < g)) ? 1 : 0;
-      taken[i] = ahead >= keep;      // (out of the choice from the start)
+    for (int i = 0; i < kOwn; ++i)
+      if (lane + i * kWave < experts) all[lane + i * kWave] = c[i];
+    wave_lds_sync();
+    for (int g = lane; g < groups; g += kWave) {      // a group's score: the largest of its members' (a lane a group)
+      float m = all[g * size];
+      for (int o = 1; o < size; ++o) m = fmaxf(m, all[g * size + o]);
+      best[g] = m;
+    }
+    wave_lds_sync();
+#pragma unroll
+    for (int i = 0; i < kOwn; ++i) {
+      const int e = lane + i * kWave;
+      if (e < experts) {
+        const int g = e / size;
+        const float mine = best[g];
+        int ahead = 0;      // groups that come before this one: a larger best, or an equal one with a lower index
+        for (int o = 0; o < groups; ++o) ahead += (best[o] > mine || (best[o] == mine && o < g)) ? 1 : 0;
+        out_of_it[i] = ahead >= keep;      // (out of the choice from the start)
+      }
     }
   }
-  Acc total = 0, passed = 0;
+  // pick k stays with lane k % 64 (its place k / 64) until the sum of all is known
+  Acc total = 0;
+  float score[kOwn];
+  int pick[kOwn];
+#pragma unroll
+  for (int i = 0; i < kOwn; ++i) score[i] = 0.f, pick[i] = -1;
   for (int k = 0; k < top; ++k) {
     float bc = 0.f, bs = 0.f;
     int be = 1 << 30;
 #pragma unroll
     for (int i = 0; i < kOwn; ++i) {
       const int e = lane + i * kWave;
-      if (!taken[i] && (be == 1 << 30 || c[i] > bc)) {
+      if (!out_of_it[i] && (be == 1 << 30 || c[i] > bc)) {
         bc = c[i];
         bs = s[i];
         be = e;
@@ -192,28 +201,33 @@ __global__ void __launch_bounds__(256) route_groups_kernel(const float* __restri
         be = oe;
       }
     }
-#pragma unroll
-    for (int i = 0; i < kOwn; ++i)
-      if (lane + i * kWave == be) taken[i] = true;
     total += static_cast<Acc>(bs);
-    if (lane == 0) {
-      chosen[static_cast<int64_t>(t) * top + k] = be == 1 << 30 ? -1 : be;
-      weights[static_cast<int64_t>(t) * top + k] = be == 1 << 30 ? 0.f : bs;      // (made final below)
+#pragma unroll
+    for (int i = 0; i < kOwn; ++i) {
+      if (lane + i * kWave == be) out_of_it[i] = taken[i] = true;
+      if (lane + i * kWave == k) score[i] = bs, pick[i] = be == 1 << 30 ? -1 : be;
     }
   }
-  wave_lds_sync();
-  if (lane == 0) {
-    for (int k = 0; k < top; ++k) {
-      const int e = chosen[static_cast<int64_t>(t) * top + k];
-      Acc w = static_cast<Acc>(weights[static_cast<int64_t>(t) * top + k]);
-      if (renorm) w /= total + static_cast<Acc>(1e-20f);      // (scores that are all next to nothing stay numbers)
-      const float f = static_cast<float>(w * static_cast<Acc>(scale));
-      weights[static_cast<int64_t>(t) * top + k] = f;
-      if (e >= 0 && e < real) d[e] = f;
-      else if (e >= real) passed += static_cast<Acc>(f);
+  auto final_weight = [&](float x) {
+    Acc w = static_cast<Acc>(x);
+    if (renorm) w /= total + static_cast<Acc>(1e-20f);      // (scores that are all next to nothing stay numbers)
+    return static_cast<float>(w * static_cast<Acc>(scale));
+  };
+  Acc passed = 0;
+  float* d = dense + static_cast<int64_t>(t) * real;
+#pragma unroll
+  for (int i = 0; i < kOwn; ++i) {
+    const int e = lane + i * kWave, k = e;
+    if (k < top) {
+      chosen[static_cast<int64_t>(t) * top + k] = pick[i];
+      weights[static_cast<int64_t>(t) * top + k] = final_weight(score[i]);
     }
-    if (pass_weight) pass_weight[t] = static_cast<float>(passed);
+    const float mine = taken[i] ? final_weight(s[i]) : 0.f;      // (an expert's weight is its own lane's to write)
+    if (e < real) d[e] = mine;
+    else passed += static_cast<Acc>(mine);
   }
+  passed = wave_sum(passed);
+  if (pass_weight && lane == 0) pass_weight[t] = static_cast<float>(passed);
 }
 
 // ---- gated activation of all experts side by side ------------------------------------------------
@@ -309,7 +323,10 @@ extern "C" int alofa_route_groups(const float* z, const float* correction, float
                 "route_groups: %d experts in %d groups of which %d are kept cannot give %d choices", experts, groups, keep, top);
   if (tokens == 0) return 0;
   const unsigned grid = static_cast<unsigned>((tokens + 3) / 4);
-  if (exact) route_groups_kernel<double><<<grid, 256, 0, stream>>>(z, correction, dense, chosen, weights, pass_weight, tokens, experts, pass, top, groups, keep, scale, renorm);
-  else route_groups_kernel<float><<<grid, 256, 0, stream>>>(z, correction, dense, chosen, weights, pass_weight, tokens, experts, pass, top, groups, keep, scale, renorm);
+#define ALOFA_GROUPS(ACC, OWN) route_groups_kernel<ACC, OWN><<<grid, 256, 0, stream>>>(z, correction, dense, chosen, weights, pass_weight, tokens, experts, pass, top, groups, keep, scale, renorm)
+  if (exact) ALOFA_GROUPS(double, kMaxExperts / kWave);
+  else if (experts <= kWave) ALOFA_GROUPS(float, 1);
+  else ALOFA_GROUPS(float, kMaxExperts / kWave);
+#undef ALOFA_GROUPS
   return check_launch("route_groups");
 }

@@ -6,6 +6,9 @@
 //                  weight (or as it is), to rows of the reader's type. `source` [T, h]: every x[t, s] is source[t] (the first step of a
 //                  pass: the copies are spread and read in one launch). The copies are stored only where asked for.
 //
+// Instead of y there may be the results of a mixture of experts slot by slot (grouped.hip): y[t] is then the sum over row t's slots, its place in the
+// shared expert's and, where experts hand the row on, weight * row, formed here in the order of `experts_sum`.
+//
 // A block per row; a thread takes kVec neighbouring channels of all copies at a time, kOwn such runs in registers with their loads on their
 // way together, so a row is read once, written once and normed from registers. Rows longer than the registers hold are walked in a loop and the
 // sum for the norm is formed again from the copies just stored (by the thread that stored them). Products and sums in Acc (double in
@@ -13,6 +16,15 @@
 #include "common.h"
 
 namespace alofa {
+
+struct SlotRows {
+  const float* y;                // [slots, h] (null: no slots)
+  const int32_t* slot_of;        // [T * top (+ T)]: the slot of row t's k-th choice (-1: none), then of row t's place in the shared expert
+  int top, shared, tokens;
+  const float* pass_weight;      // [T] or null
+  const bf16_t* pass_x;          // [T, h]
+  int64_t pass_stride;
+};
 
 struct StreamArgs {
   float* x;                // [T, S, h]
@@ -24,24 +36,26 @@ struct StreamArgs {
   const float* norm_w;     // [h] or null: no norm
   int streams, h, write;
   float eps;
+  SlotRows slots;
 };
 
-template <typename Acc, typename TO, int SM, int kVec, int kOwn>
-__global__ void __launch_bounds__(256) streams_step_kernel(TO* __restrict__ out, StreamArgs a) {
-  constexpr int kRun = 256 * kVec;
-  __shared__ Acc meet[4];
+template <typename Acc, typename TO, int SM, int kVec, int kOwn, int kThreads = 256>
+__global__ void __launch_bounds__(kThreads) streams_step_kernel(TO* __restrict__ out, StreamArgs a) {
+  constexpr int kRun = kThreads * kVec;
+  __shared__ Acc meet[kThreads / kWave];
   const int S = a.streams, h = a.h;
   const int64_t t = blockIdx.x;
   float* x = a.x + t * S * h;
   const float* source = a.source ? a.source + t * h : nullptr;
   const float* y = a.y ? a.y + t * h : nullptr;
+  const bool slots = a.slots.y != nullptr, adds = y != nullptr || slots;
   Acc m[SM][SM], wo[SM], wi[SM];      // (the same for every thread: scalar loads)
 #pragma unroll
   for (int s = 0; s < SM; ++s) {
-    wo[s] = (y && s < S) ? static_cast<Acc>(a.w_out[s]) : Acc(0);
+    wo[s] = (adds && s < S) ? static_cast<Acc>(a.w_out[s]) : Acc(0);
     wi[s] = (out && s < S) ? static_cast<Acc>(a.w_in[s]) : Acc(0);
 #pragma unroll
-    for (int v = 0; v < SM; ++v) m[s][v] = (y && s < S && v < S) ? static_cast<Acc>(a.mix[s * S + v]) : Acc(0);
+    for (int v = 0; v < SM; ++v) m[s][v] = (adds && s < S && v < S) ? static_cast<Acc>(a.mix[s * S + v]) : Acc(0);
   }
   auto load = [&](const float* p, float (&v)[kVec]) {
     if constexpr (kVec == 4) {
@@ -61,7 +75,7 @@ __global__ void __launch_bounds__(256) streams_step_kernel(TO* __restrict__ out,
       float now[kVec];
 #pragma unroll
       for (int e = 0; e < kVec; ++e) {
-        if (y) {
+        if (adds) {
           Acc n = 0;
 #pragma unroll
           for (int s = 0; s < SM; ++s) n += m[s][v] * static_cast<Acc>(old[s][e]);
@@ -86,27 +100,56 @@ __global__ void __launch_bounds__(256) streams_step_kernel(TO* __restrict__ out,
 #pragma unroll
         for (int e = 0; e < kVec; ++e) old[s][e] = 0.f;
     }
-    if (y) load(y + c, add);
-    else
+    if (y) {
+      load(y + c, add);
+      return;
+    }
 #pragma unroll
-      for (int e = 0; e < kVec; ++e) add[e] = 0.f;
+    for (int e = 0; e < kVec; ++e) add[e] = 0.f;
+    if (!slots) return;
+    const SlotRows& r = a.slots;
+    auto slot_at = [&](int k) { return k < r.top ? r.slot_of[t * r.top + k] : (r.shared && k == r.top ? r.slot_of[static_cast<int64_t>(r.tokens) * r.top + t] : -1); };
+    for (int k0 = 0; k0 < r.top + r.shared; k0 += 5) {      // (five slots' values on their way together)
+      float part[5][kVec];
+#pragma unroll
+      for (int u = 0; u < 5; ++u) {
+        const int slot = slot_at(k0 + u);
+        if (slot >= 0) load(r.y + static_cast<int64_t>(slot) * h + c, part[u]);
+        else
+#pragma unroll
+          for (int e = 0; e < kVec; ++e) part[u][e] = 0.f;
+      }
+#pragma unroll
+      for (int u = 0; u < 5; ++u)
+#pragma unroll
+        for (int e = 0; e < kVec; ++e) add[e] += part[u][e];
+    }
+    if (r.pass_weight) {
+      const float w = r.pass_weight[t];
+      const bf16_t* px = r.pass_x + t * r.pass_stride + c;
+#pragma unroll
+      for (int e = 0; e < kVec; ++e) add[e] += w * bf16_to_f32(px[e]);
+    }
   };
-  auto put = [&](int c, const Acc (&r)[kVec], Acc factor) {
+  auto put = [&](int c, const Acc (&r)[kVec], Acc factor, const float (&nw)[kVec]) {
     TO* dst = out + t * h + c;
     float v[kVec];
 #pragma unroll
-    for (int e = 0; e < kVec; ++e) v[e] = static_cast<float>(a.norm_w ? r[e] * factor * static_cast<Acc>(a.norm_w[c + e]) : r[e]);
+    for (int e = 0; e < kVec; ++e) v[e] = static_cast<float>(a.norm_w ? r[e] * factor * static_cast<Acc>(nw[e]) : r[e]);
     if constexpr (kVec == 4 && sizeof(TO) == 2) *reinterpret_cast<uint2*>(dst) = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
     else if constexpr (kVec == 4) *reinterpret_cast<float4*>(dst) = make_float4(v[0], v[1], v[2], v[3]);
     else store_f32(dst, v[0]);
   };
   const int c0 = threadIdx.x * kVec;
   if constexpr (kOwn > 0) {
-    float old[kOwn][SM][kVec], add[kOwn][kVec];
+    float old[kOwn][SM][kVec], add[kOwn][kVec], nw[kOwn][kVec];
     Acc read[kOwn][kVec], ss = 0;
 #pragma unroll
     for (int i = 0; i < kOwn; ++i)
-      if (c0 + i * kRun < h) fetch(c0 + i * kRun, old[i], add[i]);
+      if (c0 + i * kRun < h) {
+        if (a.norm_w) load(a.norm_w + c0 + i * kRun, nw[i]);      // (the norm's weights set out with the rest)
+        fetch(c0 + i * kRun, old[i], add[i]);
+      }
 #pragma unroll
     for (int i = 0; i < kOwn; ++i)
       if (c0 + i * kRun < h) {
@@ -116,10 +159,10 @@ __global__ void __launch_bounds__(256) streams_step_kernel(TO* __restrict__ out,
       }
     if (!out) return;
     Acc factor = 1;
-    if (a.norm_w) factor = static_cast<Acc>(1) / sqrt(block_sum<Acc, 256>(ss, meet) / static_cast<Acc>(h) + static_cast<Acc>(a.eps));
+    if (a.norm_w) factor = static_cast<Acc>(1) / sqrt(block_sum<Acc, kThreads>(ss, meet) / static_cast<Acc>(h) + static_cast<Acc>(a.eps));
 #pragma unroll
     for (int i = 0; i < kOwn; ++i)
-      if (c0 + i * kRun < h) put(c0 + i * kRun, read[i], factor);
+      if (c0 + i * kRun < h) put(c0 + i * kRun, read[i], factor, nw[i]);
   } else {
     Acc ss = 0;
     for (int c = c0; c < h; c += kRun) {
@@ -127,12 +170,12 @@ __global__ void __launch_bounds__(256) streams_step_kernel(TO* __restrict__ out,
       Acc read[kVec];
       fetch(c, old, add);
       step(c, old, add, read);
-      if (out && !a.norm_w) put(c, read, Acc(1));
+      if (out && !a.norm_w) put(c, read, Acc(1), add);
 #pragma unroll
       for (int e = 0; e < kVec; ++e) ss += read[e] * read[e];
     }
     if (!out || !a.norm_w) return;
-    const Acc factor = static_cast<Acc>(1) / sqrt(block_sum<Acc, 256>(ss, meet) / static_cast<Acc>(h) + static_cast<Acc>(a.eps));
+    const Acc factor = static_cast<Acc>(1) / sqrt(block_sum<Acc, kThreads>(ss, meet) / static_cast<Acc>(h) + static_cast<Acc>(a.eps));
     for (int c = c0; c < h; c += kRun) {      // (the copies as they are now: this thread stored these channels, or nothing changed)
       Acc read[kVec];
 #pragma unroll
@@ -145,22 +188,25 @@ __global__ void __launch_bounds__(256) streams_step_kernel(TO* __restrict__ out,
 #pragma unroll
           for (int e = 0; e < kVec; ++e) read[e] += wi[v] * static_cast<Acc>(now[e]);
         }
-      put(c, read, factor);
+      float nw[kVec];
+      load(a.norm_w + c, nw);
+      put(c, read, factor, nw);
     }
   }
 }
 
 template <typename Acc, typename TO, int SM>
 static void launch_streams(void* out, const StreamArgs& a, int tokens, hipStream_t stream) {
-#define ALOFA_STREAMS(VEC, OWN) streams_step_kernel<Acc, TO, SM, VEC, OWN><<<tokens, 256, 0, stream>>>(static_cast<TO*>(out), a)
-  constexpr bool kMany = SM > 4 || sizeof(Acc) > 4;      // (many copies, or double: one run at a time fills the registers)
+#define ALOFA_STREAMS(VEC, OWN, THREADS) streams_step_kernel<Acc, TO, SM, VEC, OWN, THREADS><<<tokens, THREADS, 0, stream>>>(static_cast<TO*>(out), a)
+  // a run of four channels a thread where a block's threads cover the row; many copies, or double, fill the registers with one run of a small block
+  constexpr bool kMany = SM > 4 || sizeof(Acc) > 4;
   if (a.h % 4 != 0) {
-    if (a.h <= 256) ALOFA_STREAMS(1, 1);
-    else ALOFA_STREAMS(1, 0);
-  } else if (a.h <= 1024) ALOFA_STREAMS(4, 1);
-  else if (!kMany && a.h <= 2048) ALOFA_STREAMS(4, (kMany ? 1 : 2));
-  else if (!kMany && a.h <= 4096) ALOFA_STREAMS(4, (kMany ? 1 : 4));
-  else ALOFA_STREAMS(4, 0);
+    if (a.h <= 256) ALOFA_STREAMS(1, 1, 256);
+    else ALOFA_STREAMS(1, 0, 256);
+  } else if (a.h <= 1024) ALOFA_STREAMS(4, 1, 256);
+  else if (!kMany && a.h <= 2048) ALOFA_STREAMS(4, 1, (kMany ? 256 : 512));
+  else if (!kMany && a.h <= 4096) ALOFA_STREAMS(4, (kMany ? 1 : 2), (kMany ? 256 : 512));
+  else ALOFA_STREAMS(4, 0, 256);
 #undef ALOFA_STREAMS
 }
 
@@ -182,13 +228,16 @@ static void pick_streams(void* out, const StreamArgs& a, int tokens, hipStream_t
 using namespace alofa;
 
 extern "C" int alofa_streams_step(void* out, int o_dtype, float* x, const float* source, const float* y, const float* mix, const float* w_out, const float* w_in,
-                                  const float* norm_w, float eps, int tokens, int streams, int h, int write, int exact, hipStream_t stream) {
+                                  const float* norm_w, float eps, int tokens, int streams, int h, int write, const float* slots_y, const int32_t* slot_of, int top, int shared,
+                                  const float* pass_weight, const void* pass_x, int64_t pass_stride, int exact, hipStream_t stream) {
+  ALOFA_REQUIRE(slots_y == nullptr || (y == nullptr && slot_of && top > 0 && mix && w_out && !exact && (pass_weight == nullptr || pass_x)), "streams_step: slots come in y's place, with weights to add them by");
   ALOFA_REQUIRE(tokens >= 0 && h > 0 && streams >= 1 && streams <= 16, "streams_step: tokens=%d h=%d streams=%d (1 to 16)", tokens, h, streams);
   ALOFA_REQUIRE(x != nullptr && (y == nullptr || (mix && w_out)) && (out == nullptr || w_in), "streams_step: operands are missing");
-  ALOFA_REQUIRE(write || y == nullptr || norm_w == nullptr || out == nullptr || h <= 1024, "streams_step: a norm of long rows that are not stored");
+  ALOFA_REQUIRE(write || (y == nullptr && slots_y == nullptr) || norm_w == nullptr || out == nullptr || h <= 1024, "streams_step: a norm of long rows that are not stored");
   ALOFA_REQUIRE(!exact || out == nullptr || o_dtype == kF32, "streams_step: the exact path is float32");
   if (tokens == 0) return 0;
-  const StreamArgs a{x, source, y, mix, w_out, w_in, norm_w, streams, h, write, eps};
+  const StreamArgs a{x, source, y, mix, w_out, w_in, norm_w, streams, h, write, eps,
+                     SlotRows{slots_y, slot_of, top, shared, tokens, pass_weight, static_cast<const bf16_t*>(pass_x), pass_stride}};
   if (exact) pick_streams<double, float>(out, a, tokens, stream);
   else if (o_dtype == kF32) pick_streams<float, float>(out, a, tokens, stream);
   else pick_streams<float, bf16_t>(out, a, tokens, stream);

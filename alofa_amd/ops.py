@@ -2190,13 +2190,28 @@ MAX_STREAMS = 16
 
 def streams_step(x: torch.Tensor, source: Optional[torch.Tensor] = None, y: Optional[torch.Tensor] = None, mix: Optional[torch.Tensor] = None,
                  w_out: Optional[torch.Tensor] = None, w_in: Optional[torch.Tensor] = None, norm: Optional[tuple] = None, out: Optional[torch.Tensor] = None,
-                 write: bool = True, exact: bool = False) -> None:
+                 write: bool = True, exact: bool = False, slots: Optional[tuple] = None) -> None:
     """Copies of the stream, x [T, S, h] float32. With ``y`` [T, h] float32, ``mix`` [S, S] (from, to) and ``w_out`` [S]:
     x[t, v] becomes sum_s mix[s, v] x[t, s] + w_out[v] y[t], all copies from the old ones. With ``out`` [T, h] and ``w_in`` [S]: out[t] = sum_v w_in[v] x[t, v] of
     the new copies, through an RMSNorm where ``norm`` = (weight, eps) is given. ``source`` [T, h] float32: every copy is source[t] at the start.
-    ``write`` False: the new copies are not stored (nobody reads them again)."""
+    ``write`` False: the new copies are not stored (nobody reads them again). ``slots`` = (y [slots, h] float32, ``ExpertRows``, None or (weight [T], rows [T, h]
+    bfloat16)) in ``y``'s place: a mixture's results slot by slot, which ``experts_sum`` would add up."""
     _gpu("x", x, torch.float32, 3), _contig("x", x)
     T, S, h = x.shape
+    more = (_ptr(None), _ptr(None), _I(0), _I(0), _ptr(None), _ptr(None), _L(0))
+    if slots is not None:
+        ys, rows, passed = slots
+        _gpu("y", ys, torch.float32, 2), _contig("y", ys)
+        if y is not None or exact or rows.T != T or tuple(ys.shape) != (rows.slots, h):
+            raise AlofaError("shape_mismatch", "the slots' results do not fit the copies of the stream", f"y={tuple(ys.shape)} x={tuple(x.shape)} rows={rows.T}")
+        pw = px = None
+        if passed is not None:
+            pw, px = passed
+            _gpu("pass weight", pw, torch.float32, 1), _contig("pass weight", pw), _gpu("passed rows", px, torch.bfloat16, 2)
+            if pw.shape[0] != T or tuple(px.shape) != (T, h):
+                raise AlofaError("shape_mismatch", "one weight and one row to hand on per row of the stream", f"weight={tuple(pw.shape)} rows={tuple(px.shape)}")
+        more = (_ptr(ys), _ptr(rows.slot_of), _I(rows.top), _I(int(rows.shared)), _ptr(pw), _ptr(px), _L(_rows("passed rows", px) if px is not None else 0))
+    adds = y is not None or slots is not None
     if not 1 <= S <= MAX_STREAMS:
         raise AlofaError("unsupported", f"one to {MAX_STREAMS} copies of the stream", f"streams={S}")
     for n, t in (("source", source), ("y", y)):
@@ -2204,7 +2219,7 @@ def streams_step(x: torch.Tensor, source: Optional[torch.Tensor] = None, y: Opti
             _gpu(n, t, torch.float32, 2), _contig(n, t)
             if tuple(t.shape) != (T, h):
                 raise AlofaError("shape_mismatch", "rows do not fit the copies of the stream", f"operand={n} shape={tuple(t.shape)} x={tuple(x.shape)}")
-    for n, t, shape, needed in (("mix", mix, (S, S), y is not None), ("w_out", w_out, (S,), y is not None), ("w_in", w_in, (S,), out is not None)):
+    for n, t, shape, needed in (("mix", mix, (S, S), adds), ("w_out", w_out, (S,), adds), ("w_in", w_in, (S,), out is not None)):
         if needed:
             _gpu(n, t, torch.float32), _contig(n, t)
             if tuple(t.shape) != shape:
@@ -2218,9 +2233,9 @@ def streams_step(x: torch.Tensor, source: Optional[torch.Tensor] = None, y: Opti
             _gpu("norm weight", weight, torch.float32, 1), _contig("norm weight", weight)
             if weight.shape[0] != h:
                 raise AlofaError("shape_mismatch", "norm width does not fit", f"weight={tuple(weight.shape)} h={h}")
-    _call("alofa_streams_step", _ptr(out), _I(dtype_code(out) if out is not None else F32), _ptr(x), _ptr(source), _ptr(y), _ptr(mix if y is not None else None),
-          _ptr(w_out if y is not None else None), _ptr(w_in if out is not None else None), _ptr(weight if out is not None else None), _F(eps), _I(T), _I(S), _I(h),
-          _I(int(write)), _I(int(exact)), _stream())
+    _call("alofa_streams_step", _ptr(out), _I(dtype_code(out) if out is not None else F32), _ptr(x), _ptr(source), _ptr(y), _ptr(mix if adds else None),
+          _ptr(w_out if adds else None), _ptr(w_in if out is not None else None), _ptr(weight if out is not None else None), _F(eps), _I(T), _I(S), _I(h),
+          _I(int(write)), *more, _I(int(exact)), _stream())
 
 
 # ------------------------------------------------------------- two maps per head over the same values
@@ -2291,6 +2306,11 @@ def maps_prefill(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_ca
           *end.arguments(), _stream())
 
 
+def can_turn_in_maps_decode(d: int) -> bool:
+    """Head sizes for which ``maps_decode`` can turn and write the new token itself."""
+    return d in MAPS_HEAD_DIMS and d % 128 == 0
+
+
 def maps_decode_plan(tokens: int, heads: int, kv_heads: int, d: int, max_context: int, window: Optional[int], keep_first: int) -> tuple:
     """(parts, whether the last block combines them, floats of scratch) of ``maps_decode`` for these sizes."""
     n = decode_splits(tokens, 2 * heads, kv_heads, d, min(max_context, window + keep_first if window else max_context))
@@ -2301,11 +2321,14 @@ def maps_decode_plan(tokens: int, heads: int, kv_heads: int, d: int, max_context
 
 def maps_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor, req_of_token: Optional[torch.Tensor],
                 positions: torch.Tensor, heads: int, kv_heads: int, d: int, window: Optional[int], keep_first: int, scale: float, softcap: Optional[float], end: HeadEnd,
-                max_context: int, scratch: Optional[torch.Tensor] = None, sums: Optional[torch.Tensor] = None, rows: Optional[torch.Tensor] = None, plan: Optional[tuple] = None) -> None:
+                max_context: int, scratch: Optional[torch.Tensor] = None, sums: Optional[torch.Tensor] = None, rows: Optional[torch.Tensor] = None, plan: Optional[tuple] = None,
+                rope: Optional[tuple] = None) -> None:
     """The same for tokens of requests that bring few tokens: all of the batch, or the tokens ``rows``; all heads of a key head with both their maps
     share the keys and values a block reads. ``req_of_token`` None: token i is the one token of request i. ``scratch`` and ``sums`` (float32 [T, 2 heads * d]): needed
     where ``maps_decode_plan`` asks for floats of scratch (a second kernel then combines the parts and ``combine_maps`` ends the heads). ``plan``: that
-    function's answer, if another is wanted."""
+    function's answer, if another is wanted. With ``rope`` = (cos, sin, slots) the rows of ``q`` are the projection's [queries | keys | values] of one new token per request, not
+    yet turned: the kernel turns queries and the new key itself, uses the new key and value from registers and writes them to the token's cache slot
+    (``can_turn_in_maps_decode``)."""
     T, bs = _maps_operands(out, q, k_cache, v_cache, block_table, heads, kv_heads, d, window, keep_first, softcap, end)
     _gpu("positions", positions, torch.int32, 1), _contig("positions", positions)
     if req_of_token is not None:
@@ -2318,6 +2341,14 @@ def maps_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cac
     if rows is not None:
         _gpu("rows", rows, torch.int32, 1), _contig("rows", rows)
         n_tok = rows.shape[0]
+    cos = sin = slots = None
+    if rope is not None:
+        cos, sin, slots = rope
+        if not can_turn_in_maps_decode(d) or q.shape[1] < (heads + 2 * kv_heads) * d or rows is not None:
+            raise AlofaError("unsupported", "turned on the way: head sizes in steps of 128, rows of queries, keys and values, and all of them", f"d={d} q={tuple(q.shape)}")
+        _gpu("cos", cos, torch.float32, 2), _gpu("sin", sin, torch.float32, 2), _contig("cos", cos), _contig("sin", sin), _gpu("slots", slots, torch.int64, 1), _contig("slots", slots)
+        if cos.shape != sin.shape or cos.shape[1] != d // 4 or slots.shape[0] != T:
+            raise AlofaError("shape_mismatch", "the table of angles or the slots do not fit", f"cos={tuple(cos.shape)} d={d} slots={tuple(slots.shape)}")
     n_splits, hand_over, floats = plan or maps_decode_plan(n_tok, heads, kv_heads, d, max_context, window, keep_first)
     if floats:
         _gpu("scratch", scratch, torch.float32), _contig("scratch", scratch), _gpu("sums", sums, torch.float32, 2), _contig("sums", sums)
@@ -2327,7 +2358,7 @@ def maps_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cac
     stride = 2 * heads * d if floats else _rows("out", out)
     _call("alofa_attention_decode_v", _ptr(None if floats else out), _L(stride), _ptr(scratch if floats else None), _ptr(q), _L(_rows("q", q)),
           _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _I(block_table.shape[1]), _ptr(req_of_token), _ptr(positions), _ptr(rows),
-          _I(n_tok), _I(2 * heads), _I(kv_heads), _I(d), _I(bs), _I(int(window or 0)), _F(scale), _I(n_splits), _ptr(None), _ptr(None), _ptr(None), _I(int(hand_over)), _I(-1),
+          _I(n_tok), _I(2 * heads), _I(kv_heads), _I(d), _I(bs), _I(int(window or 0)), _F(scale), _I(n_splits), _ptr(cos), _ptr(sin), _ptr(slots), _I(int(hand_over)), _I(-1),
           _ptr(sums if floats else None), _I(1), _I(0), _L(0), _ptr(None), _I(decode_block_heads(n_tok, 2 * heads, kv_heads, d)),
           _I(1), _I(int(keep_first)), _F(softcap or 0.0), *end.arguments(), _I(end.true_d), _stream())
     if floats:

@@ -8,12 +8,14 @@ loaded) a head gives (a1 - lambda a2) over its root mean square over its channel
 
 The pages hold a key as two key heads of one half each, [2 kv_heads, slot, d / 2], and values transposed; d is the size both halves of a key and a value
 are widened to with zeros. Keys of the first ``keep_first`` tokens stay in their pages for good, the others go as the window passes. In bfloat16, with sizes
-the matrix-core kernels are built for, portions of prompts and single tokens take one launch each from turned queries to the heads' ends; every other case
+the matrix-core kernels are built for, portions of prompts and single tokens take one launch each from turned queries to the heads' ends (single tokens of
+heads in steps of 128 channels: from the projection on); every other case
 runs the always-valid window kernel on both maps and the kernel that ends the heads. Softmax weights are 32-bit numbers: on the matrix cores each meets
 the values as two bfloat16 numbers."""
 from __future__ import annotations
 
 import math
+import os
 
 import torch
 
@@ -24,6 +26,8 @@ from .attention import RowPlan, _padded_heads
 from .base import SLOT, CacheNeed, CacheTensor, Mixer, build_part, part_class, register_part
 
 NAMES = {"q": "q", "k": "k", "v": "v", "o": "o", "q_bias": "q.b", "k_bias": "k.b", "v_bias": "v.b", "lq1": "lq1", "lk1": "lk1", "lq2": "lq2", "lk2": "lk2"}
+
+TURN_IN_DECODE = os.environ.get("ALOFA_TURN_IN_DECODE", "1") != "0"      # 0 (for measurements): a launch of its own turns and writes single tokens too
 
 
 class DifferentialAttention(Mixer):
@@ -109,27 +113,32 @@ class DifferentialAttention(Mixer):
         proj = ctx.scratch("maps_proj", (T, self.w_in.shape[0]), self.rt.dtype)
         ops.gemm(proj, x, self.w_in, self.b_in, exact=exact)
         table, qkv = self.position.table(ctx.n_positions), proj[:, :self.width]
-        if 2 * self.dm == D:
+        fast = not exact and ops.maps_attention_fast(D, self.dm, kv.k.shape[2], self.keep_first, self.rt.dtype)
+        plan = ctx.memo("gqa_attention.rows", lambda: RowPlan(ctx)) if fast else None
+        # one new token per request: the decode kernel turns it and writes its cache slot itself
+        turns = fast and TURN_IN_DECODE and ctx.max_q_len == 1 and plan.long_runs is None and ops.can_turn_in_maps_decode(D)
+        if turns:
+            pass
+        elif 2 * self.dm == D:
             ops.rope_kv_write(qkv, *table, ctx.positions, 2 * H, 2 * G, self.dm, kv.slots, kv.k, kv.v)
         else:
             ops.norm_turn_write(qkv, ctx.positions, table, 2 * H, 2 * G, self.dm, D // 2, ops.NORM_NONE, None, None, 0.0, exact, kv.slots, kv.k, kv.v)
         attn = ctx.scratch("maps_out", (T, H * D), self.rt.dtype)
-        self._attend(ctx, proj[:, :2 * H * self.dm], kv, attn)
+        self._attend(ctx, qkv if turns else proj[:, :2 * H * self.dm], kv, attn, plan, (*table, kv.slots) if turns else None)
         if out is not None:
             ops.gemm(out, attn, self.w_o, exact=exact)
         else:
             ops.gemm(residual, attn, self.w_o, add_to_out=True, exact=exact)
 
-    def _attend(self, ctx, q, kv, attn) -> None:
+    def _attend(self, ctx, q, kv, attn, plan, rope) -> None:
         T, H, G, D = q.shape[0], self.heads, self.kv_heads, self.d
-        if self.rt.exact or not ops.maps_attention_fast(D, self.dm, kv.k.shape[2], self.keep_first, self.rt.dtype):
+        if plan is None:
             # the exact path, and page or head sizes the bfloat16 kernels are not built for
             sums = ctx.scratch("maps_sums", (T, 2 * H * D), torch.float32)
             ops.span_attention(sums, q, kv.k, kv.v, kv.block_table, ctx.req_of_token, ctx.positions, 2 * H, 2 * G, self.dm, D, self.window, self.scale, self.rt.exact,
                                keep_first=self.keep_first, softcap=self.softcap, maps=2)
             ops.combine_maps(attn, sums, H, D, self.end, self.rt.exact)
             return
-        plan = ctx.memo("gqa_attention.rows", lambda: RowPlan(ctx))
         common = (H, G, D, self.window, self.keep_first, self.scale, self.softcap, self.end)
         if plan.long_runs is not None:      # portions of prompts
             tiles = ctx.memo("runs of 64 rows", lambda: torch.tensor(plan.long_runs, dtype=torch.int32, device=ctx.device))
@@ -141,7 +150,7 @@ class DifferentialAttention(Mixer):
             # (one token per request and nothing else in the step: token i is request i)
             one_each = ctx.max_q_len == 1 and plan.short_rows is None and plan.long_runs is None
             ops.maps_decode(attn, q, kv.k, kv.v, kv.block_table, None if one_each else ctx.req_of_token, ctx.positions, *common, ctx.max_context, scratch, sums,
-                            plan.short_rows, parts)
+                            plan.short_rows, parts, rope)
 
 
 register_part("mixer", "differential_attention", DifferentialAttention)

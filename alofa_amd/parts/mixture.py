@@ -145,7 +145,12 @@ class RoutedExperts(FeedForward):
         return (SPARSE_EXPERTS and not self.rt.exact and 2 * self.top <= self.experts
                 and ops.can_group_experts(x, self.w_up, self.ff, self.shared_ff))
 
-    def forward(self, ctx, x, residual, scale=None, out=None, post=None):
+    def forward_slots(self, ctx, x, out):
+        """The mixture's results slot by slot, (y, ``ExpertRows``, None or (weight, rows)), for a reader that adds them up itself; where the experts do not run
+        slot by slot the result is stored in ``out`` and None returned."""
+        return self.forward(ctx, x, out, out=out, slots=True)
+
+    def forward(self, ctx, x, residual, scale=None, out=None, post=None, slots=False):
         T, exact = residual.shape[0], self.rt.exact
         dense, chosen, weights, passed = self.route(ctx, x)
         if passed is not None and scale is not None:
@@ -163,6 +168,8 @@ class RoutedExperts(FeedForward):
                 ops.experts_gate_up(act, x, self.w_gate, self.w_up, rows, self.ff, self.shared_ff, self.limit, self.shared_limit, self.slope, self.offset)
             y = ctx.scratch("experts_out", (rows.slots, self.hidden), torch.float32)
             ops.experts_down(y, act, self.w_down, rows, self.ff, self.shared_ff)
+            if slots:
+                return y, rows, None if passed is None else (passed, x)
             if post is not None:
                 ops.experts_sum_norm(residual, y, rows, *post, scratch=ctx.scratch)
                 return

@@ -75,9 +75,9 @@ class HyperConnectedBlock(Block):
     def can_leave(self, norm):
         return isinstance(norm, StreamRead)
 
-    def _write(self, x, y, sub, read=None, rows=None):
-        """The sub-layer's result into the copies; ``rows`` afterwards holds what ``read`` sees of them."""
-        ops.streams_step(x, y=y, mix=self.mix[sub], w_out=self.w_out[sub], w_in=read.weights if read else None, norm=read.norm if read else None, out=rows,
+    def _write(self, x, y, sub, read=None, rows=None, slots=None):
+        """The sub-layer's result (``y``, or a mixture's ``slots``) into the copies; ``rows`` afterwards holds what ``read`` sees of them."""
+        ops.streams_step(x, y=None if slots is not None else y, slots=slots, mix=self.mix[sub], w_out=self.w_out[sub], w_in=read.weights if read else None, norm=read.norm if read else None, out=rows,
                          write=read is None or not read.last, exact=self.rt.exact)
 
     def forward(self, ctx, entry, x, normed=None, then=None):
@@ -88,11 +88,15 @@ class HyperConnectedBlock(Block):
         if normed is None:
             ops.streams_step(x, w_in=self.w_in[0], norm=self.reads[0].norm, out=buf, write=False, exact=self.rt.exact)
             normed = buf
+        slots = None
         self.mixer.forward(ctx, (entry, 0), normed, apart, out=apart)
         if self.feed_forward is not None:
             self._write(x, apart, 0, self.reads[1], buf)
-            self.feed_forward.forward(ctx, buf, apart, out=apart)
-        self._write(x, apart, len(self.mix) - 1, *(then or ()))
+            if hasattr(self.feed_forward, "forward_slots"):      # (the launch that mixes the result in adds the experts' results up)
+                slots = self.feed_forward.forward_slots(ctx, buf, apart)
+            else:
+                self.feed_forward.forward(ctx, buf, apart, out=apart)
+        self._write(x, apart, len(self.mix) - 1, *(then or (None, None)), slots=slots)
         return then is not None
 
 

@@ -69,6 +69,35 @@ def test_streams(S, h, dtype, exact):
     near(out, pl.rms_norm(source * wi.sum(), w, eps), dtype, "read from the source", 2.0)
 
 
+@pytest.mark.parametrize("out_dtype", [F32, BF])
+@pytest.mark.parametrize("S, h, top, shared, passing", [(4, 2048, 4, True, 2), (2, 96, 3, False, 0), (3, 1030, 7, True, 1), (1, 4100, 5, True, 3), (8, 320, 1, False, 1), (2, 3000, 11, True, 2)])
+def test_streams_take_a_mixture_slot_by_slot(S, h, top, shared, passing, out_dtype):
+    from alofa_amd import ops
+    rng = np.random.default_rng(h)
+    T, experts, eps = 9, 12, 1e-5
+    chosen = np.stack([rng.permutation(experts + passing)[:top] for _ in range(T)])
+    rows = ops.ExpertRows(T, top, experts, shared, lambda name, shape, dtype: torch.zeros(shape, dtype=dtype, device=DEV))
+    ops.expert_rows(rows, dev(chosen, torch.int32), dev(rng.random((T, top))))
+    y, px, pw = f32(rng.normal(0, 1, (rows.slots, h))), b16(rng.normal(0, 1, (T, h))), f32(rng.random(T))
+    of = rows.slot_of.cpu().numpy()
+    want = np.zeros((T, h))
+    for t in range(T):
+        for k in range(top):
+            assert (of[t * top + k] < 0) == (chosen[t, k] >= experts)
+            if of[t * top + k] >= 0:
+                want[t] += y[of[t * top + k]]
+        if shared:
+            want[t] += y[of[T * top + t]]
+    if passing:
+        want += pw[:, None] * px
+    X, mix, wo, wi, w = f32(rng.normal(0, 2, (T, S, h))), f32(rng.normal(0, 0.7, (S, S))), f32(rng.normal(1, 0.5, S)), f32(rng.normal(0.5, 0.5, S)), f32(rng.normal(1, 0.2, h))
+    x, out = dev(X), torch.full((T, h), 7.0, dtype=out_dtype, device=DEV)
+    ops.streams_step(x, slots=(dev(y), rows, (dev(pw), dev(px, BF)) if passing else None), mix=dev(mix), w_out=dev(wo), w_in=dev(wi), norm=(dev(w), eps), out=out)
+    new = pl.write_streams(X, want, mix, wo)
+    near(x, new, F32, "copies")
+    near(out, pl.rms_norm(pl.read_streams(new, wi), w, eps), out_dtype, "normed")
+
+
 def test_streams_refuses_what_does_not_fit():
     from alofa_amd import ops
     from alofa_amd.errors import AlofaError
@@ -263,6 +292,38 @@ def test_two_maps_for_single_tokens(d, H, G, page, window, keep, cap, scale, pla
     got = back(run(rows))
     near(dev(got[rows]), want[rows], BF, "some rows", 1.5)
     assert (np.delete(got, rows, axis=0) == 9.0).all()
+
+
+@pytest.mark.parametrize("plan", [None, (1, False), (4, True), (6, False)])
+@pytest.mark.parametrize("d, H, G, page, window, keep, cap, scale", [z for z in SIZES if z[0] % 128 == 0] + [(128, 20, 1, 16, 17, 16, 50.0, 0.25), (128, 3, 3, 8, 1, 0, None, 0.3)])
+def test_single_tokens_turned_and_written_on_the_way(d, H, G, page, window, keep, cap, scale, plan):
+    """One new token per request, straight from the projection: as turned by the plain function, and written to its slot."""
+    from alofa_amd import ops
+    spans = [(n, 1) for n in (1, 2, 16, 17, 100, 163, 481, 64)]
+    r = Requests(spans, G, d // 2, d, page, window, keep, BF, d + 3)
+    rng = np.random.default_rng(7)
+    T, dims, base = r.T, d // 2, 300.0
+    q, k, v = (b16(rng.normal(0, 1, shape)) for shape in ((T, H, 2, d // 2), (T, G, 2, d // 2), (T, G, d)))
+    at = np.array([n - 1 for n, _ in spans])
+    turned_q, turned_k = (b16(pl.turn(x.reshape(T, -1, d // 2), at, {"base": base, "dims": dims})).reshape(x.shape) for x in (q, k))
+    table, slots = r.table.cpu().numpy(), []
+    for i, (n, _) in enumerate(spans):      # (the new token's slot holds nothing yet)
+        b, o = table[i, (n - 1) // page], (n - 1) % page
+        slots.append(b * page + o)
+        r.kc[b, :, o] = float("nan")
+        r.vc[b, :, :, o] = float("nan")
+        r.k[i][n - 1], r.v[i][n - 1] = turned_k[i], v[i]
+    angles = np.arange(512)[:, None].astype(np.float32) * pl.frequencies(dims, base).astype(np.float32)
+    rope = (dev(np.cos(angles.astype(np.float64))), dev(np.sin(angles.astype(np.float64))), dev(slots, torch.int64))
+    rows = dev(np.concatenate([q.reshape(T, -1), k.reshape(T, -1), v.reshape(T, -1)], axis=1), BF)
+    p = ops.maps_decode_plan(T, H, G, d, 512, window, keep) if plan is None else (*plan, T * 2 * H * plan[0] * (d + 2) if plan[0] > 1 and not plan[1] else 0)
+    scratch, sums = (torch.empty(p[2], device=DEV), torch.empty((T, 2 * H * d), device=DEV)) if p[2] else (None, None)
+    out = torch.full((T, H * d), 9.0, dtype=BF, device=DEV)
+    ops.maps_decode(out, rows, r.kc, r.vc, r.table, None, r.positions, H, G, d, window, keep, scale, cap, head_end(d), 512, scratch, sums, None, p, rope)
+    near(out, ends(r.sums(turned_q, H, window, keep, scale, cap), d).reshape(T, -1), BF, "turned here", 2.0)
+    for i, s in enumerate(slots):
+        near(r.kc[s // page, :, s % page], turned_k[i].reshape(2 * G, d // 2), BF, "the new key")
+        assert (back(r.vc.reshape(len(r.vc), G, d, page)[s // page, :, :, s % page]) == v[i]).all()
 
 
 def test_prompts_and_single_tokens_give_a_row_the_same():
