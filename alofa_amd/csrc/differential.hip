@@ -2,13 +2,13 @@
 // of its own, and what the head gives is a1 - lambda a2 over its root mean square, times a factor.
 //
 //   combine_maps          the always-valid end: both maps' sums as float rows, the difference, its norm, the factor.
-//   maps_prefill          portions of prompts in bfloat16 on the matrix cores: a wavefront owns 16 rows of one head with BOTH maps, so a tile of values
-//                         that is read from LDS meets four operands (two maps, each weight as two bfloat16 numbers), and the head's
+//   maps_prefill          portions of prompts in bfloat16 on the matrix cores: a wavefront owns 16 rows of one head, with both maps (a tile of values
+//                         that is read from LDS then meets four operands: two maps, each weight as two bfloat16 numbers) or with one, and the head's
 //                         end is made in registers: one launch from queries to the output product's rows.
 // (Single tokens go through the decode kernel of attention_decode.hip, in its form for two maps.)
 //
-// maps_prefill: a block serves, with TEAMS teams of four wavefronts, 64 consecutive rows of one request and one head. The visible keys are
-// walked in tiles of 64 (of 32 for heads of more than 128 channels) that start at absolute multiples of their size: first those that hold the sequence's kept first tokens, then the window's;
+// maps_prefill: a block serves, with TEAMS teams of four or eight wavefronts, 64 consecutive rows of one request and one head. The visible keys are
+// walked in tiles of 64 (heads of 256 channels: 32) that start at absolute multiples of their size: first those that hold the sequence's kept first tokens, then the window's;
 // the teams take the tiles in turn and their states meet in LDS at the end, in team order. Per tile a team stages
 // the keys [tile, d] (a key's two halves side by side) and the values transposed [d, tile].
 // Both products are taken transposed (v_mfma_f32_16x16x32_bf16; lane l: A row and B column l % 16, reduction slots 8 (l / 16) .. + 7, D column
@@ -69,20 +69,24 @@ struct MapsArgs {
   float scale, cap, lambda, gain, eps;
 };
 
+// NM: maps a wavefront owns. 2: both, four wavefronts a team. 1: one, eight wavefronts a team; the second map's sums go through LDS at the end.
 // kCap: 0 scores as they are; 1 capped, with a running maximum; 2 capped so that no maximum is needed
-template <int DT, int TEAMS, int kTileKeys, int kCap>
-__global__ void __launch_bounds__(256 * TEAMS) maps_prefill_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache,
+template <int DT, int TEAMS, int kTileKeys, int NM, int kCap>
+__global__ void __launch_bounds__(512 / NM * TEAMS, (NM == 1 && DT <= 8) ? 4 : 1) maps_prefill_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache,
                                                                    const bf16_t* __restrict__ v_cache, MapsArgs a) {
   constexpr int d = DT * 16, dm = d / 2, DS = (dm + 31) / 32;
   constexpr int KQ = kTileKeys / 16, KH = kTileKeys / 32;      // quarters of 16 keys for the first product, halves of 32 for the second
   constexpr int KROW = d + kPad, VROW = kTileKeys + kPad;
   constexpr int kStageBytes = ((kTileKeys * KROW + d * VROW) * 2 + 15) / 16 * 16;
   constexpr int kStateFloats = 2 * 4 * DT + 4;      // per lane: two maxima, two sums, two maps' channels
-  constexpr int kStateBytes = (TEAMS - 1) * 256 * kStateFloats * 4;
+  constexpr int kTeam = 512 / NM;                   // threads of a team
+  static_assert(NM == 2 || TEAMS == 1, "one map a wavefront: one team");
+  constexpr int kStateBytes = NM == 2 ? (TEAMS - 1) * 256 * kStateFloats * 4 : 256 * (4 * DT + 1) * 4;
   constexpr int kRoom = TEAMS * kStageBytes > kStateBytes ? TEAMS * kStageBytes : kStateBytes;
   __shared__ __attribute__((aligned(16))) char room[kRoom];
   const int wave_of_block = __builtin_amdgcn_readfirstlane(threadIdx.x / 64);
-  const int team = wave_of_block / 4, wave = wave_of_block % 4, lane = threadIdx.x % 64, tid = wave * 64 + lane;
+  const int team = wave_of_block / (8 / NM), wave = wave_of_block % 4, lane = threadIdx.x % 64, tid = threadIdx.x % kTeam;
+  const int own = NM == 2 ? 0 : wave_of_block / 4;      // the (first) map of this wavefront
   bf16_t* Ks = reinterpret_cast<bf16_t*>(room + team * kStageBytes);
   bf16_t* Vt = Ks + kTileKeys * KROW;
   const int c16 = lane % 16, g = lane / 16;
@@ -93,22 +97,24 @@ __global__ void __launch_bounds__(256 * TEAMS) maps_prefill_kernel(bf16_t* __res
   const int W = a.window, my_row = wave * 16 + c16, my_pos = pos0 + my_row;
   const bool row_ok = my_row < n_rows;
 
-  bf16x8 qf[2][DS];
+  bf16x8 qf[NM][DS];
 #pragma unroll
-  for (int m = 0; m < 2; ++m)
+  for (int m = 0; m < NM; ++m)
 #pragma unroll
     for (int ds = 0; ds < DS; ++ds) {
       uint4 v = make_uint4(0, 0, 0, 0);
       const int c = ds * 32 + g * 8;
-      if (row_ok && c < dm) v = *reinterpret_cast<const uint4*>(q + static_cast<int64_t>(row0 + my_row) * a.q_stride + static_cast<int64_t>(2 * head + m) * dm + c);
+      if (row_ok && c < dm) v = *reinterpret_cast<const uint4*>(q + static_cast<int64_t>(row0 + my_row) * a.q_stride + static_cast<int64_t>(2 * head + own + m) * dm + c);
       qf[m][ds] = __builtin_bit_cast(bf16x8, v);
     }
-  f32x4 o[2][DT];
+  f32x4 o[NM][DT];
 #pragma unroll
-  for (int m = 0; m < 2; ++m)
+  for (int m = 0; m < NM; ++m)
 #pragma unroll
     for (int nt = 0; nt < DT; ++nt) o[m][nt] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float top[2] = {-FLT_MAX, -FLT_MAX}, l[2] = {0.f, 0.f};
+  float top[NM], l[NM];
+#pragma unroll
+  for (int m = 0; m < NM; ++m) top[m] = -FLT_MAX, l[m] = 0.f;
   const float scale2 = a.scale * kLog2e;                       // scores in units of log2 e
   const float inner = kCap ? 2.f * scale2 / a.cap : 0.f;       // exp(2 s / cap) = exp2(inner * product)
   const float cap2 = a.cap * kLog2e;
@@ -125,12 +131,12 @@ __global__ void __launch_bounds__(256 * TEAMS) maps_prefill_kernel(bf16_t* __res
   // Staging as in attention_prefill.hip: 16-byte chunks (eight channels of a key, eight keys of a channel); every lane issues every load, from a key
   // whose page is held in place of one that is not seen, and what such a load brings is cleared.
   constexpr int kChunks = kTileKeys * d / 8;
-  constexpr int kPerThread = (kChunks + 255) / 256;
+  constexpr int kPerThread = (kChunks + kTeam - 1) / kTeam;
   const int page_mask = (1 << a.bs_shift) - 1;
   const int v_first = first_key & ~7, v_last = last_pos & ~7;
   uint4 k_reg[kPerThread], v_reg[kPerThread];
   int k_page[kPerThread], v_page[kPerThread];
-  auto chunk_of = [&](int j) { const int c = tid + 256 * j; return c < kChunks ? c : kChunks - 1; };
+  auto chunk_of = [&](int j) { const int c = tid + kTeam * j; return c < kChunks ? c : kChunks - 1; };
   auto held = [&](int key, int lo, int hi) { return key < keep ? key : (key < lo ? lo : (key > hi ? hi : key)); };
   auto k_key = [&](int t, int j) { return t * kTileKeys + chunk_of(j) / (d / 8); };
   auto v_key0 = [&](int t, int j) { return t * kTileKeys + (chunk_of(j) % (kTileKeys / 8)) * 8; };
@@ -159,7 +165,7 @@ __global__ void __launch_bounds__(256 * TEAMS) maps_prefill_kernel(bf16_t* __res
     const bool whole = (t0 >= first_key || t0 + kTileKeys <= keep) && t0 + kTileKeys - 1 <= last_pos;      // uniform over the team
 #pragma unroll
     for (int j = 0; j < kPerThread; ++j) {
-      const int c = tid + 256 * j;
+      const int c = tid + kTeam * j;
       if (c >= kChunks) continue;
       uint4 kv = k_reg[j], vv = v_reg[j];
       if (!whole) {
@@ -199,10 +205,10 @@ __global__ void __launch_bounds__(256 * TEAMS) maps_prefill_kernel(bf16_t* __res
 
     // every row of the block sees every key of the tile: no masks
     const bool whole = t0 + kTileKeys - 1 <= pos0 && (W <= 0 || t0 > last_pos - W || t0 + kTileKeys <= keep);
-    bf16x8 pf[2][KH], pl[2][KH];
-    float corr[2];
+    bf16x8 pf[NM][KH], pl[NM][KH];
+    float corr[NM];
 #pragma unroll
-    for (int m = 0; m < 2; ++m) {
+    for (int m = 0; m < NM; ++m) {
       f32x4 s[KQ];
 #pragma unroll
       for (int kt = 0; kt < KQ; ++kt) {
@@ -211,9 +217,10 @@ __global__ void __launch_bounds__(256 * TEAMS) maps_prefill_kernel(bf16_t* __res
         for (int ds = 0; ds < DS; ++ds) {
           const int c = ds * 32 + g * 8;
           uint4 kv = make_uint4(0, 0, 0, 0);
-          if (c < dm) kv = *reinterpret_cast<const uint4*>(&Ks[(kt * 16 + c16) * KROW + m * dm + c]);
+          if (c < dm) kv = *reinterpret_cast<const uint4*>(&Ks[(kt * 16 + c16) * KROW + (own + m) * dm + c]);
           s[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, kv), qf[m][ds], s[kt], 0, 0, 0);
         }
+        if constexpr (DT > 8 || NM == 1) __builtin_amdgcn_sched_barrier(0);
       }
       float p[4 * KQ];
 #pragma unroll
@@ -265,26 +272,29 @@ __global__ void __launch_bounds__(256 * TEAMS) maps_prefill_kernel(bf16_t* __res
 #pragma unroll
     for (int nt = 0; nt < DT; ++nt) {
       if constexpr (kCap != 2) {
-        o[0][nt] *= corr[0];
-        o[1][nt] *= corr[1];
+#pragma unroll
+        for (int m = 0; m < NM; ++m) o[m][nt] *= corr[m];
       }
-      const bf16_t* vrow = &Vt[(nt * 16 + c16) * VROW];
-      const int sw = ((nt * 2 + (c16 >> 3)) & 7) << 2;   // this row's permutation of its four-key groups
+      // (row nt * 16 + c16 and its permutation of the four-key groups, which comes round every four tiles of channels: wide heads keep four addresses, not all)
+      constexpr int kRound = (DT > 8 || (NM == 1 && DT >= 4)) ? 4 : DT;
+      const bf16_t* vrow = Vt + (nt % kRound * 16 + c16) * VROW;
+      const int sw = ((nt % kRound * 2 + (c16 >> 3)) & 7) << 2, on = nt / kRound * kRound * 16 * VROW;
 #pragma unroll
       for (int half = 0; half < KH; ++half) {
-        const uint2 lo = *reinterpret_cast<const uint2*>(vrow + ((half * 32 + g * 4) ^ sw));
-        const uint2 hi = *reinterpret_cast<const uint2*>(vrow + ((half * 32 + 16 + g * 4) ^ sw));
+        const uint2 lo = *reinterpret_cast<const uint2*>(vrow + ((half * 32 + g * 4) ^ sw) + on);
+        const uint2 hi = *reinterpret_cast<const uint2*>(vrow + ((half * 32 + 16 + g * 4) ^ sw) + on);
         const bf16x8 vv = __builtin_bit_cast(bf16x8, make_uint4(lo.x, lo.y, hi.x, hi.y));
 #pragma unroll
-        for (int m = 0; m < 2; ++m) o[m][nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pf[m][half], o[m][nt], 0, 0, 0);
+        for (int m = 0; m < NM; ++m) o[m][nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pf[m][half], o[m][nt], 0, 0, 0);
 #pragma unroll
-        for (int m = 0; m < 2; ++m) o[m][nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pl[m][half], o[m][nt], 0, 0, 0);
+        for (int m = 0; m < NM; ++m) o[m][nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pl[m][half], o[m][nt], 0, 0, 0);
       }
+      if constexpr (DT > 8 || NM == 1) __builtin_amdgcn_sched_barrier(0);      // (operands read far ahead of their use would not fit the registers)
     }
   }
 
 #pragma unroll
-  for (int m = 0; m < 2; ++m) l[m] = rows_sum(l[m]);
+  for (int m = 0; m < NM; ++m) l[m] = rows_sum(l[m]);
   if constexpr (TEAMS > 1) {
     // the other teams leave their states where the tiles were; team 0 adds them in team order
     __syncthreads();      // every tile has been read
@@ -325,14 +335,29 @@ __global__ void __launch_bounds__(256 * TEAMS) maps_prefill_kernel(bf16_t* __res
       }
     }
   }
+  float l2 = l[NM - 1];
+  float* second = reinterpret_cast<float*>(room) + wave * 64 + lane;      // NM 1: [value][row group][lane], what the second map's wavefronts hand over
+  if constexpr (NM == 1) {
+    __syncthreads();      // every tile has been read
+    if (own == 1) {
+      second[0] = l[0];
+#pragma unroll
+      for (int nt = 0; nt < DT; ++nt)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) second[(1 + nt * 4 + e) * 256] = o[0][nt][e];
+    }
+    __syncthreads();
+    if (own == 1) return;
+    l2 = second[0];
+  }
   // the head's end: the difference, its root mean square over the row's channels (four lanes hold a row), the factor
-  const float i1 = 1.f / l[0], i2 = a.lambda / l[1];
+  const float i1 = 1.f / l[0], i2 = a.lambda / l2;
   float ss = 0.f;
 #pragma unroll
   for (int nt = 0; nt < DT; ++nt)
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      const float y = o[0][nt][e] * i1 - o[1][nt][e] * i2;
+      const float y = o[0][nt][e] * i1 - (NM == 2 ? o[NM - 1][nt][e] : second[(1 + nt * 4 + e) * 256]) * i2;
       o[0][nt][e] = y;
       ss += y * y;
     }
@@ -345,9 +370,9 @@ __global__ void __launch_bounds__(256 * TEAMS) maps_prefill_kernel(bf16_t* __res
     *reinterpret_cast<uint2*>(dst + nt * 16) = make_uint2(pack_bf16x2(o[0][nt][0] * f, o[0][nt][1] * f), pack_bf16x2(o[0][nt][2] * f, o[0][nt][3] * f));
 }
 
-template <int DT, int TEAMS, int KT = 64>
+template <int DT, int TEAMS, int KT = 64, int NM = 2>
 static void launch_maps(dim3 grid, hipStream_t stream, void* out, const void* q, const void* k_cache, const void* v_cache, const MapsArgs& a) {
-#define ALOFA_MAPS(CAP) maps_prefill_kernel<DT, TEAMS, KT, CAP><<<grid, 256 * TEAMS, 0, stream>>>(static_cast<bf16_t*>(out), static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_cache), static_cast<const bf16_t*>(v_cache), a)
+#define ALOFA_MAPS(CAP) maps_prefill_kernel<DT, TEAMS, KT, NM, CAP><<<grid, 512 / NM * TEAMS, 0, stream>>>(static_cast<bf16_t*>(out), static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_cache), static_cast<const bf16_t*>(v_cache), a)
   if (a.cap <= 0.f) ALOFA_MAPS(0);
   else if (a.cap * kLog2e > 80.f) ALOFA_MAPS(1);
   else ALOFA_MAPS(2);
@@ -389,15 +414,18 @@ extern "C" int alofa_maps_prefill(void* out, int64_t out_stride, const void* q, 
   while ((1 << shift) < block_size) ++shift;
   const MapsArgs a{out_stride, q_stride, table, max_blocks, tiles, heads, kv_heads, shift, window, keep_first, d_true, scale, cap, lambda, gain, eps};
   const dim3 grid(n_tiles, heads);
+  // Which form (2,048 rows of 2,048 channels, a window of 1,024, scores capped at 50, us a layer, and the other form's): one map a wavefront where that leaves room for four
+  // wavefronts a SIMD (size 32: 181 against 200, 48: 149 against 191, 64: 107 against 125) or where two maps do not fit the registers (192: 116 against 184, 256:
+  // 83 against 185); both maps at 96 and 128 channels (117 and 88 against 134 and 96), whose values are then read from LDS once for both.
   switch (d / 16) {
-    case 1: launch_maps<1, 4>(grid, stream, out, q, k_cache, v_cache, a); break;
-    case 2: launch_maps<2, 4>(grid, stream, out, q, k_cache, v_cache, a); break;
-    case 3: launch_maps<3, 2>(grid, stream, out, q, k_cache, v_cache, a); break;
-    case 4: launch_maps<4, 2>(grid, stream, out, q, k_cache, v_cache, a); break;
+    case 1: launch_maps<1, 1, 64, 1>(grid, stream, out, q, k_cache, v_cache, a); break;
+    case 2: launch_maps<2, 1, 64, 1>(grid, stream, out, q, k_cache, v_cache, a); break;
+    case 3: launch_maps<3, 1, 64, 1>(grid, stream, out, q, k_cache, v_cache, a); break;
+    case 4: launch_maps<4, 1, 64, 1>(grid, stream, out, q, k_cache, v_cache, a); break;
     case 6: launch_maps<6, 2>(grid, stream, out, q, k_cache, v_cache, a); break;
     case 8: launch_maps<8, 2>(grid, stream, out, q, k_cache, v_cache, a); break;
-    case 12: launch_maps<12, 1, 32>(grid, stream, out, q, k_cache, v_cache, a); break;
-    case 16: launch_maps<16, 1, 32>(grid, stream, out, q, k_cache, v_cache, a); break;
+    case 12: launch_maps<12, 1, 64, 1>(grid, stream, out, q, k_cache, v_cache, a); break;
+    case 16: launch_maps<16, 1, 32, 1>(grid, stream, out, q, k_cache, v_cache, a); break;
   }
   return check_launch("maps_prefill");
 }
